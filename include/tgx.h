@@ -27,10 +27,11 @@ extern "C" {
 
 /* 3 (round 5): per-row sequence lifecycle (tgx_reset_row / tgx_forward_row / tgx_sample_row / tgx_past_length_row); tgx_get_option added and
  * tgx_engine_read_stats + the options engine.*, pf.*, attn.fold_*, lmhead.fuse_finalize removed since 2. */
-#define TGX_ABI_VERSION 7   /* 4: layered models (tgx_create_stack, tgx_step_ragged); 5: Modepel (more mixers / feed-forward kinds in tgx_layer_desc);
+#define TGX_ABI_VERSION 8   /* 4: layered models (tgx_create_stack, tgx_step_ragged); 5: Modepel (more mixers / feed-forward kinds in tgx_layer_desc);
                              * 6: Vitudra (masks, score bias and cap, shared key / value layers, two recurrent mixers, parallel sublayers);
                              * 7: Zaluvik (layer norms around every sublayer, a looped span of layers, un-normalised sigmoid attention with mixed heads,
-                             *    windowed latent attention with a shared rotated key part, sigmoid group-limited router) */
+                             *    windowed latent attention with a shared rotated key part, sigmoid group-limited router);
+                             * 8: Nusovik (norms on the sublayers' outputs only, two state-space mixers, bucketed distance bias, per-head sink and gate) */
 
 #if defined(__GNUC__)
 #define TGX_API __attribute__((visibility("default")))
@@ -63,9 +64,11 @@ typedef enum tgx_family {
   TGX_FAMILY_MODEPEL = 7,  /* a layered model: rotary grouped-query attention and matrix-memory (mLSTM) layers, sandwich norms */
   TGX_FAMILY_VITUDRA = 8,  /* a layered model: one norm per layer in front of a mixer and a gated feed-forward that run side by side; windowed and chunked
                             * attention, shared key / value layers, decaying matrix states (token-shift "wkv" and gated delta rule) */
-  TGX_FAMILY_ZALUVIK = 9   /* a layered model: layer norms (weight and bias) before and after every sublayer, a span of layers run several times with the
+  TGX_FAMILY_ZALUVIK = 9,  /* a layered model: layer norms (weight and bias) before and after every sublayer, a span of layers run several times with the
                             * embedding output fed back in, windowed sigmoid attention whose weights are mixed across heads, windowed latent attention
                             * with a rotated key part all heads share, erf-gelu feed-forwards and sigmoid-routed experts; logits against the embedding table */
+  TGX_FAMILY_NUSOVIK = 10  /* a layered model: norms on the sublayers' outputs only; selective-scan layers and layers that run chunked attention (keys as values,
+                            * bucketed distance bias, sinks) beside a scalar-decay state-space mixer; squared-relu feed-forwards */
 } tgx_family;
 
 /* tinytorch::DType values the CLI accepts (examples/inference/main.cpp:82-88) */
@@ -154,8 +157,23 @@ typedef struct tgx_model_desc {
  *                             share; score = (q_plain . W_uk c + q_rot . k_rot) * scale; softmax without sink; mask_kind / mask_size as above
  *   erf-gelu feed-forward     ff_act 1: down(gelu(up h)), gelu(z) = z (1 + erf(z / sqrt 2)) / 2
  *   sigmoid router            router_fn 1: scores = sigmoid(W_r h) (32-bit), no correction; group_score 1: a group counts as the sum of its two largest
- *                             scores; router_norm 1: weights = chosen scores / (their sum + 1e-20); a shared expert (shared_ff) without a gate of its own */
-typedef enum tgx_mixer { TGX_MIXER_LATENT_ATTENTION = 1, TGX_MIXER_ATTENTION = 2, TGX_MIXER_MLSTM = 3, TGX_MIXER_WKV = 4, TGX_MIXER_PARALLEL = 5 } tgx_mixer;
+ *                             scores; router_norm 1: weights = chosen scores / (their sum + 1e-20); a shared expert (shared_ff) without a gate of its own
+ * and, for TGX_FAMILY_NUSOVIK (x <- x + norm1(mixer(x)), x <- x + norm2(ff(x)): the sublayers read the stream itself, norm(v) = v / sqrt(mean(v^2) +
+ * norm_eps) * w; embedding rows times embed_scale plus the sinusoidal positions above; slots hold pages of the attention halves' key / value pools, one
+ * state per state-space head or channel and the convolution tails):
+ *   keys as values            v_is_k 1: no value projection, a head's values are its key projections (bias included) before the key norm (vdim = dim)
+ *   weighted query / key norm qk_norm 2: every query and key head is divided by sqrt(mean(head^2) + norm_eps) and multiplied by a learned vector of `dim`
+ *   bucketed distance bias    bias_max D > 0: the scaled score gains rel[bucket(i - j)][head]; with B rows in the table and b = B / 2, bucket(n) = n below b,
+ *                             min(B - 1, b + floor(ln(n / b) / ln(D / b) * (B - b))) from b on; bias_buckets = B (0: from the tensor)
+ *   sink                      head_sink 1: a learned number per head whose exponential joins the softmax's denominator
+ *   output gate               gate_kind 2: per head
+ *   mamba1                    selective scan: causal depth-wise convolution of conv_taps taps (with bias) and silu on `inner` channels, step sizes softplus(W_dt . + b)
+ *                             through a product of inner size dt_rank, a state of d_dim numbers per channel, each with its own decay, silu gate
+ *   parallel mixer            right_kind 1: the right half is a scalar-decay state-space mixer (state-space duality): d_heads heads of d_vdim values over d_kv_heads groups
+ *                             of d_dim state numbers; convolution (with bias) and silu on x | B | C, dt = softplus(. + dt_bias), S <- exp(-exp(A_log) dt) S +
+ *                             dt B x^T, y = S^T C + D x, then y * silu(z) RMS-normed in part_norms equal parts
+ *   squared-relu feed-forward ff_act 2: down(max(up x, 0)^2) */
+typedef enum tgx_mixer { TGX_MIXER_LATENT_ATTENTION = 1, TGX_MIXER_ATTENTION = 2, TGX_MIXER_MLSTM = 3, TGX_MIXER_WKV = 4, TGX_MIXER_PARALLEL = 5, TGX_MIXER_MAMBA1 = 6 } tgx_mixer;
 typedef enum tgx_mlp { TGX_MLP_NONE = 0, TGX_MLP_MOE = 1, TGX_MLP_DENSE = 2 } tgx_mlp;
 typedef enum tgx_mask { TGX_MASK_CAUSAL = 0, TGX_MASK_WINDOW = 1, TGX_MASK_CHUNK = 2 } tgx_mask;
 
@@ -201,19 +219,28 @@ typedef struct tgx_layer_desc {
   float left_scale;  /* parallel: weight of the attention half                                    */
   float right_scale; /* parallel: weight of the gated delta rule                                  */
   /* ABI 7 (zero for the kinds that do not read them) */
-  int32_t qk_norm;   /* attention: 1 = unit-RMS queries and keys per head                         */
+  int32_t qk_norm;   /* attention: 1 = unit-RMS queries and keys per head, 2 (ABI 8) = times a learned vector */
   int32_t score_fn;  /* attention: 0 = softmax over the visible keys, 1 = sigmoid(score + per-head bias), not normalised */
   int32_t head_mix;  /* attention: 1 = weights mixed across heads by a [heads][heads] matrix      */
   int32_t gate_kind; /* output gate: 0 = the family's own, 1 = per channel, 2 = per head          */
   int32_t rot_dim;   /* latent attention: rotated query / key dimensions per head beside `dim` (0: none) */
-  int32_t ff_act;    /* dense feed-forward: 0 = the family's own, 1 = erf gelu without a gate     */
+  int32_t ff_act;    /* dense feed-forward: 0 = the family's own, 1 = erf gelu without a gate, 2 (ABI 8) = squared relu without a gate */
   int32_t router_fn; /* experts: 0 = softmax scores + correction, 1 = sigmoid scores              */
   int32_t group_score; /* experts: a group counts as 0 = its largest, 1 = the sum of its two largest scores */
   int32_t router_norm; /* experts: 1 = weights divided by their sum + 1e-20                       */
+  /* ABI 8 (zero for the kinds that do not read them) */
+  int32_t v_is_k;    /* attention: 1 = the key projections are the values                         */
+  int32_t head_sink; /* attention: 1 = a learned sink per head                                    */
+  int32_t bias_max;  /* attention: distance from which the bucketed distance bias takes its last row (0: no such bias) */
+  int32_t bias_buckets; /* ... rows of its table (0: from the tensor)                             */
+  int32_t right_kind; /* parallel: the right half is 0 = the gated delta rule, 1 = a scalar-decay state-space mixer */
+  int32_t part_norms; /* state-space mixer: equal parts of its output norm                        */
+  int32_t inner;     /* mamba1: channels                                                          */
+  int32_t dt_rank;   /* mamba1: inner size of the step sizes' product                             */
 } tgx_layer_desc;
 
 typedef struct tgx_stack_desc {
-  int32_t family;         /* tgx_family (TGX_FAMILY_ZAKUSUN, TGX_FAMILY_MODEPEL, TGX_FAMILY_VITUDRA, TGX_FAMILY_ZALUVIK) */
+  int32_t family;         /* tgx_family (TGX_FAMILY_ZAKUSUN, TGX_FAMILY_MODEPEL, TGX_FAMILY_VITUDRA, TGX_FAMILY_ZALUVIK, TGX_FAMILY_NUSOVIK) */
   int32_t width;          /* residual width                                                        */
   int32_t layers;         /* entries of the tgx_layer_desc array                                   */
   int32_t vocab;
@@ -227,7 +254,7 @@ typedef struct tgx_stack_desc {
   int32_t canon_taps;     /* taps of the input convolution (>= 1)                                  */
   float logit_scale;      /* logits = embed . norm(x) * logit_scale                                */
   float residual_mult;    /* ABI 6, TGX_FAMILY_VITUDRA / ZALUVIK: the factor on what a sublayer adds to the stream */
-  /* ABI 7, TGX_FAMILY_ZALUVIK */
+  /* ABI 7, TGX_FAMILY_ZALUVIK (embed_scale also TGX_FAMILY_NUSOVIK) */
   float embed_scale;      /* x = embed[token] * embed_scale                                         */
   int32_t loop_start;     /* layers loop_start .. loop_stop - 1 run loop_times times (an empty span: no loop) */
   int32_t loop_stop;
@@ -260,7 +287,9 @@ TGX_API int tgx_create(const tgx_model_desc* desc, int device_ordinal, tgx_ctx**
  * TGX_FAMILY_VITUDRA: "embed", "head", "final.norm", "l<i>.norm1", "l<i>.mlp.gate|up|down", attention "l<i>.mix.q|k|v|o" (no k, v with kv_share), wkv
  * "l<i>.mix.mu.r|k|v|g|w", "l<i>.mix.r|k|v|g|w1|w2|w0|u|norm|o", parallel "l<i>.mix.left.q|k|v|o", "l<i>.mix.right.q|k|v(.conv)|b|a|A_log|dt_bias|g|norm|o".
  * TGX_FAMILY_ZALUVIK: "embed", "loop.in" (with a loop), "final.norm(.b)", "l<i>.norm1|norm1b|norm2|norm2b(.b)", attention "l<i>.mix.q|k|v|talk|pb|g|o", latent
- * attention "l<i>.mix.q|dkv|dkv.norm|uk|uv|g|o", dense "l<i>.mlp.up|down", experts "l<i>.mlp.router|e<j>.gate|up|down|shared.gate|up|down". */
+ * attention "l<i>.mix.q|dkv|dkv.norm|uk|uv|g|o", dense "l<i>.mlp.up|down", experts "l<i>.mlp.router|e<j>.gate|up|down|shared.gate|up|down".
+ * TGX_FAMILY_NUSOVIK: "embed", "head", "final.norm", "l<i>.norm1|norm2", "l<i>.mlp.up|down", mamba1 "l<i>.mix.in|conv(.b)|x|dt(.b)|A_log|D|o", parallel
+ * "l<i>.mix.left.q(.b|.norm)|k(.b|.norm)|rel|sink|g|o", "l<i>.mix.right.in|conv(.b)|dt_bias|A_log|D|norm|o". */
 TGX_API int tgx_create_stack(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int device_ordinal, tgx_ctx** out_ctx);
 
 /* == SafeTensors::loadInternal -> Storage::copyOnDevice for ONE named tensor

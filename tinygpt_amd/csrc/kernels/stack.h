@@ -17,18 +17,19 @@
 namespace tgx {
 
 
-// ---- x[t] = embed[id] + pe(pos): entry 2i = sin(pos * f_i), 2i + 1 = cos(pos * f_i); f (fp32) comes from the host.  Writes the stream and layer-result slot 0.
+// ---- x[t] = embed[id] * scale + pe(pos): entry 2i = sin(pos * f_i), 2i + 1 = cos(pos * f_i); f (fp32) comes from the host.  Writes the stream and, where the
+// design keeps layer results, slot 0 of them (x0).
 template <int DT>
-__global__ __launch_bounds__(256) void sinusoid_embed_kernel(StepMeta m, const elem_t<DT>* embed, const float* freq, float* x, float* x0, int W) {
+__global__ __launch_bounds__(256) void sinusoid_embed_kernel(StepMeta m, const elem_t<DT>* embed, float scale, const float* freq, float* x, float* x0, int W) {
   const int t = blockIdx.x;
   const size_t id = (size_t)m.tok_id[t];
   const float p = (float)m.tok_pos[t];
   for (int c = threadIdx.x; c < W; c += 256) {
     const float ang = p * freq[c >> 1];
     const float pe = (c & 1) ? cosf(ang) : sinf(ang);
-    const float v = elem_to_f32<DT>(embed[id * W + c]) + pe;
+    const float v = fmaf(elem_to_f32<DT>(embed[id * W + c]), scale, pe);
     x[(size_t)t * W + c] = v;
-    x0[(size_t)t * W + c] = v;
+    if (x0) x0[(size_t)t * W + c] = v;
   }
 }
 

@@ -14,7 +14,7 @@
 
 namespace tgx {
 
-enum { SG_ACT_NONE = 0, SG_ACT_TANH = 1, SG_ACT_DECAY = 2, SG_ACT_GELU = 3 };
+enum { SG_ACT_NONE = 0, SG_ACT_TANH = 1, SG_ACT_DECAY = 2, SG_ACT_GELU = 3, SG_ACT_SOFTPLUS = 4, SG_ACT_RELU2 = 5 };
 enum { SG_STORE = 0, SG_ADD = 1, SG_GATE = 2, SG_EXPERT_ACT = 3, SG_ROWSCALE = 4, SG_SILU_MUL = 5 };
 constexpr bool sg_dual(int epi) { return epi == SG_EXPERT_ACT || epi == SG_SILU_MUL; }
 struct StackGemmArgs {
@@ -26,8 +26,8 @@ struct StackGemmArgs {
   const int* z_off; const int* tile_z; const int* tile_m0; const int* n_tiles;      // grouped
   int M, N, K;
   float scale;                 // SG_STORE: C = act(acc * scale + bias); SG_ADD: C += acc * scale
-  int act;                     // SG_STORE: SG_ACT_NONE, SG_ACT_TANH, SG_ACT_DECAY = exp(-exp(v)) (a decay in (0, 1) from a log-log pre-activation), or
-                               //           SG_ACT_GELU = v (1 + erf(v / sqrt 2)) / 2
+  int act;                     // SG_STORE: SG_ACT_NONE, SG_ACT_TANH, SG_ACT_DECAY = exp(-exp(v)) (a decay in (0, 1) from a log-log pre-activation),
+                               //           SG_ACT_GELU = v (1 + erf(v / sqrt 2)) / 2, SG_ACT_SOFTPLUS = ln(1 + e^v), or SG_ACT_RELU2 = max(v, 0)^2
   const float* bias;           // SG_STORE: [N] per z (column z * c_zoff + n), nullptr: none
   int gate_col0, gate_heads;   // SG_STORE: columns [gate_col0, + gate_heads) leave as log input gates cap tanh(v / cap), the next gate_heads columns as log forget gates
   float gate_cap;              //           logsigmoid(cap tanh(v / cap)) (the two gate rows of a matrix-memory layer's input product); gate_heads 0: none
@@ -51,6 +51,8 @@ __device__ __forceinline__ float store_value(const StackGemmArgs& a, float v, si
   if (a.gate_heads > 0 && n >= a.gate_col0) { o = soft_cap(o, a.gate_cap); if (n >= a.gate_col0 + a.gate_heads) o = log_sigmoid(o); }
   if (a.act == SG_ACT_TANH) o = tanhf(o);
   else if (a.act == SG_ACT_DECAY) o = expf(-expf(o));
+  else if (a.act == SG_ACT_SOFTPLUS) o = o > 20.f ? o : log1pf(expf(o));
+  else if (a.act == SG_ACT_RELU2) { o = fmaxf(o, 0.f); o *= o; }
   else if (a.act == SG_ACT_GELU) o = 0.5f * o * (1.0f + erff(o * 0.70710678118654752f));
   return o;
 }

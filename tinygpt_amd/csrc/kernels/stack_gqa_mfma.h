@@ -30,6 +30,10 @@ struct GqaMfmaArgs {
   float scale, sink; int has_sink;
   int mask_kind, mask_size;            // MASK_* (stack_meta.h): a row sees the keys [first_key(position), position]
   float softcap; int dist_bias;        // score shaping as in gqa_attn_kernel (softcap <= 0: none)
+  const float* sinks;                  // per-head sinks, distance table, one gate per head and output factor as in gqa_attn_kernel
+  const float* dist_tab; int dist_len;
+  int gate_per_head;
+  float out_scale;
 };
 
 template <int DT, int ND, int NT, bool SPLIT>      // ND = dim / 64: 16-channel steps of a wave's share of the contraction; NT = ceil(vdim / 128): 32-column output tiles per wave
@@ -85,8 +89,9 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
   const int skeys = svalid ? past + sr / Gq + 1 : 0;
   const int slo = first_key(skeys - 1, a.mask_kind, a.mask_size);
   const float slope2 = a.dist_bias && svalid ? distance_slope(kvh * Gq + sr % Gq, a.heads) * LOG2E : 0.f;
-  const bool sinked = a.has_sink && svalid && (!SPLIT || blockIdx.z == 0);
-  float m_s = sinked ? a.sink * LOG2E : -INFINITY, l_s = sinked ? 1.f : 0.f;      // the running maximum in base-2 units
+  const float* dist = a.dist_tab && svalid ? a.dist_tab + (size_t)(kvh * Gq + sr % Gq) * a.dist_len : nullptr;
+  const bool sinked = (a.has_sink || a.sinks) && svalid && (!SPLIT || blockIdx.z == 0);
+  float m_s = sinked ? (a.sinks ? a.sinks[kvh * Gq + sr % Gq] : a.sink) * LOG2E : -INFINITY, l_s = sinked ? 1.f : 0.f;      // the running maximum in base-2 units
 
   auto key_rows = [&](int kt) -> const bf16_t* {
     const size_t pg = (size_t)m.tbl[(size_t)slot * m.tbl_stride + (kt >> m.page_shift)];
@@ -109,6 +114,9 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
 #pragma unroll
       for (int kk = 0; kk < 4; kk++) bt[t][kk] = *reinterpret_cast<const u32x4*>(tp + 16 * kk);
     }
+    float db[8];      // the distance table's entries of this lane's eight keys (loaded ahead of the products that hide them)
+#pragma unroll
+    for (int c = 0; c < 8; c++) db[c] = dist ? dist[min(max(skeys - 1 - (kt + kq + c), 0), a.dist_len - 1)] * LOG2E : 0.f;
     // 1. partial scores over this wave's channels, keys kt .. kt + 31 and kt + 32 .. kt + 63
     f32x16 s[2];
 #pragma unroll
@@ -140,7 +148,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
         float v = s_part[0][srow][kq + c] + s_part[1][srow][kq + c] + s_part[2][srow][kq + c] + s_part[3][srow][kq + c];
         const int key = kt + kq + c;
         if (capped) v = a.softcap * tanhf(v / a.softcap) * LOG2E;
-        v = fmaf(-slope2, (float)(skeys - 1 - key), v);
+        v = fmaf(-slope2, (float)(skeys - 1 - key), v) + db[c];
         sv[c] = (key >= slo && key < min(skeys, k1)) ? v : -INFINITY;
         tmax = fmaxf(tmax, sv[c]);
       }
@@ -204,8 +212,8 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
       else {
         const size_t tok = (size_t)(start + gr / Gq), hc = (size_t)(kvh * Gq + gr % Gq) * a.vdim + col;
         float v = s_l[ri] > 0.f ? acc[t][r] / s_l[ri] : 0.f;
-        if (a.gate) v = v / (1.0f + expf(-a.gate[tok * a.ldg + hc]));
-        a.out[tok * a.ldo + hc] = v;
+        if (a.gate) v = v / (1.0f + expf(-a.gate[tok * a.ldg + (a.gate_per_head ? (size_t)(kvh * Gq + gr % Gq) : hc)]));
+        a.out[tok * a.ldo + hc] = v * a.out_scale;
       }
     }
 }

@@ -8,6 +8,7 @@
 //   rec_scan_kernel         the recurrence over an entry's tokens with the head's matrix state in registers:
 //                             REC_WKV     o = (S + diag(u) k v^T)^T r;  S <- diag(w) S + k v^T
 //                             REC_DELTA   S <- g S;  S += k (beta (v - S^T k))^T;  o = S^T q
+//                             REC_SSD     S <- g S + k (beta v)^T;  o = S^T q + skip v (a scalar-decay state-space recurrence)
 // A sequence whose first token has position 0 starts from zero state whatever its slot held.
 #pragma once
 #include "stack.h"
@@ -115,14 +116,15 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(StepMeta m, DeltaPrepAr
 // inputs (up to three vectors of `dim`) and the workgroup's value columns are staged in LDS (the next block's travel in registers meanwhile), then every
 // lane updates its DPER rows of its column with no barrier inside the block: a wave owns 8 columns, its lanes = 8 columns x 8 row groups (the row groups
 // of a column are adjacent lanes), 8 DPER >= dim.  Sums over the key channels cross the row groups on the lane crossbar.
-enum { REC_WKV = 0, REC_DELTA = 1 };
+enum { REC_WKV = 0, REC_DELTA = 1, REC_SSD = 2 };
 struct RecScanArgs {
-  const float* a; long long lda;     // per token and key head [dim]: the read vector (wkv: r, delta: q)
-  const float* k; long long ldk;     //                               k
+  const float* a; long long lda;     // per token and key head [dim]: the read vector (wkv: r, delta: q, ssd: C)
+  const float* k; long long ldk;     //                               k (ssd: B)
   const float* w; long long ldw;     //                               wkv: the decay per channel
   const float* v; long long ldv;     // per token and head [vdim]
-  const float* beta; const float* g; long long ldg;      // delta: per token and head
+  const float* beta; const float* g; long long ldg;      // delta, ssd: per token and head
   const float* u;                    // wkv: [heads][dim] bonus
+  const float* skip;                 // ssd: [heads]
   float* S;                          // [slots][heads][dim][vdim]
   float* out; long long ldo;         // [T][heads * vdim]
   int heads, kv_heads, dim, vdim;
@@ -141,6 +143,7 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
   const int kh = h / (a.heads / a.kv_heads), d0 = rg * DPER, l0 = rg * LP;
   const bool col = j < a.vdim;
   float* Sg = a.S + ((size_t)row * a.heads + h) * (size_t)a.dim * a.vdim;
+  const float skip = KIND == REC_SSD ? a.skip[h] : 0.f;
   float S[DPER], ub[KIND == REC_WKV ? DPER : 1];
 #pragma unroll
   for (int dd = 0; dd < DPER; dd++) {
@@ -166,7 +169,7 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
       const int i = tid + 256 * u, t = i / CB, c = i - t * CB;
       rv[u] = (t < nb && blockIdx.z * CB + c < a.vdim) ? a.v[(size_t)(start + t0 + t) * a.ldv + (size_t)h * a.vdim + blockIdx.z * CB + c] : 0.f;
     }
-    if (KIND == REC_DELTA && tid < nb) { rb = a.beta[(size_t)(start + t0 + tid) * a.ldg + h]; rgt = a.g[(size_t)(start + t0 + tid) * a.ldg + h]; }
+    if (KIND != REC_WKV && tid < nb) { rb = a.beta[(size_t)(start + t0 + tid) * a.ldg + h]; rgt = a.g[(size_t)(start + t0 + tid) * a.ldg + h]; }
   };
   fetch(0);
   for (int t0 = 0; t0 < cnt; t0 += TB) {
@@ -180,7 +183,7 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
     }
 #pragma unroll
     for (int u = 0; u < NV; u++) { const int i = tid + 256 * u; if (i < TB * CB) s_v[i / CB][i % CB] = rv[u]; }
-    if (KIND == REC_DELTA && tid < TB) { s_b[tid] = rb; s_g[tid] = rgt; }
+    if (KIND != REC_WKV && tid < TB) { s_b[tid] = rb; s_g[tid] = rgt; }
     __syncthreads();
     if (t0 + TB < cnt) fetch(t0 + TB);
     // a token's operands travel from LDS to registers one token ahead of their use (two register sets, taken in turn), so the reads' latency lies under
@@ -192,7 +195,7 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
 #pragma unroll
         for (int dd = 0; dd < DPER; dd += 4) k.in[s][dd / 4] = *reinterpret_cast<const f32x4*>(&s_in[s][t][l0 + dd]);
       k.v = s_v[t][jl];
-      if (KIND == REC_DELTA) { k.g = s_g[t]; k.b = s_b[t]; }
+      if (KIND != REC_WKV) { k.g = s_g[t]; k.b = s_b[t]; }
     };
     auto advance = [&](const Tok& k, int t) {
       float po = 0.f;
@@ -203,6 +206,10 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
           po = fmaf(k.in[0][dd / 4][dd & 3], fmaf(ub[dd], kv, S[dd]), po);
           S[dd] = fmaf(k.in[NA - 1][dd / 4][dd & 3], S[dd], kv);
         }
+      } else if (KIND == REC_SSD) {
+        const float bv = k.b * k.v;
+#pragma unroll
+        for (int dd = 0; dd < DPER; dd++) { S[dd] = fmaf(k.g, S[dd], k.in[1][dd / 4][dd & 3] * bv); po = fmaf(S[dd], k.in[0][dd / 4][dd & 3], po); }
       } else {
         float pk = 0.f;
 #pragma unroll
@@ -213,6 +220,7 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
         for (int dd = 0; dd < DPER; dd++) { S[dd] = fmaf(k.in[1][dd / 4][dd & 3], uj, S[dd]); po = fmaf(S[dd], k.in[0][dd / 4][dd & 3], po); }
       }
       po = row_group_sum<RG>(po);
+      if (KIND == REC_SSD) po = fmaf(skip, k.v, po);
       if (rg == 0 && col) a.out[(size_t)(start + t0 + t) * a.ldo + (size_t)h * a.vdim + j] = po;
     };
     Tok ka, kb;

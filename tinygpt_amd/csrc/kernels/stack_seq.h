@@ -117,7 +117,9 @@ struct GqaAppendArgs {
   const float* lam;
   int rot_pairs;             // 1: neighbours turn together
   float q_temp_coef; int q_temp_every;      // coef 0: no query temperature
-  float qk_unit_eps;         // > 0: every q and k head is first divided by sqrt(mean(head^2) + qk_unit_eps) (no weight)
+  float qk_unit_eps;         // > 0: every q and k head is first divided by sqrt(mean(head^2) + qk_unit_eps) ...
+  const float *q_norm, *k_norm;     // ... and multiplied by a vector of `dim` all heads share (nullptr: no weight)
+  int v_is_k;                // 1: the row holds no v: the values are the k columns as they come from the projection (vdim = dim)
   unsigned short *q_hi, *q_lo;      // [T][heads * dim] (nullptr: not kept): the finished queries as two 16-bit terms, the A operand of a matrix-core score product
 };
 template <int DT>
@@ -125,6 +127,21 @@ __global__ __launch_bounds__(256) void gqa_append_kernel(StepMeta m, GqaAppendAr
   const int t = blockIdx.x, pos = m.tok_pos[t];
   float* row = a.proj + (size_t)t * a.ldp;
   const int half = a.rot_dims >> 1, nh = a.heads + (a.poolK ? a.kv_heads : 0);      // q heads and k heads are adjacent in the row: head index hd, offset hd * dim
+  int page = 0;
+  if (a.poolK) page = m.tbl[(size_t)m.tok_row[t] * m.tbl_stride + (pos >> m.page_shift)];
+  const int pmask = (1 << m.page_shift) - 1;
+  const size_t slot = ((size_t)page << m.page_shift) + (size_t)(pos & pmask);
+  const int kd = a.kv_heads * a.dim, vd = a.kv_heads * a.vdim;
+  const float* ksrc = row + (size_t)a.heads * a.dim;
+  auto put_value = [&](int c, float v) {
+    const elem_t<DT> sv = f32_to_elem<DT>(v);
+    reinterpret_cast<elem_t<DT>*>(a.poolV)[slot * vd + c] = sv;
+    if (a.poolVT) reinterpret_cast<elem_t<DT>*>(a.poolVT)[((((size_t)page * vd) + c) << m.page_shift) + (size_t)(pos & pmask)] = sv;
+  };
+  if (a.v_is_k && a.poolK) {
+    for (int c = threadIdx.x; c < vd; c += 256) put_value(c, ksrc[c]);
+    __syncthreads();
+  }
   if (a.qk_unit_eps > 0.f) {      // a wave per head
     const int lane = threadIdx.x & 63;
     for (int hd = threadIdx.x >> 6; hd < nh; hd += 4) {
@@ -133,7 +150,8 @@ __global__ __launch_bounds__(256) void gqa_append_kernel(StepMeta m, GqaAppendAr
       for (int c = lane; c < a.dim; c += 64) ss = fmaf(u[c], u[c], ss);
       ss = wave_sum(ss);
       const float r = 1.0f / sqrtf(ss / (float)a.dim + a.qk_unit_eps);
-      for (int c = lane; c < a.dim; c += 64) u[c] *= r;
+      const float* nw = hd < a.heads ? a.q_norm : a.k_norm;
+      for (int c = lane; c < a.dim; c += 64) u[c] *= nw ? r * nw[c] : r;
     }
     __syncthreads();
   }
@@ -160,22 +178,16 @@ __global__ __launch_bounds__(256) void gqa_append_kernel(StepMeta m, GqaAppendAr
   }
   if (!a.poolK) return;
   __syncthreads();
-  const int page = m.tbl[(size_t)m.tok_row[t] * m.tbl_stride + (pos >> m.page_shift)];
-  const size_t slot = ((size_t)page << m.page_shift) + (size_t)(pos & ((1 << m.page_shift) - 1));
-  const int kd = a.kv_heads * a.dim, vd = a.kv_heads * a.vdim;
   elem_t<DT>* kdst = reinterpret_cast<elem_t<DT>*>(a.poolK) + slot * kd;
-  elem_t<DT>* vdst = reinterpret_cast<elem_t<DT>*>(a.poolV) + slot * vd;
-  const float* ksrc = row + (size_t)a.heads * a.dim;
   const float* vsrc = ksrc + kd;
   for (int c = threadIdx.x; c < kd; c += 256) kdst[c] = f32_to_elem<DT>(ksrc[c]);
+  if (a.v_is_k) return;
   const float lam = a.vmode == 2 ? a.lam[0] : 0.f;
   for (int c = threadIdx.x; c < vd; c += 256) {
     float v = vsrc[c];
     if (a.vmode == 1) a.vfirst[(size_t)t * vd + c] = v;
     if (a.vmode == 2) v = fmaf(lam, a.vfirst[(size_t)t * vd + c], __fmul_rn(1.0f - lam, v));
-    const elem_t<DT> sv = f32_to_elem<DT>(v);
-    vdst[c] = sv;
-    if (a.poolVT) reinterpret_cast<elem_t<DT>*>(a.poolVT)[((((size_t)page * vd) + c) << m.page_shift) + (size_t)(pos & ((1 << m.page_shift) - 1))] = sv;
+    put_value(c, v);
   }
 }
 
@@ -184,7 +196,7 @@ __global__ __launch_bounds__(256) void gqa_append_kernel(StepMeta m, GqaAppendAr
 // those of the step's own tokens, is read from the pool.  The output is multiplied by sigmoid(gate) where a gate is given.
 // The query at position i sees the keys [first_key(i), i]: all before it, a sliding window of mask_size positions, or its own block of mask_size
 // positions (blocks counted from position 0 of the sequence).  score = q . k * scale, then softcap * tanh(score / softcap), then minus
-// slope_h * (i - j), slope_h = 2^(-8 (h + 1) / heads), each where the layer has it.
+// slope_h * (i - j), slope_h = 2^(-8 (h + 1) / heads), then plus a table's entry for the head and the distance, each where the layer has it.
 // (first_key and distance_slope: stack_meta.h)
 struct GqaAttnArgs {
   const float* q; long long ldq;       // head h of token t at q + t * ldq + h * dim
@@ -196,7 +208,17 @@ struct GqaAttnArgs {
   float* part; int nsplit, keys_per;   // split form: records (m, l, acc[vdim]) per (token, head, split); split z takes keys_per keys from first_key on
   int mask_kind, mask_size;            // MASK_*
   float softcap; int dist_bias;        // softcap <= 0: none
+  const float* sinks;                  // [heads]: a sink per head (instead of `sink`; nullptr: none)
+  const float* dist_tab; int dist_len; // [heads][dist_len]: added to the score by distance i - j, the last entry for every larger one (nullptr: none)
+  int gate_per_head;                   // 1: one gate pre-activation per head, at gate + t * ldg + h
+  float out_scale;                     // factor on the output
 };
+// the gate's and the scale's share of one output (t, h, c)
+template <class Args>
+__device__ __forceinline__ float gated_out(const Args& a, float v, size_t t, int h, int c) {
+  if (a.gate) v = v / (1.0f + expf(-a.gate[t * a.ldg + (a.gate_per_head ? (size_t)h : (size_t)h * a.vdim + c)]));
+  return v * a.out_scale;
+}
 constexpr int GQA_MAX_RPL = 4;          // channels per lane: dim, vdim <= 256
 template <int DT, int RPL, bool SPLIT>
 __global__ __launch_bounds__(256) void gqa_attn_kernel(StepMeta m, GqaAttnArgs a) {
@@ -212,8 +234,9 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(StepMeta m, GqaAttnArgs a
   float qv[RPL], acc[RPL];
 #pragma unroll
   for (int k = 0; k < RPL; k++) { const int c = lane + 64 * k; qv[k] = c < a.dim ? q[c] : 0.f; acc[k] = 0.f; }
-  const bool sink_here = a.has_sink && wv == 0 && (!SPLIT || blockIdx.z == 0);      // the sink enters once
-  float mx = sink_here ? a.sink : -INFINITY, l = sink_here ? 1.f : 0.f;
+  const float* dist = a.dist_tab ? a.dist_tab + (size_t)h * a.dist_len : nullptr;
+  const bool sink_here = (a.has_sink || a.sinks) && wv == 0 && (!SPLIT || blockIdx.z == 0);      // the sink enters once
+  float mx = sink_here ? (a.sinks ? a.sinks[h] : a.sink) : -INFINITY, l = sink_here ? 1.f : 0.f;
   const elem_t<DT>* pk = reinterpret_cast<const elem_t<DT>*>(a.poolK) + (size_t)kvh * a.dim;
   const elem_t<DT>* pv = reinterpret_cast<const elem_t<DT>*>(a.poolV) + (size_t)kvh * a.vdim;
   const int pmask = (1 << m.page_shift) - 1;
@@ -232,6 +255,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(StepMeta m, GqaAttnArgs a
     s = wave_sum(s) * a.scale;
     if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
     s = fmaf(-slope, (float)(nkeys - 1 - j), s);
+    if (dist) s += dist[min(nkeys - 1 - j, a.dist_len - 1)];
     const float mn = fmaxf(mx, s);
     const float corr = expf(mx - mn), p = expf(s - mn);      // mx = -inf on a wave's first key: corr = 0
     l = fmaf(l, corr, p);
@@ -255,9 +279,8 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(StepMeta m, GqaAttnArgs a
     const float inv = L > 0.f ? 1.0f / L : 0.f;
     float* o = a.out + (size_t)t * a.ldo + (size_t)h * a.vdim;
     for (int c = threadIdx.x; c < a.vdim; c += 256) {
-      float v = (s_acc[c] * f[0] + s_acc[a.vdim + c] * f[1] + s_acc[2 * a.vdim + c] * f[2] + s_acc[3 * a.vdim + c] * f[3]) * inv;
-      if (a.gate) v = v / (1.0f + expf(-a.gate[(size_t)t * a.ldg + (size_t)h * a.vdim + c]));
-      o[c] = v;
+      const float v = (s_acc[c] * f[0] + s_acc[a.vdim + c] * f[1] + s_acc[2 * a.vdim + c] * f[2] + s_acc[3 * a.vdim + c] * f[3]) * inv;
+      o[c] = gated_out(a, v, (size_t)t, h, c);
     }
   }
 }
@@ -284,9 +307,7 @@ __global__ __launch_bounds__(256) void gqa_attn_merge_kernel(GqaAttnArgs a) {
   for (int c = threadIdx.x; c < a.vdim; c += 256) {
     float v = 0.f;
     for (int s = 0; s < a.nsplit; s++) v = fmaf(rec[(size_t)s * rs + 2 + c], s_f[s], v);
-    v *= inv;
-    if (a.gate) v = v / (1.0f + expf(-a.gate[(size_t)t * a.ldg + (size_t)h * a.vdim + c]));
-    o[c] = v;
+    o[c] = gated_out(a, v * inv, (size_t)t, h, c);
   }
 }
 

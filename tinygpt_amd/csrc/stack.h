@@ -53,6 +53,14 @@ struct StackLayerW {
   //   dense: w_up / w_down; experts: w_router (fp32), w_gate / w_up / w_down stacked, ws_* the shared expert
   // The caches of these layers belong to their RUNS (StackModel::runs): a layer inside the loop has one per pass.
   float *ln = nullptr, *talk = nullptr, *pb = nullptr;
+  // output-norm designs (Nusovik).  norm1 / norm2 hold the weights behind the mixer and the feed-forward (w_up / w_down).
+  //   mamba1:   w_in = [x | z] rows, conv_w / conv_b the filters, w_w1 the product for [dt | B | C], w_w2 / w0 the step sizes' product and bias, decay2 =
+  //             -exp(A_log) log2(e) [inner][state], d_skip; mS the state [slots][inner][state], conv_state the tails of the raw x columns
+  //   parallel: w_in = [left q | k | right in (z | x | B | C | dt) | left gate] rows, b_in the biases of q and k, q_norm / k_norm, sink, dist the distance bias
+  //             expanded to [heads][dist_len]; w_o = [left | right] output projections side by side [width][heads * vdim + d_heads * d_vdim]; conv_w / conv_b,
+  //             a_log, dt_bias, d_skip, head_w (the weight of the part norm) of the right half, mS its state [slots][d_heads][d_dim][d_vdim]
+  float *conv_b = nullptr, *d_skip = nullptr, *decay2 = nullptr, *q_norm = nullptr, *k_norm = nullptr, *dist = nullptr;
+  int dist_len = 0;
 };
 
 // one run of a layer (layer-norm designs): which layer's weights, whether the loop's input product comes first, and the run's own cache
@@ -76,6 +84,8 @@ struct StackModel {
   bool sandwich = false;               // scalar RMS norms before and after every sublayer, no convolutions, no depth average, no position vector, a separate head
   bool joint = false;                  // one offset-weight RMS norm per layer; mixer and feed-forward read it side by side; x += residual_mult * (their sum); a separate head
   bool affine = false;                 // layer norms (weight and bias) before and after every sublayer, x += residual_mult * norm(sublayer(norm(x))); a looped span; logits against the embedding table
+  bool post = false;                   // RMS norms (with weight) behind the sublayers only, x += norm(sublayer(x)); scaled embedding rows plus a position vector; a separate head
+  bool latent() const { return !sandwich && !joint && !affine && !post; }      // the first layered design: grouped norms, input convolutions, depth average
   std::vector<StackRun> runs;          // affine designs: the layers in the order they run
   ebyte* w_loop = nullptr;             // [width][2 width]: the loop's input product on [x; x0]
   float* xcat = nullptr;               // step workspace [T][2 width]: the stream beside the embedding output

@@ -18,6 +18,7 @@
 #include "kernels/stack_rec.h"
 #include "kernels/stack_loop.h"
 #include "kernels/stack_mix_mfma.h"
+#include "kernels/stack_ssm.h"
 
 int upload_param_ext(tgx_ctx* c, ebyte* dst, const void* host, int64_t n, int src_dtype);      // abi.hip
 
@@ -184,7 +185,7 @@ int ensure_ws(tgx_ctx* c, int T) {
   } else if (sm->affine) {   // the seam's scratch row, the shared expert's row, the stream beside the embedding output
     if ((rc = dev_alloc(c, &sm->ytmp, n * W)) || (rc = dev_alloc(c, &sm->ysh, n * W)) || (rc = dev_alloc(c, &sm->xcat, 2 * n * W)) ||
         (rc = dev_alloc(c, &sm->qplanes, 2 * n * (size_t)std::max(1, sm->max_qd) + 8))) return rc;
-  } else if (sm->joint) {    // the recurrent mixers' side buffers: un-normed outputs, token-shift mixes, the decay's inner product, the delta rule's inputs
+  } else if (sm->joint || sm->post) {    // the recurrent mixers' side buffers: un-normed outputs, token-shift mixes, low-rank inner products, the recurrences' inputs
     if ((rc = dev_alloc(c, &sm->hs, n * (size_t)std::max(1, sm->max_hv))) || (rc = dev_alloc(c, &sm->mixed, n * (size_t)std::max(1, sm->max_shift))) ||
         (rc = dev_alloc(c, &sm->lora, n * (size_t)std::max(1, sm->max_lora))) || (rc = dev_alloc(c, &sm->rec_in, n * (size_t)std::max(1, sm->max_rec)))) return rc;
   } else if ((rc = dev_alloc(c, &sm->xs, (size_t)(sm->d.layers + 1) * n * W))) return rc;
@@ -223,7 +224,7 @@ int run_layers_latent(tgx_ctx* c, const MetaPtrs& mp, int T, int S, int max_keys
   const tgx::StepMeta m = step_meta(sm, mp, T, S);
   const int W = sm->d.width, nslots = sm->d.max_seqs, nb = sm->d.canon_taps - 1;
   const size_t slot_stride = (size_t)sm->cap_tokens * W;
-  TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::sinusoid_embed_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, reinterpret_cast<const tgx::elem_t<DT>*>(c->embed), sm->freq, sm->x, sm->xs, W))
+  TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::sinusoid_embed_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, reinterpret_cast<const tgx::elem_t<DT>*>(c->embed), 1.0f, sm->freq, sm->x, sm->xs, W))
   for (int li = 0; li < sm->d.layers; li++) {
     StackLayerW& w = sm->L[(size_t)li];
     const tgx_layer_desc& ld = w.d;
@@ -356,6 +357,10 @@ struct GqaSpec {
   int mask_kind, mask_size; float softcap; int dist_bias;
   float q_temp_coef; int q_temp_every;
   float* out; long long ldo;
+  float qk_eps; const float *q_norm, *k_norm; int v_is_k;      // unit (or weighted) queries and keys; the key projections are the values
+  const float* sinks; const float* dist; int dist_len;         // per-head sinks, distance table
+  int gate_per_head;
+  float out_scale = 1.0f;
 };
 int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, int S, int max_keys, int max_count) {
   StackModel* sm = c->stack;
@@ -364,7 +369,8 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
   ap.proj = sp.proj; ap.ldp = sp.ldp; ap.heads = H; ap.kv_heads = G; ap.dim = sp.dim; ap.vdim = sp.vdim; ap.rot_dims = sp.cs ? sp.rot_dims : 0; ap.rot_pairs = sp.rot_pairs;
   ap.cs = sp.cs; ap.poolK = sp.append ? sp.poolK : nullptr; ap.poolV = sp.poolV; ap.poolVT = sp.poolVT; ap.vfirst = sm->vfirst; ap.vmode = sp.vmode; ap.lam = sp.lam;
   ap.q_temp_coef = sp.q_temp_every > 0 ? sp.q_temp_coef : 0.f; ap.q_temp_every = sp.q_temp_every;
-  if (sp.append || ap.rot_dims > 0 || ap.q_temp_coef != 0.f) TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::gqa_append_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, ap))
+  ap.qk_unit_eps = sp.qk_eps; ap.q_norm = sp.q_norm; ap.k_norm = sp.k_norm; ap.v_is_k = sp.v_is_k;
+  if (sp.append || ap.rot_dims > 0 || ap.q_temp_coef != 0.f || ap.qk_unit_eps > 0.f) TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::gqa_append_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, ap))
   // the longest run of keys any workgroup walks: everything before the token, or the mask's span (plus the matrix-core kernel's tile alignment)
   const int span = sp.mask_kind == tgx::MASK_CAUSAL ? max_keys : std::min(max_keys, sp.mask_size + 96);
   if (sp.poolVT && sm->attn_mfma) {
@@ -373,6 +379,7 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
     ma.q = sp.proj; ma.ldq = sp.ldp; ma.poolK = sp.poolK; ma.poolVT = sp.poolVT; ma.gate = sp.gate; ma.ldg = sp.ldg; ma.out = sp.out; ma.ldo = sp.ldo;
     ma.heads = H; ma.kv_heads = G; ma.dim = sp.dim; ma.vdim = sp.vdim; ma.terms = c->act16 ? 1 : 2; ma.scale = sp.scale; ma.sink = sp.sink; ma.has_sink = sp.has_sink;
     ma.mask_kind = sp.mask_kind; ma.mask_size = sp.mask_size; ma.softcap = sp.softcap; ma.dist_bias = sp.dist_bias;
+    ma.sinks = sp.sinks; ma.dist_tab = sp.dist; ma.dist_len = sp.dist_len; ma.gate_per_head = sp.gate_per_head; ma.out_scale = sp.out_scale;
     const int tiles = (max_count * (H / G) + 31) / 32;
     const long long wgs = (long long)tiles * S * G;
     int nsplit = 1;
@@ -389,6 +396,7 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
       launch_gqa_mfma(c, m, ma, dim3(tiles, S * G, nsplit), true);
       tgx::GqaAttnArgs mg{};
       mg.part = sm->part; mg.nsplit = nsplit; mg.heads = H; mg.vdim = sp.vdim; mg.gate = sp.gate; mg.ldg = sp.ldg; mg.out = sp.out; mg.ldo = sp.ldo;
+      mg.gate_per_head = sp.gate_per_head; mg.out_scale = sp.out_scale;
       hipLaunchKernelGGL(tgx::gqa_attn_merge_kernel, dim3(T, H), dim3(256), 0, c->stream, mg);
     } else {
       launch_gqa_mfma(c, m, ma, dim3(tiles, S * G), false);
@@ -399,6 +407,7 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
   aa.q = sp.proj; aa.ldq = sp.ldp; aa.poolK = sp.poolK; aa.poolV = sp.poolV; aa.gate = sp.gate; aa.ldg = sp.ldg; aa.out = sp.out; aa.ldo = sp.ldo;
   aa.heads = H; aa.kv_heads = G; aa.dim = sp.dim; aa.vdim = sp.vdim; aa.scale = sp.scale; aa.sink = sp.sink; aa.has_sink = sp.has_sink;
   aa.mask_kind = sp.mask_kind; aa.mask_size = sp.mask_size; aa.softcap = sp.softcap; aa.dist_bias = sp.dist_bias;
+  aa.sinks = sp.sinks; aa.dist_tab = sp.dist; aa.dist_len = sp.dist_len; aa.gate_per_head = sp.gate_per_head; aa.out_scale = sp.out_scale;
   int nsplit = 1;
   if (span >= sm->gqa_split_min_keys && (long long)T * H < 2LL * c->num_cus) {      // few (token, head) pairs and a long context: the keys are divided between workgroups
     nsplit = (int)std::min<long long>(64, (4LL * c->num_cus) / ((long long)T * H));
@@ -580,7 +589,9 @@ void launch_rec_scan(tgx_ctx* c, const tgx::StepMeta& m, const tgx::RecScanArgs&
     else if (dper <= 16) hipLaunchKernelGGL((tgx::rec_scan_kernel<16, KIND>), grid, dim3(256), 0, c->stream, m, a);
     else hipLaunchKernelGGL((tgx::rec_scan_kernel<32, KIND>), grid, dim3(256), 0, c->stream, m, a);
   };
-  if (kind == tgx::REC_WKV) go(std::integral_constant<int, tgx::REC_WKV>{}); else go(std::integral_constant<int, tgx::REC_DELTA>{});
+  if (kind == tgx::REC_WKV) go(std::integral_constant<int, tgx::REC_WKV>{});
+  else if (kind == tgx::REC_SSD) go(std::integral_constant<int, tgx::REC_SSD>{});
+  else go(std::integral_constant<int, tgx::REC_DELTA>{});
 }
 
 int run_joint_attention(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T, int S, int max_keys, int max_count) {
@@ -1143,7 +1154,310 @@ int check_affine_desc(const tgx_stack_desc& d, const tgx_layer_desc* layers) {
   return TGX_OK;
 }
 
+// ---- output-norm designs (Nusovik): per layer  x += norm1(mixer(x))  and  x += norm2(ff(x)); the sublayers read the stream itself.
+int pad4(int n) { return (n + 3) & ~3; }      // row strides of buffers whose rows are read in vectors of four
+
+// y = A . W^T into the sublayers' output rows
+void sublayer_out(tgx_ctx* c, const float* A, int K, const ebyte* Wm, int T) {
+  StackModel* sm = c->stack;
+  tgx::StackGemmArgs g{};
+  g.A = A; g.lda = K; g.B = Wm; g.ldb = K; g.C = sm->yd; g.ldc = sm->d.width; g.M = T; g.N = sm->d.width; g.K = K; g.scale = 1.f;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+}
+void post_norm_add(tgx_ctx* c, const float* w, int T) {
+  StackModel* sm = c->stack;
+  tgx::PostNormArgs a{};
+  a.x = sm->x; a.y = sm->yd; a.w = w; a.W = sm->d.width; a.eps = sm->d.norm_eps;
+  hipLaunchKernelGGL(tgx::post_norm_add_kernel, dim3(T), dim3(256), 0, c->stream, a);
+}
+void launch_conv_silu(tgx_ctx* c, const tgx::StepMeta& m, tgx::ConvSiluArgs a, int T) {
+  const int cols = (a.C + 255) / 256 + (a.heads > 0 ? 1 : 0);
+  a.tile = (long long)T * cols >= 16LL * c->num_cus ? 8 : 1;      // tokens per workgroup: rows are kept in registers from token to token once the grid fills the chip
+  const dim3 grid((T + a.tile - 1) / a.tile, cols);
+  switch (a.taps) {
+    case 2: hipLaunchKernelGGL(tgx::conv_silu_kernel<2>, grid, dim3(256), 0, c->stream, m, a); break;
+    case 3: hipLaunchKernelGGL(tgx::conv_silu_kernel<3>, grid, dim3(256), 0, c->stream, m, a); break;
+    case 4: hipLaunchKernelGGL(tgx::conv_silu_kernel<4>, grid, dim3(256), 0, c->stream, m, a); break;
+    default: hipLaunchKernelGGL(tgx::conv_silu_kernel<0>, grid, dim3(256), 0, c->stream, m, a); break;
+  }
+}
+template <int SPL, int LPC>
+void launch_sel_scan_t(tgx_ctx* c, const tgx::StepMeta& m, const tgx::SelScanArgs& a, int S) {
+  hipLaunchKernelGGL((tgx::selective_scan_kernel<SPL, LPC>), dim3((a.C + 256 / LPC - 1) / (256 / LPC), S), dim3(256), 0, c->stream, m, a);
+}
+constexpr int SEL_SCAN_MAX_STATE = 256;
+void launch_sel_scan(tgx_ctx* c, const tgx::StepMeta& m, const tgx::SelScanArgs& a, int S) {
+  if (a.N <= 8) launch_sel_scan_t<1, 8>(c, m, a, S);
+  else if (a.N <= 16) launch_sel_scan_t<1, 16>(c, m, a, S);
+  else if (a.N <= 24) launch_sel_scan_t<3, 8>(c, m, a, S);
+  else if (a.N <= 32) launch_sel_scan_t<2, 16>(c, m, a, S);
+  else if (a.N <= 64) launch_sel_scan_t<4, 16>(c, m, a, S);
+  else if (a.N <= 128) launch_sel_scan_t<8, 16>(c, m, a, S);
+  else launch_sel_scan_t<16, 16>(c, m, a, S);
+}
+
+void run_mamba1(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T, int S) {
+  StackModel* sm = c->stack;
+  const tgx_layer_desc& ld = w.d;
+  const int W = sm->d.width, I = ld.inner, N = ld.d_dim, R = ld.dt_rank, ldq = pad4(R + 2 * N), nb = ld.conv_taps - 1;
+  // [x | z] = h . w_in^T
+  tgx::StackGemmArgs g{};
+  g.A = sm->x; g.lda = W; g.B = w.w_in; g.ldb = W; g.C = sm->proj; g.ldc = 2LL * I; g.M = T; g.N = 2 * I; g.K = W; g.scale = 1.f;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  tgx::ConvSiluArgs ca{};
+  ca.proj = sm->proj; ca.ldp = 2LL * I; ca.cw = w.conv_w; ca.cb = w.conv_b; ca.out = sm->rec_in; ca.ldo = I; ca.state = nb > 0 ? w.conv_state : nullptr;
+  ca.state_buf = (size_t)sm->d.max_seqs * nb * I; ca.C = I; ca.taps = ld.conv_taps;
+  launch_conv_silu(c, m, ca, T);
+  // [dt | B | C] = x . w_x^T, then the step sizes softplus(dt . w_dt^T + b), which take the place of the raw x columns
+  g = tgx::StackGemmArgs{};
+  g.A = sm->rec_in; g.lda = I; g.B = w.w_w1; g.ldb = I; g.C = sm->lora; g.ldc = ldq; g.M = T; g.N = R + 2 * N; g.K = I; g.scale = 1.f;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  g = tgx::StackGemmArgs{};
+  g.A = sm->lora; g.lda = ldq; g.B = w.w_w2; g.ldb = R; g.C = sm->proj; g.ldc = 2LL * I; g.M = T; g.N = I; g.K = R; g.scale = 1.f; g.bias = w.w0; g.act = tgx::SG_ACT_SOFTPLUS;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  tgx::SelScanArgs sa{};
+  sa.dt = sm->proj; sa.ldt = 2LL * I; sa.x = sm->rec_in; sa.ldx = I; sa.z = sm->proj + I; sa.ldz = 2LL * I; sa.bc = sm->lora + R; sa.ldbc = ldq; sa.ccol = N;
+  sa.A2 = w.decay2; sa.D = w.d_skip; sa.S = w.mS; sa.out = sm->o; sa.ldo = I; sa.C = I; sa.N = N;
+  launch_sel_scan(c, m, sa, S);
+  sublayer_out(c, sm->o, I, w.w_o, T);
+}
+
+int run_ssm_parallel(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T, int S, int max_keys, int max_count) {
+  StackModel* sm = c->stack;
+  const tgx_layer_desc& ld = w.d;
+  const int W = sm->d.width, H = ld.heads, G = ld.kv_heads, lq = H * ld.dim, lk = G * ld.dim, lvd = H * ld.vdim;
+  const int rH = ld.d_heads, I = rH * ld.d_vdim, gn = ld.d_kv_heads * ld.d_dim, C = I + 2 * gn, r0 = lq + lk, nin = r0 + I + C + rH + H, ldp = pad4(nin), ldo = lvd + I, nb = ld.conv_taps - 1;
+  // [left q | k | right z | x | B | C | dt | left gate] = h . w_in^T (+ the biases of q and k): both halves read the same input
+  tgx::StackGemmArgs g{};
+  g.A = sm->x; g.lda = W; g.B = w.w_in; g.ldb = W; g.C = sm->proj; g.ldc = ldp; g.M = T; g.N = nin; g.K = W; g.scale = 1.f; g.bias = w.b_in;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  GqaSpec sp{};
+  sp.proj = sm->proj; sp.ldp = ldp; sp.heads = H; sp.kv_heads = G; sp.dim = ld.dim; sp.vdim = ld.vdim; sp.poolK = w.pool; sp.poolV = w.poolV; sp.poolVT = w.poolVT; sp.append = true;
+  sp.qk_eps = sm->d.norm_eps; sp.q_norm = w.q_norm; sp.k_norm = w.k_norm; sp.v_is_k = 1; sp.sinks = w.sink; sp.dist = w.dist; sp.dist_len = w.dist_len;
+  sp.gate = sm->proj + r0 + I + C + rH; sp.ldg = ldp; sp.gate_per_head = 1; sp.scale = ld.scale; sp.mask_kind = ld.mask_kind; sp.mask_size = ld.mask_size;
+  sp.out = sm->o; sp.ldo = ldo; sp.out_scale = ld.left_scale;
+  int rc = run_gqa_core(c, m, sp, T, S, max_keys, max_count);
+  if (rc) return rc;
+  // the right half: rec_in row = [x | B | C | dt | decay | log decay]
+  const int ldr = pad4(C + 3 * rH);
+  tgx::ConvSiluArgs ca{};
+  ca.proj = sm->proj; ca.ldp = ldp; ca.col0 = r0 + I; ca.cw = w.conv_w; ca.cb = w.conv_b; ca.out = sm->rec_in; ca.ldo = ldr; ca.state = nb > 0 ? w.conv_state : nullptr;
+  ca.state_buf = (size_t)sm->d.max_seqs * nb * C; ca.C = C; ca.taps = ld.conv_taps; ca.heads = rH; ca.dt_col = r0 + I + C; ca.dt_bias = w.dt_bias; ca.a_log = w.a_log;
+  launch_conv_silu(c, m, ca, T);
+  tgx::RecScanArgs ra{};
+  ra.a = sm->rec_in + I + gn; ra.lda = ldr; ra.k = sm->rec_in + I; ra.ldk = ldr; ra.v = sm->rec_in; ra.ldv = ldr; ra.beta = sm->rec_in + C; ra.g = sm->rec_in + C + rH; ra.ldg = ldr;
+  ra.skip = w.d_skip; ra.S = w.mS; ra.out = sm->hs; ra.ldo = I; ra.heads = rH; ra.kv_heads = ld.d_kv_heads; ra.dim = ld.d_dim; ra.vdim = ld.d_vdim;
+  launch_rec_scan(c, m, ra, tgx::REC_SSD, S);
+  tgx::PartNormArgs pa{};
+  pa.y = sm->hs; pa.ldy = I; pa.z = sm->proj + r0; pa.ldz = ldp; pa.w = w.head_w; pa.out = sm->o + lvd; pa.ldo = ldo; pa.n = I / ld.part_norms; pa.eps = sm->d.norm_eps; pa.scale = ld.right_scale;
+  hipLaunchKernelGGL(tgx::part_norm_gate_kernel, dim3(T, ld.part_norms), dim3(256), 0, c->stream, pa);
+  sublayer_out(c, sm->o, ldo, w.w_o, T);      // one product over both halves' outputs
+  return TGX_OK;
+}
+
+int run_layers_post(tgx_ctx* c, const MetaPtrs& mp, int T, int S, int max_keys, int max_count) {
+  StackModel* sm = c->stack;
+  const tgx::StepMeta m = step_meta(sm, mp, T, S);
+  const int W = sm->d.width;
+  TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::sinusoid_embed_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, reinterpret_cast<const tgx::elem_t<DT>*>(c->embed), sm->d.embed_scale, sm->freq,
+                                          sm->x, (float*)nullptr, W))
+  for (int li = 0; li < sm->d.layers; li++) {
+    StackLayerW& w = sm->L[(size_t)li];
+    const tgx_layer_desc& ld = w.d;
+    if (ld.mixer == TGX_MIXER_MAMBA1) run_mamba1(c, m, w, T, S);
+    else { int rc = run_ssm_parallel(c, m, w, T, S, max_keys, max_count); if (rc) return rc; }
+    post_norm_add(c, w.norm1, T);
+    if (ld.mlp != TGX_MLP_DENSE) continue;
+    tgx::StackGemmArgs g{};      // down(max(up x, 0)^2)
+    g.A = sm->x; g.lda = W; g.B = w.w_up; g.ldb = W; g.C = sm->yh; g.ldc = ld.ff; g.M = T; g.N = ld.ff; g.K = W; g.scale = 1.f; g.act = tgx::SG_ACT_RELU2;
+    launch_gemm(c, g, tgx::SG_STORE, 1);
+    sublayer_out(c, sm->yh, ld.ff, w.w_down, T);
+    post_norm_add(c, w.norm2, T);
+  }
+  return TGX_OK;
+}
+
+// parameter storage of an output-norm design (Nusovik)
+int create_post_layers(tgx_ctx* c, const tgx_layer_desc* layers) {
+  StackModel* sm = c->stack;
+  const tgx_stack_desc& d = sm->d;
+  const size_t W = (size_t)d.width, es = c->esz;
+  int rc;
+  if ((rc = dev_alloc(c, &sm->head, (size_t)d.vocab * W * es))) return rc;
+  sm->missing.insert("head");
+  sm->max_top = 1; sm->max_E = 1; sm->max_ff = 1;      // the feed-forward's hidden row and the sublayers' outputs use the expert buffers with one row per token
+  auto need = [&](const std::string& p, std::initializer_list<const char*> names) { for (const char* n : names) sm->missing.insert(p + n); };
+  for (int i = 0; i < d.layers; i++) {
+    StackLayerW& w = sm->L[(size_t)i];
+    w.d = layers[i];
+    const tgx_layer_desc& l = w.d;
+    const std::string p = "l" + std::to_string(i) + ".";
+    if ((rc = dev_alloc(c, &w.norm1, W))) return rc;
+    need(p, {"norm1"});
+    if (l.mixer == TGX_MIXER_MAMBA1) {
+      const size_t I = (size_t)l.inner, N = (size_t)l.d_dim, R = (size_t)l.dt_rank;
+      if ((rc = dev_alloc(c, &w.w_in, 2 * I * W * es)) || (rc = dev_alloc(c, &w.w_o, W * I * es)) || (rc = dev_alloc(c, &w.conv_w, I * (size_t)l.conv_taps)) || (rc = dev_alloc(c, &w.conv_b, I)) ||
+          (rc = dev_alloc(c, &w.w_w1, (R + 2 * N) * I * es)) || (rc = dev_alloc(c, &w.w_w2, I * R * es)) || (rc = dev_alloc(c, &w.w0, I)) || (rc = dev_alloc(c, &w.decay2, I * N)) ||
+          (rc = dev_alloc(c, &w.d_skip, I))) return rc;
+      need(p, {"mix.in", "mix.conv", "mix.conv.b", "mix.x", "mix.dt", "mix.dt.b", "mix.A_log", "mix.D", "mix.o"});
+      sm->max_in = std::max(sm->max_in, 2 * l.inner); sm->max_hv = std::max(sm->max_hv, l.inner); sm->max_rec = std::max(sm->max_rec, l.inner);
+      sm->max_lora = std::max(sm->max_lora, pad4(l.dt_rank + 2 * l.d_dim));
+    } else {
+      const size_t H = (size_t)l.heads, lq = H * l.dim, lk = (size_t)l.kv_heads * l.dim, lvd = H * l.vdim, rH = (size_t)l.d_heads, I = rH * l.d_vdim, C = I + 2 * (size_t)l.d_kv_heads * l.d_dim;
+      const size_t nin = lq + lk + I + C + rH + H;
+      if ((rc = dev_alloc(c, &w.w_in, nin * W * es)) || (rc = dev_alloc(c, &w.b_in, nin)) || (rc = dev_alloc(c, &w.w_o, W * (lvd + I) * es)) || (rc = dev_alloc(c, &w.q_norm, (size_t)l.dim)) ||
+          (rc = dev_alloc(c, &w.k_norm, (size_t)l.dim)) || (rc = dev_alloc(c, &w.sink, H)) || (rc = dev_alloc(c, &w.conv_w, C * (size_t)l.conv_taps)) || (rc = dev_alloc(c, &w.conv_b, C)) ||
+          (rc = dev_alloc(c, &w.a_log, rH)) || (rc = dev_alloc(c, &w.dt_bias, rH)) || (rc = dev_alloc(c, &w.d_skip, rH)) || (rc = dev_alloc(c, &w.head_w, I))) return rc;
+      HIP_OK(c, hipMemset(w.b_in, 0, nin * 4));
+      w.dist_len = std::min(l.bias_max, d.max_ctx - 1) + 1;      // distances 0 .. bias_max; from there on every distance takes the last row
+      if ((rc = dev_alloc(c, &w.dist, H * (size_t)w.dist_len))) return rc;
+      need(p, {"mix.left.q", "mix.left.q.b", "mix.left.q.norm", "mix.left.k", "mix.left.k.b", "mix.left.k.norm", "mix.left.rel", "mix.left.sink", "mix.left.g", "mix.left.o",
+               "mix.right.in", "mix.right.conv", "mix.right.conv.b", "mix.right.dt_bias", "mix.right.A_log", "mix.right.D", "mix.right.norm", "mix.right.o"});
+      sm->max_in = std::max(sm->max_in, pad4((int)nin)); sm->max_hv = std::max(sm->max_hv, (int)(lvd + I)); sm->max_rec = std::max(sm->max_rec, pad4((int)(C + 3 * rH)));
+    }
+    if (l.mlp == TGX_MLP_DENSE) {
+      const size_t F = (size_t)l.ff;
+      if ((rc = dev_alloc(c, &w.norm2, W)) || (rc = dev_alloc(c, &w.w_up, F * W * es)) || (rc = dev_alloc(c, &w.w_down, W * F * es))) return rc;
+      need(p, {"norm2", "mlp.up", "mlp.down"});
+      sm->max_ff = std::max(sm->max_ff, l.ff);
+    }
+  }
+  return TGX_OK;
+}
+
+// row of a bucketed distance table with B rows for distance n: exact below B / 2, logarithmic up to D, the last row from there on
+int distance_bucket(int n, int B, int D) {
+  const int half = B / 2;
+  if (n < half) return n;
+  if (n >= D) return B - 1;
+  // (the small term keeps a logarithm that is a whole number, such as ln 4 / ln 16 * 8, on its own side of the floor)
+  return std::min(B - 1, half + (int)floor(log((double)n / half) / log((double)D / half) * (B - half) + 1e-9));
+}
+
+// tensors of an output-norm design by checkpoint name
+int upload_post(tgx_ctx* c, const char* name, const void* host, const int64_t* shape, int nd, int src_dtype) {
+  StackModel* sm = c->stack;
+  const tgx_stack_desc& d = sm->d;
+  const int64_t W = d.width;
+  const bool probe = nd < 0;
+  auto bad_shape = [&]() { return set_err(c, TGX_ERR_SHAPE, "shape not equal for tensor: %s", name); };
+  auto is = [&](int64_t a, int64_t b) { return b < 0 ? (nd == 1 && shape[0] == a) : (nd == 2 && shape[0] == a && shape[1] == b); };
+  auto done = [&](int rc) { if (!rc) sm->missing.erase(name); return rc; };
+  auto mat = [&](ebyte* dst, int64_t row0, int64_t rows, int64_t cols) {
+    if (probe) return (int)TGX_ERR_SHAPE;
+    if (!is(rows, cols)) return bad_shape();
+    return done(upload_param_ext(c, dst + (size_t)(row0 * cols) * c->esz, host, rows * cols, src_dtype));
+  };
+  auto vec = [&](float* dst, int64_t n, int64_t n2 = -1) {      // an fp32 vector, or (n2 >= 0) an fp32 matrix [n][n2]
+    if (probe) return (int)TGX_ERR_SHAPE;
+    if (!is(n, n2)) return bad_shape();
+    return done(upload_f32(c, dst, host, n2 < 0 ? n : n * n2, src_dtype));
+  };
+  auto columns = [&](ebyte* dst, int64_t rows, int64_t cols, int64_t ld, int64_t col0) {      // a matrix into columns col0 .. of one with rows of ld
+    if (probe) return (int)TGX_ERR_SHAPE;
+    if (!is(rows, cols)) return bad_shape();
+    ebyte* tmp = nullptr;
+    int rc = dev_alloc(c, &tmp, (size_t)(rows * cols) * c->esz);
+    if (!rc) rc = upload_param_ext(c, tmp, host, rows * cols, src_dtype);
+    if (!rc && hipMemcpy2D(dst + (size_t)col0 * c->esz, (size_t)ld * c->esz, tmp, (size_t)cols * c->esz, (size_t)cols * c->esz, (size_t)rows, hipMemcpyDeviceToDevice) != hipSuccess)
+      rc = set_err(c, TGX_ERR_DEVICE, "hipMemcpy2D failed for tensor %s", name);
+    if (!rc && hipDeviceSynchronize() != hipSuccess) rc = set_err(c, TGX_ERR_DEVICE, "copy of tensor %s failed", name);
+    if (tmp) (void)hipFree(tmp);
+    return done(rc);
+  };
+  if (!strcmp(name, "embed")) return mat(c->embed, 0, d.vocab, W);
+  if (!strcmp(name, "head")) return mat(sm->head, 0, d.vocab, W);
+  if (!strcmp(name, "final.norm")) return vec(sm->final_norm, W);
+  int li = -1;
+  char rest[128] = {0};
+  if (sscanf(name, "l%d.%127s", &li, rest) != 2 || li < 0 || li >= d.layers) return set_err(c, TGX_ERR_NAME, "Unexpected key: %s", name);
+  StackLayerW& w = sm->L[(size_t)li];
+  const tgx_layer_desc& l = w.d;
+  if (!strcmp(rest, "norm1")) return vec(w.norm1, W);
+  if (l.mlp == TGX_MLP_DENSE) {
+    if (!strcmp(rest, "norm2")) return vec(w.norm2, W);
+    if (!strcmp(rest, "mlp.up")) return mat(w.w_up, 0, l.ff, W);
+    if (!strcmp(rest, "mlp.down")) return mat(w.w_down, 0, W, l.ff);
+  }
+  if (l.mixer == TGX_MIXER_MAMBA1) {
+    const int64_t I = l.inner, N = l.d_dim, R = l.dt_rank;
+    if (!strcmp(rest, "mix.in")) return mat(w.w_in, 0, 2 * I, W);
+    if (!strcmp(rest, "mix.conv")) return vec(w.conv_w, I, l.conv_taps);
+    if (!strcmp(rest, "mix.conv.b")) return vec(w.conv_b, I);
+    if (!strcmp(rest, "mix.x")) return mat(w.w_w1, 0, R + 2 * N, I);
+    if (!strcmp(rest, "mix.dt")) return mat(w.w_w2, 0, I, R);
+    if (!strcmp(rest, "mix.dt.b")) return vec(w.w0, I);
+    if (!strcmp(rest, "mix.D")) return vec(w.d_skip, I);
+    if (!strcmp(rest, "mix.o")) return mat(w.w_o, 0, W, I);
+    if (!strcmp(rest, "mix.A_log")) {      // the decay's exponent in base 2 per unit step
+      if (probe) return TGX_ERR_SHAPE;
+      if (!is(I, N)) return bad_shape();
+      std::vector<float> v = to_f32(host, I * N, src_dtype);
+      for (float& a : v) a = (float)(-exp((double)a) * 1.4426950408889634);
+      return done(upload_f32(c, w.decay2, v.data(), I * N, TGX_F32));
+    }
+  } else {
+    const int64_t H = l.heads, lq = H * l.dim, lk = (int64_t)l.kv_heads * l.dim, lvd = H * l.vdim, rH = l.d_heads, I = rH * l.d_vdim, C = I + 2 * (int64_t)l.d_kv_heads * l.d_dim, nr = I + C + rH;
+    if (!strcmp(rest, "mix.left.q")) return mat(w.w_in, 0, lq, W);
+    if (!strcmp(rest, "mix.left.q.b")) return vec(w.b_in, lq);
+    if (!strcmp(rest, "mix.left.q.norm")) return vec(w.q_norm, l.dim);
+    if (!strcmp(rest, "mix.left.k")) return mat(w.w_in, lq, lk, W);
+    if (!strcmp(rest, "mix.left.k.b")) return vec(w.b_in + lq, lk);
+    if (!strcmp(rest, "mix.left.k.norm")) return vec(w.k_norm, l.dim);
+    if (!strcmp(rest, "mix.left.sink")) return vec(w.sink, H);
+    if (!strcmp(rest, "mix.left.g")) return mat(w.w_in, lq + lk + nr, H, W);
+    if (!strcmp(rest, "mix.left.o")) return columns(w.w_o, W, lvd, lvd + I, 0);
+    if (!strcmp(rest, "mix.left.rel")) {      // [rows][heads] -> one value per (head, distance)
+      if (probe) return TGX_ERR_SHAPE;
+      if (nd != 2 || shape[1] != H || shape[0] < 2 || shape[0] > (1 << 20) || (l.bias_buckets > 0 && shape[0] != l.bias_buckets)) return bad_shape();
+      const int B = (int)shape[0];
+      if (l.bias_max <= B / 2) return set_err(c, TGX_ERR_INVALID, "%s: bias_max %d within the %d exact rows of the table", name, l.bias_max, B / 2);
+      const std::vector<float> v = to_f32(host, (int64_t)B * H, src_dtype);
+      std::vector<float> t((size_t)H * w.dist_len);
+      for (int n = 0; n < w.dist_len; n++) {
+        const int b = distance_bucket(n, B, l.bias_max);
+        for (int64_t h = 0; h < H; h++) t[(size_t)h * w.dist_len + n] = v[(size_t)b * H + h];
+      }
+      return done(upload_f32(c, w.dist, t.data(), (int64_t)t.size(), TGX_F32));
+    }
+    if (!strcmp(rest, "mix.right.in")) return mat(w.w_in, lq + lk, nr, W);
+    if (!strcmp(rest, "mix.right.conv")) return vec(w.conv_w, C, l.conv_taps);
+    if (!strcmp(rest, "mix.right.conv.b")) return vec(w.conv_b, C);
+    if (!strcmp(rest, "mix.right.dt_bias")) return vec(w.dt_bias, rH);
+    if (!strcmp(rest, "mix.right.A_log")) return vec(w.a_log, rH);
+    if (!strcmp(rest, "mix.right.D")) return vec(w.d_skip, rH);
+    if (!strcmp(rest, "mix.right.norm")) return vec(w.head_w, I);
+    if (!strcmp(rest, "mix.right.o")) return columns(w.w_o, W, I, lvd + I, lvd);
+  }
+  return set_err(c, TGX_ERR_NAME, "Unexpected key: %s", name);
+}
+
+// what an output-norm design's description may ask for
+int check_post_desc(const tgx_stack_desc& d, const tgx_layer_desc* layers) {
+  for (int i = 0; i < d.layers; i++) {
+    const tgx_layer_desc& l = layers[i];
+    if (l.conv_taps < 1 || l.conv_taps > tgx::DELTA_MAX_TAPS) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: %d convolution taps (1 .. %d)", i, l.conv_taps, tgx::DELTA_MAX_TAPS);
+    if (l.mixer == TGX_MIXER_MAMBA1) {
+      if (l.inner <= 0 || l.d_dim <= 0 || l.d_dim > SEL_SCAN_MAX_STATE || l.dt_rank <= 0)
+        return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: mamba1: %d channels, %d state numbers (1 .. %d), step-size rank %d", i, l.inner, l.d_dim, SEL_SCAN_MAX_STATE, l.dt_rank);
+    } else if (l.mixer == TGX_MIXER_PARALLEL) {
+      if (l.right_kind != 1 || !l.v_is_k || !l.head_sink || l.qk_norm != 2 || l.gate_kind != 2) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: this family's parallel mixer runs sink attention with keys as values beside a state-space mixer", i);
+      if (l.heads <= 0 || l.kv_heads <= 0 || l.heads % l.kv_heads || l.dim <= 0 || l.dim > 64 * tgx::GQA_MAX_RPL || l.vdim != l.dim)
+        return set_err(nullptr, TGX_ERR_INVALID, "layer %d: attention: %d query heads over %d key heads of %d (1 .. %d), values of %d", i, l.heads, l.kv_heads, l.dim, 64 * tgx::GQA_MAX_RPL, l.vdim);
+      if (l.mask_kind < 0 || l.mask_kind > 2 || (l.mask_kind != 0 && l.mask_size < 1)) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: mask", i);
+      if (l.bias_max < 1 || l.bias_buckets < 0) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: bias_max %d, bias_buckets %d", i, l.bias_max, l.bias_buckets);
+      if (l.d_heads <= 0 || l.d_kv_heads <= 0 || l.d_heads % l.d_kv_heads || l.d_dim <= 0 || l.d_dim > 256 || l.d_vdim <= 0)
+        return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: state-space half: %d heads over %d groups, %d state numbers (1 .. 256) x %d", i, l.d_heads, l.d_kv_heads, l.d_dim, l.d_vdim);
+      if (l.part_norms < 1 || (l.d_heads * l.d_vdim) % l.part_norms) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: %d channels in %d equal parts", i, l.d_heads * l.d_vdim, l.part_norms);
+    } else return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: mixer %d is not part of this family (mamba1 and parallel are)", i, l.mixer);
+    if (l.mlp != TGX_MLP_NONE && l.mlp != TGX_MLP_DENSE) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: feed-forward kind %d is not implemented", i, l.mlp);
+    if (l.mlp == TGX_MLP_DENSE && (l.ff <= 0 || l.ff_act != 2)) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: ff %d, activation %d", i, l.ff, l.ff_act);
+  }
+  return TGX_OK;
+}
+
 int run_layers(tgx_ctx* c, const MetaPtrs& mp, int T, int S, int max_keys, int max_count) {
+  if (c->stack->post) return run_layers_post(c, mp, T, S, max_keys, max_count);
   if (c->stack->affine) return run_layers_affine(c, mp, T, S, max_keys, max_count);
   if (c->stack->joint) return run_layers_joint(c, mp, T, S, max_keys, max_count);
   return c->stack->sandwich ? run_layers_sandwich(c, mp, T, S, max_keys, max_count) : run_layers_latent(c, mp, T, S, max_keys, max_count);
@@ -1154,7 +1468,7 @@ void run_logits(tgx_ctx* c, const int* want_dev, int nw, float* C, const int* c_
   StackModel* sm = c->stack;
   const int W = sm->d.width, V = sm->d.vocab;
   if (sm->affine) hipLaunchKernelGGL(tgx::layer_norm_rows_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->final_norm, sm->final_norm + W, sm->xn, W, sm->d.norm_eps);
-  else if (sm->joint) hipLaunchKernelGGL(tgx::offset_norm_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->final_norm, 1.0f, sm->xn, W, sm->d.norm_eps);
+  else if (sm->joint || sm->post) hipLaunchKernelGGL(tgx::offset_norm_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->final_norm, sm->joint ? 1.0f : 0.0f, sm->xn, W, sm->d.norm_eps);
   else if (sm->sandwich) hipLaunchKernelGGL(tgx::scalar_norm_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->norm_g + 4 * (size_t)sm->d.layers, sm->xn, W, sm->d.norm_eps);
   else hipLaunchKernelGGL(tgx::final_norm_rows_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->final_norm, sm->xn, W, sm->d.norm_groups, sm->d.norm_eps);
   tgx::StackGemmArgs g{};
@@ -1513,17 +1827,19 @@ int stack_create(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int d
   if (!desc || !layers || !out_ctx) return set_err(nullptr, TGX_ERR_INVALID, "null argument");
   *out_ctx = nullptr;
   const tgx_stack_desc& d = *desc;
-  if (d.family != TGX_FAMILY_ZAKUSUN && d.family != TGX_FAMILY_MODEPEL && d.family != TGX_FAMILY_VITUDRA && d.family != TGX_FAMILY_ZALUVIK) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "family %d is not a layered model", d.family);
-  const bool sandwich = d.family == TGX_FAMILY_MODEPEL, joint = d.family == TGX_FAMILY_VITUDRA, affine = d.family == TGX_FAMILY_ZALUVIK;
+  if (d.family != TGX_FAMILY_ZAKUSUN && d.family != TGX_FAMILY_MODEPEL && d.family != TGX_FAMILY_VITUDRA && d.family != TGX_FAMILY_ZALUVIK && d.family != TGX_FAMILY_NUSOVIK) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "family %d is not a layered model", d.family);
+  const bool sandwich = d.family == TGX_FAMILY_MODEPEL, joint = d.family == TGX_FAMILY_VITUDRA, affine = d.family == TGX_FAMILY_ZALUVIK, post = d.family == TGX_FAMILY_NUSOVIK;
+  const bool latent = !sandwich && !joint && !affine && !post;
   if (d.width <= 0 || d.layers <= 0 || d.vocab <= 0 || d.max_seqs <= 0 || d.max_ctx <= 0) return set_err(nullptr, TGX_ERR_INVALID, "non-positive model dimension");
   if (d.compute_dtype != TGX_BF16 && d.compute_dtype != TGX_F16 && d.compute_dtype != TGX_F32) return set_err(nullptr, TGX_ERR_INVALID, "unknown compute dtype %d", d.compute_dtype);
   if (affine) { const int rc = check_affine_desc(d, layers); if (rc) return rc; }
-  if (!sandwich && !joint && !affine && (d.norm_groups < 1 || d.norm_groups > tgx::NORM_MAX_GROUPS || d.width % d.norm_groups)) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "norm groups %d: 1..%d, dividing the width", d.norm_groups, tgx::NORM_MAX_GROUPS);
-  if (!sandwich && !joint && !affine && (d.canon_taps < 1 || d.canon_taps > tgx::CONV_MAX_TAPS)) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "convolution taps %d: 1..%d", d.canon_taps, tgx::CONV_MAX_TAPS);
+  if (post) { const int rc = check_post_desc(d, layers); if (rc) return rc; }
+  if (latent && (d.norm_groups < 1 || d.norm_groups > tgx::NORM_MAX_GROUPS || d.width % d.norm_groups)) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "norm groups %d: 1..%d, dividing the width", d.norm_groups, tgx::NORM_MAX_GROUPS);
+  if (latent && (d.canon_taps < 1 || d.canon_taps > tgx::CONV_MAX_TAPS)) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "convolution taps %d: 1..%d", d.canon_taps, tgx::CONV_MAX_TAPS);
   int page = d.page_tokens > 0 ? d.page_tokens : 64;
   if (page & (page - 1)) return set_err(nullptr, TGX_ERR_INVALID, "page_tokens %d is not a power of two", page);
   int first_mix = -1;
-  for (int i = 0; i < d.layers && !affine; i++) {
+  for (int i = 0; i < d.layers && !affine && !post; i++) {
     const tgx_layer_desc& l = layers[i];
     if (joint) {
       auto attention_ok = [&](const char*& why) {
@@ -1601,8 +1917,8 @@ int stack_create(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int d
   while ((1 << sm->page_shift) < page) sm->page_shift++;
   // what the shared sampler / token rings read from the flat description
   c->d.family = d.family; c->d.hidden = d.width; c->d.layers = d.layers; c->d.vocab = d.vocab; c->d.max_ctx = d.max_ctx; c->d.max_batch = d.max_seqs;
-  c->d.compute_dtype = d.compute_dtype; c->d.tied = sandwich || joint ? 0 : 1; c->d.norm_eps = d.norm_eps;      // (a layer-norm design multiplies by the embedding table)
-  sm->sandwich = sandwich; sm->joint = joint; sm->affine = affine;
+  c->d.compute_dtype = d.compute_dtype; c->d.tied = sandwich || joint || post ? 0 : 1; c->d.norm_eps = d.norm_eps;      // (a layer-norm design multiplies by the embedding table)
+  sm->sandwich = sandwich; sm->joint = joint; sm->affine = affine; sm->post = post;
   c->device = device_ordinal;
   c->dt = d.compute_dtype == TGX_BF16 ? tgx::DT_BF16 : (d.compute_dtype == TGX_F16 ? tgx::DT_F16 : tgx::DT_F32);
   c->esz = d.compute_dtype == TGX_F32 ? 4 : 2;
@@ -1620,6 +1936,7 @@ int stack_create(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int d
   if (sandwich) return create_sandwich_layers(c, layers);
   if (joint) return create_joint_layers(c, layers);
   if (affine) return create_affine_layers(c, layers);
+  if (post) return create_post_layers(c, layers);
   for (int i = 0; i < d.layers; i++) {
     StackLayerW& w = sm->L[(size_t)i];
     w.d = layers[i];
@@ -1661,6 +1978,7 @@ int stack_upload(tgx_ctx* c, const char* name, const void* host, const int64_t* 
   if (sm->sandwich) return upload_sandwich(c, name, host, shape, nd, src_dtype);
   if (sm->joint) return upload_joint(c, name, host, shape, nd, src_dtype);
   if (sm->affine) return upload_affine(c, name, host, shape, nd, src_dtype);
+  if (sm->post) return upload_post(c, name, host, shape, nd, src_dtype);
   if (!strcmp(name, "embed")) { if (probe) return TGX_ERR_SHAPE; if (!is(d.vocab, W)) return bad_shape(); return done(upload_param_ext(c, c->embed, host, d.vocab * W, src_dtype)); }
   if (!strcmp(name, "final.norm")) { if (probe) return TGX_ERR_SHAPE; if (!is(W, -1)) return bad_shape(); return done(upload_f32(c, sm->final_norm, host, W, src_dtype)); }
   int li = -1;
@@ -1724,7 +2042,7 @@ int stack_finalize(tgx_ctx* c) {
   const size_t W = (size_t)d.width, B = (size_t)d.max_seqs, V = (size_t)d.vocab;
   int rc;
   // angles of the position vector: pos * base^(-2i / width), the factor rounded to fp32 once
-  if (!sm->sandwich && !sm->joint && !sm->affine) {
+  if (sm->latent() || sm->post) {
     std::vector<float> fq(W / 2 + 1);
     for (size_t i = 0; i < fq.size(); i++) fq[i] = (float)pow(10000.0, -2.0 * (double)i / (double)W);
     if ((rc = dev_alloc(c, &sm->freq, fq.size()))) return rc;
@@ -1740,7 +2058,7 @@ int stack_finalize(tgx_ctx* c) {
   memset(sm->tbl_host, 0, B * (size_t)sm->tbl_stride * 4);
   sm->row_pages.assign(B, 0); sm->row_par.assign(B, 0); sm->row_dirty.assign(B, 0);
   for (int p = sm->n_pages - 1; p >= 0; p--) sm->free_pages.push_back(p);
-  const size_t nb = sm->sandwich || sm->joint || sm->affine ? 0 : (size_t)d.canon_taps - 1;
+  const size_t nb = sm->latent() ? (size_t)d.canon_taps - 1 : 0;
   for (auto& r : sm->rot) {      // angle of (position, pair i) = position * base^(-2i / dims), evaluated in double, stored as fp32 cosine and sine
     const size_t half = (size_t)r.dims / 2;
     std::vector<float> cs((size_t)d.max_ctx * half * 2);
@@ -1776,6 +2094,29 @@ int stack_finalize(tgx_ctx* c) {
   }
   for (auto& w : sm->L) {
     if (sm->affine) break;
+    if (sm->post) {
+      const tgx_layer_desc& l = w.d;
+      const bool par = l.mixer == TGX_MIXER_PARALLEL;
+      const size_t C = par ? (size_t)l.d_heads * l.d_vdim + 2 * (size_t)l.d_kv_heads * l.d_dim : (size_t)l.inner, ce = 2 * B * (size_t)(l.conv_taps - 1) * C;
+      const size_t se = B * (par ? (size_t)l.d_heads * l.d_dim * l.d_vdim : (size_t)l.inner * l.d_dim);
+      if ((rc = dev_alloc(c, &w.mS, se))) return rc;
+      HIP_OK(c, hipMemset(w.mS, 0, se * 4));
+      if (ce > 0) {
+        if ((rc = dev_alloc(c, &w.conv_state, ce))) return rc;
+        HIP_OK(c, hipMemset(w.conv_state, 0, ce * 4));
+      }
+      if (par) {      // keys and values of the attention half
+        const size_t ke = (size_t)sm->n_pages * sm->page * (size_t)l.kv_heads * l.dim * c->esz;
+        if ((rc = dev_alloc(c, &w.pool, ke)) || (rc = dev_alloc(c, &w.poolV, ke))) return rc;
+        HIP_OK(c, hipMemset(w.pool, 0, ke));
+        HIP_OK(c, hipMemset(w.poolV, 0, ke));
+        if (gqa_mfma_shapes_ok(c->dt, l.dim, l.vdim, sm->page_shift, 4)) {      // (the projections' row stride is a multiple of four)
+          if ((rc = dev_alloc(c, &w.poolVT, ke))) return rc;
+          HIP_OK(c, hipMemset(w.poolVT, 0, ke));
+        }
+      }
+      continue;
+    }
     if (sm->joint) {
       const tgx_layer_desc& l = w.d;
       if (l.mixer != TGX_MIXER_WKV && w.kv_src < 0) {      // keys and values of an attention layer / a parallel mixer's attention half (a sharing layer borrows below)
@@ -1888,6 +2229,7 @@ void stack_destroy(tgx_ctx* c) {
   auto fr = [](void* p) { if (p) (void)hipFree(p); };
   for (auto& w : sm->L) {
     if (w.kv_src >= 0) w.pool = w.poolV = w.poolVT = nullptr;      // borrowed
+    fr(w.conv_b); fr(w.d_skip); fr(w.decay2); fr(w.q_norm); fr(w.k_norm); fr(w.dist);
     fr(w.w_o2); fr(w.w_w1); fr(w.w_w2); fr(w.mu); fr(w.w0); fr(w.ubonus); fr(w.conv_w); fr(w.a_log); fr(w.dt_bias); fr(w.shift);
     fr(w.norm1); fr(w.norm2); fr(w.canon1); fr(w.canon2); fr(w.dwa); fr(w.w_in); fr(w.w_ukT); fr(w.w_uv); fr(w.w_o); fr(w.lat_norm); fr(w.sink);
     fr(w.w_gate); fr(w.w_up); fr(w.w_down); fr(w.w_router); fr(w.b_router); fr(w.pool); fr(w.poolT); fr(w.conv_state);
@@ -2057,9 +2399,9 @@ int stack_read_latent(tgx_ctx* c, int row, int layer, float* out) {
   if (row < 0 || row >= sm->d.max_seqs || layer < 0 || layer >= sm->d.layers || !out) return set_err(c, TGX_ERR_INVALID, "read_kv: row / layer out of range");
   HIP_OK(c, hipStreamSynchronize(c->stream));
   const StackLayerW& w = sm->L[(size_t)layer];
-  if ((sm->sandwich && w.d.mixer != TGX_MIXER_ATTENTION) || (sm->joint && !w.pool)) return set_err(c, TGX_ERR_UNSUPPORTED, "read_kv: layer %d caches no rows (its state is recurrent)", layer);
+  if ((sm->sandwich && w.d.mixer != TGX_MIXER_ATTENTION) || ((sm->joint || sm->post) && !w.pool)) return set_err(c, TGX_ERR_UNSUPPORTED, "read_kv: layer %d caches no rows (its state is recurrent)", layer);
   const ebyte* pool = w.pool;
-  size_t R = sm->sandwich || sm->joint ? (size_t)w.d.kv_heads * w.d.dim : (size_t)w.d.kv_rank;      // an attention layer's cached keys, all key heads of a token in a row
+  size_t R = sm->sandwich || sm->joint || sm->post ? (size_t)w.d.kv_heads * w.d.dim : (size_t)w.d.kv_rank;      // an attention layer's cached keys, all key heads of a token in a row
   if (sm->affine) {      // the cache of the layer's first run: an attention layer's keys, a latent layer's rows [latent | rotated key part]
     for (const StackRun& r : sm->runs) if (r.layer == layer) { pool = r.pool; break; }
     R = w.d.mixer == TGX_MIXER_ATTENTION ? (size_t)w.d.kv_heads * w.d.dim : (size_t)(w.d.kv_rank + w.d.rot_dim);
@@ -2079,7 +2421,7 @@ int64_t stack_bytes_per_token(const tgx_ctx* c, int64_t T) {
   const StackModel* sm = c->stack;
   const int64_t W = sm->d.width, es = (int64_t)c->esz;
   int64_t b = (int64_t)sm->d.vocab * W * es;
-  if (sm->sandwich || sm->joint) b *= 2;      // embedding row aside, the head is a matrix of its own
+  if (sm->sandwich || sm->joint || sm->post) b *= 2;      // embedding row aside, the head is a matrix of its own
   if (sm->affine) {      // per run of a layer: its matrices (the chosen experts only) and the rows of its cache inside the mask's span
     if (sm->w_loop) b += (int64_t)sm->d.loop_times * 2 * W * W * es;
     for (const StackRun& r : sm->runs) {
@@ -2095,6 +2437,15 @@ int64_t stack_bytes_per_token(const tgx_ctx* c, int64_t T) {
   for (const auto& w : sm->L) {
     const tgx_layer_desc& l = w.d;
     const int64_t H = l.heads, qd = H * l.dim, R = l.kv_rank, vd = H * l.vdim;
+    if (sm->post) {      // the convolution tails are small beside a state, which is read and written
+      if (l.mixer == TGX_MIXER_MAMBA1) b += ((int64_t)l.inner * (3 * W + 2 * l.dt_rank + 2 * l.d_dim)) * es + 3 * (int64_t)l.inner * l.d_dim * 4;
+      else {
+        const int64_t I = (int64_t)l.d_heads * l.d_vdim, gn = (int64_t)l.d_kv_heads * l.d_dim, keys = l.mask_kind ? std::min<int64_t>(T, l.mask_size) : T;
+        b += ((qd + (int64_t)l.kv_heads * l.dim + 2 * I + 2 * gn + l.d_heads + H) * W + W * (vd + I)) * es + keys * 2 * l.kv_heads * l.dim * es + 2 * I * l.d_dim * 4;
+      }
+      if (l.mlp == TGX_MLP_DENSE) b += 2 * (int64_t)l.ff * W * es;
+      continue;
+    }
     if (sm->joint) {      // an attention layer reads at most its mask's span of keys; a recurrent state is read and written
       const int64_t keys = l.mask_kind ? std::min<int64_t>(T, l.mask_size) : T, kvw = (int64_t)l.kv_heads * (l.dim + l.vdim);
       if (l.mixer == TGX_MIXER_ATTENTION) b += ((qd + (w.kv_src >= 0 ? 0 : kvw)) * W + W * vd) * es + keys * kvw * es;

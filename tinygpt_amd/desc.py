@@ -272,13 +272,15 @@ FAMILY_ZAKUSUN = 6
 FAMILY_MODEPEL = 7
 FAMILY_VITUDRA = 8
 FAMILY_ZALUVIK = 9
-STACK_FAMILY = {"zakusun": FAMILY_ZAKUSUN, "modepel": FAMILY_MODEPEL, "vitudra": FAMILY_VITUDRA, "zaluvik": FAMILY_ZALUVIK}
-MIXER_BY_NAME = {"latent_attention": 1, "attention": 2, "mlstm": 3, "wkv": 4, "parallel": 5}
+FAMILY_NUSOVIK = 10
+STACK_FAMILY = {"zakusun": FAMILY_ZAKUSUN, "modepel": FAMILY_MODEPEL, "vitudra": FAMILY_VITUDRA, "zaluvik": FAMILY_ZALUVIK,
+                "nusovik": FAMILY_NUSOVIK}
+MIXER_BY_NAME = {"latent_attention": 1, "attention": 2, "mlstm": 3, "wkv": 4, "parallel": 5, "mamba1": 6}
 MLP_BY_NAME = {None: 0, "moe": 1, "dense": 2}
 MASK_BY_NAME = {None: 0, "window": 1, "chunk": 2}
 # which mixers a design is made of (config.json "architecture" -> layer "type")
 MIXERS_OF = {"zakusun": ("latent_attention",), "modepel": ("attention", "mlstm"), "vitudra": ("attention", "wkv", "parallel"),
-             "zaluvik": ("attention", "latent_attention")}
+             "zaluvik": ("attention", "latent_attention"), "nusovik": ("mamba1", "parallel")}
 
 
 class CLayerDesc(ctypes.Structure):
@@ -296,7 +298,9 @@ class CLayerDesc(ctypes.Structure):
                 ("right_scale", ctypes.c_float),
                 ("qk_norm", ctypes.c_int32), ("score_fn", ctypes.c_int32), ("head_mix", ctypes.c_int32), ("gate_kind", ctypes.c_int32),
                 ("rot_dim", ctypes.c_int32), ("ff_act", ctypes.c_int32), ("router_fn", ctypes.c_int32), ("group_score", ctypes.c_int32),
-                ("router_norm", ctypes.c_int32)]
+                ("router_norm", ctypes.c_int32),
+                ("v_is_k", ctypes.c_int32), ("head_sink", ctypes.c_int32), ("bias_max", ctypes.c_int32), ("bias_buckets", ctypes.c_int32),
+                ("right_kind", ctypes.c_int32), ("part_norms", ctypes.c_int32), ("inner", ctypes.c_int32), ("dt_rank", ctypes.c_int32)]
 
 
 class CStackDesc(ctypes.Structure):
@@ -356,15 +360,25 @@ class LayerDesc:
     right_scale: float = 1.0
     # the layer-norm design (Zaluvik): unit queries and keys, sigmoid weights mixed across heads, the kind of output gate, the rotated part of a
     # latent layer's queries and keys, the dense feed-forward's activation, the sigmoid router
-    qk_norm: bool = False
+    qk_norm: "bool | str" = False     # True: unit; "weighted": times a learned vector
     score_fn: "str | None" = None     # None: softmax; "sigmoid": sigmoid(score + per-head bias), not normalised over the keys
     head_mix: bool = False
     gate_kind: "str | None" = None    # None: the family's own; "channel" | "head"
     rot_dim: int = 0
-    ff_act: "str | None" = None       # None: the family's own; "gelu"
+    ff_act: "str | None" = None       # None: the family's own; "gelu" | "relu2"
     router_fn: "str | None" = None    # None: softmax + correction; "sigmoid"
     group_score: "str | None" = None  # None: a group's largest score; "top2": the sum of its two largest
     router_norm: bool = False
+    # the output-norm design (Nusovik): keys as values, sinks, bucketed distance bias; the kind of a parallel mixer's right half (d_heads heads of d_vdim values
+    # over d_kv_heads groups of d_dim state numbers for "ssd"); the selective scan of a "mamba1" mixer (a state of d_dim numbers per channel)
+    v_is_k: bool = False
+    head_sink: bool = False
+    bias_max: int = 0
+    bias_buckets: int = 0             # rows of the distance table (0: the table's own)
+    right_kind: "str | None" = None   # None: the gated delta rule; "ssd"
+    part_norms: int = 1
+    inner: int = 0
+    dt_rank: int = 0
 
     def to_c(self) -> CLayerDesc:
         return CLayerDesc(MIXER_BY_NAME[self.mixer], self.heads, self.dim, self.vdim, self.kv_rank, self.scale,
@@ -374,9 +388,10 @@ class LayerDesc:
                           MASK_BY_NAME[self.mask], self.mask_size, self.softcap, int(self.dist_bias), self.q_temp_coef, self.q_temp_every,
                           int(self.rot_pairs), self.rot_factor, 0 if self.kv_from is None else self.kv_from + 1, self.decay_rank,
                           self.d_heads, self.d_kv_heads, self.d_dim, self.d_vdim, self.conv_taps, self.left_scale, self.right_scale,
-                          int(self.qk_norm), {None: 0, "sigmoid": 1}[self.score_fn], int(self.head_mix), {None: 0, "channel": 1, "head": 2}[self.gate_kind],
-                          self.rot_dim, {None: 0, "gelu": 1}[self.ff_act], {None: 0, "sigmoid": 1}[self.router_fn], {None: 0, "top2": 1}[self.group_score],
-                          int(self.router_norm))
+                          2 if self.qk_norm == "weighted" else int(self.qk_norm), {None: 0, "sigmoid": 1}[self.score_fn], int(self.head_mix), {None: 0, "channel": 1, "head": 2}[self.gate_kind],
+                          self.rot_dim, {None: 0, "gelu": 1, "relu2": 2}[self.ff_act], {None: 0, "sigmoid": 1}[self.router_fn], {None: 0, "top2": 1}[self.group_score],
+                          int(self.router_norm), int(self.v_is_k), int(self.head_sink), self.bias_max, self.bias_buckets,
+                          {None: 0, "ssd": 1}[self.right_kind], self.part_norms, self.inner, self.dt_rank)
 
 
 @dataclass
@@ -396,7 +411,7 @@ class StackDesc:
     canon_taps: int = 1
     logit_scale: float = 1.0
     residual_mult: float = 1.0   # Vitudra, Zaluvik: the factor on what a (sub)layer adds to the stream
-    embed_scale: float = 1.0     # Zaluvik: the factor on the embedding rows
+    embed_scale: float = 1.0     # Zaluvik, Nusovik: the factor on the embedding rows
     loop_start: int = 0          # Zaluvik: layers loop_start .. loop_stop - 1 run loop_times times with the same weights, a cache per pass
     loop_stop: int = 0
     loop_times: int = 1
@@ -438,6 +453,8 @@ class StackDesc:
             return _vitudra_shapes(self, out)
         if self.family == "zaluvik":
             return _zaluvik_shapes(self, out)
+        if self.family == "nusovik":
+            return _nusovik_shapes(self, out)
         for i, l in enumerate(self.layers):
             p = f"l{i}."
             out[p + "norm1"] = (W,)
@@ -555,6 +572,56 @@ def _zaluvik_shapes(self: StackDesc, out: dict) -> dict:
     return out
 
 
+def _nusovik_shapes(self: StackDesc, out: dict) -> dict:
+    """checkpoint names and shapes of a Nusovik model, in file order"""
+    W = self.width
+    for i, l in enumerate(self.layers):
+        p = f"l{i}."
+        out[p + "norm1"] = (W,)
+        if l.mlp:
+            out[p + "norm2"] = (W,)
+        if l.mixer == "mamba1":
+            q, I, N = p + "mix.", l.inner, l.d_dim
+            out[q + "in"] = (2 * I, W); out[q + "conv"] = (I, l.conv_taps); out[q + "conv.b"] = (I,); out[q + "x"] = (l.dt_rank + 2 * N, I)
+            out[q + "dt"] = (I, l.dt_rank); out[q + "dt.b"] = (I,); out[q + "A_log"] = (I, N); out[q + "D"] = (I,); out[q + "o"] = (W, I)
+        else:
+            q, qd, kd = p + "mix.left.", l.heads * l.dim, l.kv_heads * l.dim
+            out[q + "q"] = (qd, W); out[q + "q.b"] = (qd,); out[q + "k"] = (kd, W); out[q + "k.b"] = (kd,); out[q + "q.norm"] = (l.dim,); out[q + "k.norm"] = (l.dim,)
+            out[q + "rel"] = (l.bias_buckets, l.heads); out[q + "sink"] = (l.heads,); out[q + "g"] = (l.heads, W); out[q + "o"] = (W, l.heads * l.vdim)
+            q, I, C = p + "mix.right.", l.d_heads * l.d_vdim, l.d_heads * l.d_vdim + 2 * l.d_kv_heads * l.d_dim
+            out[q + "in"] = (I + C + l.d_heads, W); out[q + "conv"] = (C, l.conv_taps); out[q + "conv.b"] = (C,); out[q + "dt_bias"] = (l.d_heads,)
+            out[q + "A_log"] = (l.d_heads,); out[q + "D"] = (l.d_heads,); out[q + "norm"] = (I,); out[q + "o"] = (W, I)
+        if l.mlp == "dense":
+            out[p + "mlp.up"] = (l.ff, W); out[p + "mlp.down"] = (W, l.ff)
+    out["final.norm"] = (W,)
+    out["head"] = (self.vocab, W)
+    return out
+
+
+def _nusovik_layer(i: int, l: dict, buckets: int = 0) -> LayerDesc:
+    """one entry of a Nusovik config's "layers": {"type": "mamba1" | "parallel", "mixer": {...}, "mlp": null | {"kind": "dense", "ff"}}.
+    A parallel mixer is {"left": chunked attention whose values are its keys, with a bucketed distance bias, sinks and a gate per head, "right": a scalar-decay
+    state-space mixer, "left_scale", "right_scale"}."""
+    m, f = l["mixer"], l.get("mlp")
+    ld = LayerDesc(mixer=l["type"])
+    if l["type"] == "mamba1":
+        ld.inner = int(m["inner"]); ld.d_dim = int(m["state"]); ld.dt_rank = int(m["dt_rank"]); ld.conv_taps = int(m.get("conv", 1))
+    else:
+        a, r = m["left"], m["right"]
+        ld.heads = int(a["heads"]); ld.kv_heads = int(a.get("kv_heads", a["heads"])); ld.dim = int(a["dim"]); ld.vdim = int(a.get("vdim", a["dim"])); ld.scale = float(a["scale"])
+        if a.get("mask"):
+            ld.mask = "chunk"; ld.mask_size = int(a["mask"]["size"])
+        ld.qk_norm = "weighted"; ld.v_is_k = True; ld.head_sink = True; ld.gate_kind = "head"; ld.bias_max = int(a["bias_max"]); ld.bias_buckets = int(buckets)
+        ld.right_kind = "ssd"; ld.d_heads = int(r["heads"]); ld.d_kv_heads = int(r.get("groups", 1)); ld.d_dim = int(r["state"]); ld.d_vdim = int(r["vdim"])
+        ld.conv_taps = int(r.get("conv", 1)); ld.part_norms = int(r.get("norm_groups", 1))
+        ld.left_scale = float(m.get("left_scale", 1.0)); ld.right_scale = float(m.get("right_scale", 1.0))
+    if f is not None:
+        if f.get("kind") != "dense":
+            raise ValueError(f"layer {i}: feed-forward kind {f.get('kind')!r} is not implemented")
+        ld.mlp = "dense"; ld.ff = int(f["ff"]); ld.ff_act = "relu2"
+    return ld
+
+
 def _zaluvik_layer(i: int, l: dict) -> LayerDesc:
     """one entry of a Zaluvik config's "layers": {"type": "attention" | "latent_attention", "mixer": {...}, "mlp": null | {"kind": "dense" | "moe", ...}}.
     Attention: unit queries and keys, a sliding window, sigmoid weights with a per-head bias mixed across heads, a gate per output channel.
@@ -651,8 +718,8 @@ def _modepel_layer(i: int, l: dict) -> LayerDesc:
 
 
 def stack_desc_from_config(cfg: dict, compute_dtype: str = "bf16", max_seqs: int = 4, max_ctx: int = 4096, budget_tokens: int = 0, tensor_shapes=None) -> StackDesc:
-    """config.json of a layered model ("architecture": "Zakusun" | "Modepel" | "Vitudra" | "Zaluvik") -> StackDesc.  Every size and constant comes from the file;
-    tensor_shapes (checkpoint name -> shape, optional) gives the sizes that only a tensor's shape tells (a wkv layer's decay rank; left open without it:
+    """config.json of a layered model ("architecture": "Zakusun" | "Modepel" | "Vitudra" | "Zaluvik" | "Nusovik") -> StackDesc.  Every size and constant comes from the file;
+    tensor_shapes (checkpoint name -> shape, optional) gives the sizes that only a tensor's shape tells (a wkv layer's decay rank, the rows of a distance table; left open without it:
     the device library then takes it from the tensor at upload)."""
     arch = str(cfg.get("architecture")).lower()
     if arch not in MIXERS_OF:
@@ -673,6 +740,12 @@ def stack_desc_from_config(cfg: dict, compute_dtype: str = "bf16", max_seqs: int
                          norm_eps=float(cfg["norm"]["eps"]), canon_taps=1, logit_scale=1.0, residual_mult=float(cfg.get("residual_mult", 1.0)),
                          embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), loop_start=int(lp.get("start", 0)), loop_stop=int(lp.get("stop", 0)),
                          loop_times=int(lp.get("times", 1)), name="zaluvik")
+    if arch == "nusovik":
+        ts = tensor_shapes or {}
+        return StackDesc(family="nusovik", width=int(cfg["width"]), vocab=int(cfg["vocab"]),
+                         layers=[_nusovik_layer(i, l, (ts.get(f"l{i}.mix.left.rel") or (0,))[0]) for i, l in enumerate(cfg["layers"])], compute_dtype=compute_dtype,
+                         max_seqs=max_seqs, max_ctx=max_ctx, budget_tokens=budget_tokens, norm_groups=1, norm_eps=float(cfg["norm"]["eps"]), canon_taps=1,
+                         logit_scale=float(cfg.get("logit_scale", 1.0)), embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), name="nusovik")
     if arch == "modepel":
         return StackDesc(family="modepel", width=int(cfg["width"]), vocab=int(cfg["vocab"]), layers=[_modepel_layer(i, l) for i, l in enumerate(cfg["layers"])],
                          compute_dtype=compute_dtype, max_seqs=max_seqs, max_ctx=max_ctx, budget_tokens=budget_tokens, norm_groups=1,

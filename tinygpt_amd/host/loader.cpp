@@ -184,26 +184,61 @@ static bool load_zaluvik_layer(const Json& L, size_t i, tgx_layer_desc& l, std::
   return true;
 }
 
+// one entry of a Nusovik config's "layers": {"type": "mamba1" | "parallel", "mixer": {...}, "mlp": null | {"kind": "dense", "ff"}}.  A parallel mixer is
+// {"left": chunked attention whose values are its keys, with a bucketed distance bias, sinks and a gate per head, "right": scalar-decay state-space mixer,
+// "left_scale", "right_scale"}.  The rows of a distance table are left open: the device library takes them from the tensor's shape.
+static bool load_nusovik_layer(const Json& L, size_t i, tgx_layer_desc& l, std::string& err) {
+  auto dim = [](const Json& j, const char* key) -> int32_t { const int64_t v = j.get_int(key, -1); return (v < 0 || v > ((int64_t)1 << 30)) ? -1 : (int32_t)v; };
+  const Json* mx = L.get("mixer");
+  const Json* ff = L.get("mlp");
+  const std::string type = L.get_str("type", "");
+  auto bad = [&](const std::string& what) { err = "config.json: layer " + std::to_string(i) + ": " + what; return false; };
+  if (!mx || mx->kind != Json::Obj) return bad("no mixer");
+  if (type == "mamba1") {
+    l.mixer = TGX_MIXER_MAMBA1;
+    l.inner = dim(*mx, "inner"); l.d_dim = dim(*mx, "state"); l.dt_rank = dim(*mx, "dt_rank"); l.conv_taps = mx->has("conv") ? dim(*mx, "conv") : 1;
+  } else if (type == "parallel") {
+    const Json* left = mx->get("left");
+    const Json* right = mx->get("right");
+    if (!left || left->kind != Json::Obj || !right || right->kind != Json::Obj) return bad("a parallel mixer needs left and right");
+    l.mixer = TGX_MIXER_PARALLEL;
+    l.heads = dim(*left, "heads"); l.kv_heads = left->has("kv_heads") ? dim(*left, "kv_heads") : l.heads; l.dim = dim(*left, "dim");
+    l.vdim = left->has("vdim") ? dim(*left, "vdim") : l.dim; l.scale = left->get_float("scale", 1.f);
+    const Json* mask = left->get("mask");
+    if (mask && mask->kind == Json::Obj) { l.mask_kind = TGX_MASK_CHUNK; l.mask_size = dim(*mask, "size"); }
+    l.qk_norm = 2; l.v_is_k = 1; l.head_sink = 1; l.gate_kind = 2; l.bias_max = dim(*left, "bias_max");
+    l.right_kind = 1; l.d_heads = dim(*right, "heads"); l.d_kv_heads = right->has("groups") ? dim(*right, "groups") : 1; l.d_dim = dim(*right, "state");
+    l.d_vdim = dim(*right, "vdim"); l.conv_taps = right->has("conv") ? dim(*right, "conv") : 1; l.part_norms = right->has("norm_groups") ? dim(*right, "norm_groups") : 1;
+    l.left_scale = mx->get_float("left_scale", 1.f); l.right_scale = mx->get_float("right_scale", 1.f);
+  } else return bad("mixer '" + type + "' is not implemented");
+  if (!ff || ff->kind != Json::Obj) return true;
+  if (ff->get_str("kind", "") != "dense") return bad("feed-forward kind '" + ff->get_str("kind", "") + "' is not implemented");
+  l.mlp = TGX_MLP_DENSE; l.ff = dim(*ff, "ff"); l.ff_act = 2;
+  return true;
+}
+
 // config.json of a layered model: {"architecture": "Zakusun", "width", "vocab", "logit_scale", "norm": {"eps", "groups"}, "canon": {"taps"},
 // "layers": [{"type": mixer, "mixer": {heads, dim, vdim, kv_rank, scale}, "mlp": null | {"kind": "moe", "expert": {ff, limit}, "router": {experts, top}}}]}
 // or {"architecture": "Modepel", "width", "vocab", "norm": {"eps"}, "layers": [...]} with the layer entries of load_modepel_layer
 // or {"architecture": "Vitudra", "width", "vocab", "residual_mult", "norm": {"eps"}, "layers": [...]} with the layer entries of load_vitudra_layer
 // or {"architecture": "Zaluvik", "width", "vocab", "residual_mult", "embedding": {"scale"}, "loop": {"start", "stop", "times"}, "norm": {"eps"}, "layers": [...]}
 // with the layer entries of load_zaluvik_layer (logits against the embedding table)
+// or {"architecture": "Nusovik", "width", "vocab", "logit_scale", "embedding": {"scale"}, "norm": {"eps"}, "layers": [...]} with the layer entries of
+// load_nusovik_layer
 static bool load_stack_config(const Json& doc, const std::string& path, int compute_dtype, int max_batch, int max_ctx, int budget_tokens, ModelConfig& out, std::string& err) {
   const std::string arch = doc.get_str("architecture", "");
-  const bool vitudra = arch == "Vitudra", zaluvik = arch == "Zaluvik", modepel = arch == "Modepel" || vitudra || zaluvik;      // (all three: a config header without norm groups, taps and logit scale)
+  const bool vitudra = arch == "Vitudra", zaluvik = arch == "Zaluvik", nusovik = arch == "Nusovik", modepel = arch == "Modepel" || vitudra || zaluvik || nusovik;      // (all four: a config header without norm groups and taps)
   if (arch != "Zakusun" && !modepel) { err = "Unsupported architecture: " + arch; return false; }
   auto dim = [](const Json& j, const char* key) -> int32_t { const int64_t v = j.get_int(key, -1); return (v < 0 || v > ((int64_t)1 << 30)) ? -1 : (int32_t)v; };
   out.layered = true;
-  out.model_type = zaluvik ? "zaluvik" : vitudra ? "vitudra" : modepel ? "modepel" : "zakusun";
+  out.model_type = nusovik ? "nusovik" : zaluvik ? "zaluvik" : vitudra ? "vitudra" : modepel ? "modepel" : "zakusun";
   tgx_stack_desc& s = out.stack;
-  s.family = zaluvik ? TGX_FAMILY_ZALUVIK : vitudra ? TGX_FAMILY_VITUDRA : modepel ? TGX_FAMILY_MODEPEL : TGX_FAMILY_ZAKUSUN;
+  s.family = nusovik ? TGX_FAMILY_NUSOVIK : zaluvik ? TGX_FAMILY_ZALUVIK : vitudra ? TGX_FAMILY_VITUDRA : modepel ? TGX_FAMILY_MODEPEL : TGX_FAMILY_ZAKUSUN;
   s.residual_mult = doc.get_float("residual_mult", 1.f);
   s.embed_scale = 1.f; s.loop_times = 1;
+  const Json* em = doc.get("embedding");
+  if ((zaluvik || nusovik) && em && em->kind == Json::Obj) s.embed_scale = em->get_float("scale", 1.f);
   if (zaluvik) {
-    const Json* em = doc.get("embedding");
-    if (em && em->kind == Json::Obj) s.embed_scale = em->get_float("scale", 1.f);
     const Json* lp = doc.get("loop");
     if (lp && lp->kind == Json::Obj) { s.loop_start = dim(*lp, "start"); s.loop_stop = dim(*lp, "stop"); s.loop_times = dim(*lp, "times"); }
   }
@@ -212,7 +247,7 @@ static bool load_stack_config(const Json& doc, const std::string& path, int comp
   s.max_ctx = max_ctx > 0 ? max_ctx : 4096;
   s.budget_tokens = budget_tokens > 0 ? budget_tokens : 0;
   s.page_tokens = 0;
-  s.logit_scale = modepel ? 1.f : doc.get_float("logit_scale", 1.f);
+  s.logit_scale = modepel && !nusovik ? 1.f : doc.get_float("logit_scale", 1.f);
   const Json* norm = doc.get("norm");
   const Json* canon = doc.get("canon");
   const Json* layers = doc.get("layers");
@@ -224,7 +259,7 @@ static bool load_stack_config(const Json& doc, const std::string& path, int comp
     const Json& L = layers->arr[i];
     tgx_layer_desc l{};
     if (modepel) {
-      if (!(zaluvik ? load_zaluvik_layer(L, i, l, err) : vitudra ? load_vitudra_layer(L, i, l, err) : load_modepel_layer(L, i, l, err))) return false;
+      if (!(nusovik ? load_nusovik_layer(L, i, l, err) : zaluvik ? load_zaluvik_layer(L, i, l, err) : vitudra ? load_vitudra_layer(L, i, l, err) : load_modepel_layer(L, i, l, err))) return false;
       out.layers.push_back(l);
       continue;
     }
