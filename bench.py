@@ -84,7 +84,7 @@ def parse():
     ap.add_argument("--layered", default=None, metavar="SIZE[,SIZE]", help="instead of the headline: prefill and decode throughput of the layered (Zakusun) design at "
                     "layer sizes of real models (1b, 0.5b; random weights), beside a Llama-family model of the same width, depth and active parameters")
     ap.add_argument("--only", default="", help="with --layered: measure these models only (names before the size, with commas; for profiling one of them)")
-    ap.add_argument("--design", default="zakusun", choices=["zakusun", "modepel", "vitudra", "zaluvik"], help="with --layered: which layered design is measured beside its closest relatives and the Llama-family model")
+    ap.add_argument("--design", default="zakusun", choices=["zakusun", "modepel", "vitudra", "zaluvik", "nusovik"], help="with --layered: which layered design is measured beside its closest relatives and the Llama-family model")
     ap.add_argument("--cpu-seconds", type=float, default=15.0, help="target CPU time of the cpu_baseline sample")
     return ap.parse_args()
 
@@ -382,6 +382,24 @@ def zaluvik_desc(key, z, L, V, dtype, B, ctx):
                      embed_scale=3.0, loop_start=1, loop_stop=3, loop_times=2, name=f"zaluvik-{key}", layers=layers)
 
 
+def nusovik_desc(key, z, L, V, dtype, B, ctx):
+    """Nusovik at the size of `z`: selective-scan layers (twice the width in channels, 16 state numbers each) and parallel layers (chunked attention with keys as
+    values beside a scalar-decay state-space mixer of twice the width, 128 state numbers) in turn; a squared-relu feed-forward behind every parallel mixer"""
+    from tinygpt_amd.desc import LayerDesc, StackDesc
+    W = z["width"]
+    layers = []
+    for i in range(L):
+        if i % 2 == 0:
+            l = LayerDesc(mixer="mamba1", inner=2 * W, d_dim=16, dt_rank=W // 16, conv_taps=4)
+        else:
+            l = LayerDesc(mixer="parallel", heads=W // 128, kv_heads=max(1, W // 512), dim=128, vdim=128, scale=128 ** -0.5, mask="chunk", mask_size=1024, qk_norm="weighted",
+                          v_is_k=True, head_sink=True, gate_kind="head", bias_max=1024, bias_buckets=32, right_kind="ssd", d_heads=2 * W // 64, d_kv_heads=max(1, W // 1024),
+                          d_dim=128, d_vdim=64, conv_taps=4, part_norms=max(1, W // 1024), left_scale=0.7, right_scale=0.9, mlp="dense", ff=z["top"] * z["ff"], ff_act="relu2")
+        layers.append(l)
+    return StackDesc(family="nusovik", width=W, vocab=V, compute_dtype=dtype, max_seqs=B, max_ctx=ctx, budget_tokens=B * (ctx + 64), norm_eps=1e-5, logit_scale=1.0, embed_scale=2.0,
+                     name=f"nusovik-{key}", layers=layers)
+
+
 def layered_compare(args):
     from tinygpt_amd.desc import LayerDesc, ModelDesc, StackDesc
     from tinygpt_amd.ffi import GREEDY, Model
@@ -429,7 +447,8 @@ def layered_compare(args):
                        inter=z["llama"]["inter"], vocab=V, max_ctx=ctx, tied=True, compute_dtype=args.dtype, norm_eps=1e-5, rope_theta=500000.0, max_batch=B, name=f"llama-{key}")
         todo = {"zakusun": [(sd, True)], "modepel": [(modepel_desc(key, z, L, V, args.dtype, B, ctx), True), (sd, True)],
                 "vitudra": [(vitudra_desc(key, z, L, V, args.dtype, B, ctx), True), (modepel_desc(key, z, L, V, args.dtype, B, ctx), True)],
-                "zaluvik": [(zaluvik_desc(key, z, L, V, args.dtype, B, ctx), True), (modepel_desc(key, z, L, V, args.dtype, B, ctx), True), (sd, True)]}[args.design] + [(ld, False)]
+                "zaluvik": [(zaluvik_desc(key, z, L, V, args.dtype, B, ctx), True), (modepel_desc(key, z, L, V, args.dtype, B, ctx), True), (sd, True)],
+                "nusovik": [(nusovik_desc(key, z, L, V, args.dtype, B, ctx), True), (vitudra_desc(key, z, L, V, args.dtype, B, ctx), True)]}[args.design] + [(ld, False)]
         if args.only:
             todo = [t for t in todo if t[0].name.split("-")[0] in args.only.split(",")]
         for desc, layered in todo:

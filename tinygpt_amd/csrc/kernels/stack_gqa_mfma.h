@@ -116,7 +116,14 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
     }
     float db[8];      // the distance table's entries of this lane's eight keys (loaded ahead of the products that hide them)
 #pragma unroll
-    for (int c = 0; c < 8; c++) db[c] = dist ? dist[min(max(skeys - 1 - (kt + kq + c), 0), a.dist_len - 1)] * LOG2E : 0.f;
+    for (int c = 0; c < 8; c++) db[c] = 0.f;
+    if (dist) {
+      typedef float run4 __attribute__((ext_vector_type(4), aligned(4)));
+      const int at = min(max(a.dist_len - 1 - DIST_PAD - (skeys - 1 - (kt + kq)), 0), a.dist_len - DIST_PAD);      // (a run behind the row's position is masked, whatever it reads)
+      const run4 d0 = *reinterpret_cast<const run4*>(dist + at), d1 = *reinterpret_cast<const run4*>(dist + at + 4);
+#pragma unroll
+      for (int c = 0; c < 4; c++) { db[c] = d0[c] * LOG2E; db[4 + c] = d1[c] * LOG2E; }
+    }
     // 1. partial scores over this wave's channels, keys kt .. kt + 31 and kt + 32 .. kt + 63
     f32x16 s[2];
 #pragma unroll

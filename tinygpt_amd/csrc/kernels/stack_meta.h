@@ -28,4 +28,8 @@ __device__ __forceinline__ int first_key(int pos, int kind, int size) {
 // the distance bias of head h of `heads`: scores lose slope * (i - j)
 __device__ __forceinline__ float distance_slope(int h, int heads) { return exp2f(-8.0f * (float)(h + 1) / (float)heads); }
 
+// a distance table's rows (GqaAttnArgs::dist_tab) end in this many entries behind distance 0 and begin with as many equal ones, so that the entries of eight neighbouring
+// keys are one run of memory wherever they lie
+constexpr int DIST_PAD = 8;
+
 }  // namespace tgx

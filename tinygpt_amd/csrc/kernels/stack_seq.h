@@ -6,6 +6,7 @@
 //   sandwich_kernel         x += norm_b(sublayer output) and the next sublayer's normed input, the experts' combine folded in
 //   poly_norm_kernel        a N(z) + b N(z^2) + c N(z^3) + e over a token's feed-forward values
 //   gqa_append_kernel       rotary positions on q (in place) and k, value mixing, store of k / v into the token's place in the pool
+//   key_value_append_kernel normed q (in place) and k, the un-normed k as values, store into the pool
 //   gqa_attn_kernel         one (token, head) per workgroup against the pool: softmax with a constant sink, sigmoid gate on the output
 //   gqa_attn_kernel<.., SPLIT> + gqa_attn_merge_kernel   the same with a sequence's keys divided between workgroups
 //   mlstm_scan_kernel       the matrix-memory recurrence over an entry's tokens, state per slot in fp32
@@ -117,9 +118,7 @@ struct GqaAppendArgs {
   const float* lam;
   int rot_pairs;             // 1: neighbours turn together
   float q_temp_coef; int q_temp_every;      // coef 0: no query temperature
-  float qk_unit_eps;         // > 0: every q and k head is first divided by sqrt(mean(head^2) + qk_unit_eps) ...
-  const float *q_norm, *k_norm;     // ... and multiplied by a vector of `dim` all heads share (nullptr: no weight)
-  int v_is_k;                // 1: the row holds no v: the values are the k columns as they come from the projection (vdim = dim)
+  float qk_unit_eps;         // > 0: every q and k head is first divided by sqrt(mean(head^2) + qk_unit_eps) (no weight)
   unsigned short *q_hi, *q_lo;      // [T][heads * dim] (nullptr: not kept): the finished queries as two 16-bit terms, the A operand of a matrix-core score product
 };
 template <int DT>
@@ -127,21 +126,6 @@ __global__ __launch_bounds__(256) void gqa_append_kernel(StepMeta m, GqaAppendAr
   const int t = blockIdx.x, pos = m.tok_pos[t];
   float* row = a.proj + (size_t)t * a.ldp;
   const int half = a.rot_dims >> 1, nh = a.heads + (a.poolK ? a.kv_heads : 0);      // q heads and k heads are adjacent in the row: head index hd, offset hd * dim
-  int page = 0;
-  if (a.poolK) page = m.tbl[(size_t)m.tok_row[t] * m.tbl_stride + (pos >> m.page_shift)];
-  const int pmask = (1 << m.page_shift) - 1;
-  const size_t slot = ((size_t)page << m.page_shift) + (size_t)(pos & pmask);
-  const int kd = a.kv_heads * a.dim, vd = a.kv_heads * a.vdim;
-  const float* ksrc = row + (size_t)a.heads * a.dim;
-  auto put_value = [&](int c, float v) {
-    const elem_t<DT> sv = f32_to_elem<DT>(v);
-    reinterpret_cast<elem_t<DT>*>(a.poolV)[slot * vd + c] = sv;
-    if (a.poolVT) reinterpret_cast<elem_t<DT>*>(a.poolVT)[((((size_t)page * vd) + c) << m.page_shift) + (size_t)(pos & pmask)] = sv;
-  };
-  if (a.v_is_k && a.poolK) {
-    for (int c = threadIdx.x; c < vd; c += 256) put_value(c, ksrc[c]);
-    __syncthreads();
-  }
   if (a.qk_unit_eps > 0.f) {      // a wave per head
     const int lane = threadIdx.x & 63;
     for (int hd = threadIdx.x >> 6; hd < nh; hd += 4) {
@@ -150,8 +134,7 @@ __global__ __launch_bounds__(256) void gqa_append_kernel(StepMeta m, GqaAppendAr
       for (int c = lane; c < a.dim; c += 64) ss = fmaf(u[c], u[c], ss);
       ss = wave_sum(ss);
       const float r = 1.0f / sqrtf(ss / (float)a.dim + a.qk_unit_eps);
-      const float* nw = hd < a.heads ? a.q_norm : a.k_norm;
-      for (int c = lane; c < a.dim; c += 64) u[c] *= nw ? r * nw[c] : r;
+      for (int c = lane; c < a.dim; c += 64) u[c] *= r;
     }
     __syncthreads();
   }
@@ -178,16 +161,67 @@ __global__ __launch_bounds__(256) void gqa_append_kernel(StepMeta m, GqaAppendAr
   }
   if (!a.poolK) return;
   __syncthreads();
+  const int page = m.tbl[(size_t)m.tok_row[t] * m.tbl_stride + (pos >> m.page_shift)];
+  const size_t slot = ((size_t)page << m.page_shift) + (size_t)(pos & ((1 << m.page_shift) - 1));
+  const int kd = a.kv_heads * a.dim, vd = a.kv_heads * a.vdim;
   elem_t<DT>* kdst = reinterpret_cast<elem_t<DT>*>(a.poolK) + slot * kd;
+  elem_t<DT>* vdst = reinterpret_cast<elem_t<DT>*>(a.poolV) + slot * vd;
+  const float* ksrc = row + (size_t)a.heads * a.dim;
   const float* vsrc = ksrc + kd;
   for (int c = threadIdx.x; c < kd; c += 256) kdst[c] = f32_to_elem<DT>(ksrc[c]);
-  if (a.v_is_k) return;
   const float lam = a.vmode == 2 ? a.lam[0] : 0.f;
   for (int c = threadIdx.x; c < vd; c += 256) {
     float v = vsrc[c];
     if (a.vmode == 1) a.vfirst[(size_t)t * vd + c] = v;
     if (a.vmode == 2) v = fmaf(lam, a.vfirst[(size_t)t * vd + c], __fmul_rn(1.0f - lam, v));
-    put_value(c, v);
+    const elem_t<DT> sv = f32_to_elem<DT>(v);
+    vdst[c] = sv;
+    if (a.poolVT) reinterpret_cast<elem_t<DT>*>(a.poolVT)[((((size_t)page * vd) + c) << m.page_shift) + (size_t)(pos & ((1 << m.page_shift) - 1))] = sv;
+  }
+}
+
+// ---- the append of a layer whose values are its keys: the projections' row is [q | k | ..], a token's values are its k columns as they come from the projection, and
+// every q and k head is divided by sqrt(mean(head^2) + eps) and multiplied by a vector all heads share (nullptr: none).  q is rewritten in place, k and v go to the pool.
+// A wave per head keeps the head in registers between the value store, the norm and the key store, so nothing waits for another wave.  Grid: (tokens, heads / 4).
+struct KeyValueAppendArgs {
+  float* proj; long long ldp;
+  int heads, kv_heads, dim;
+  const float *q_norm, *k_norm; float eps;
+  void *poolK, *poolV, *poolVT;      // as in GqaAppendArgs
+};
+constexpr int KV_APPEND_RPL = 4;      // channels per lane: dim <= 256
+template <int DT>
+__global__ __launch_bounds__(256) void key_value_append_kernel(StepMeta m, KeyValueAppendArgs a) {
+  const int t = blockIdx.x, hd = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (hd >= a.heads + a.kv_heads) return;
+  const bool key = hd >= a.heads;
+  float* u = a.proj + (size_t)t * a.ldp + (size_t)hd * a.dim;
+  const float* nw = key ? a.k_norm : a.q_norm;
+  float v[KV_APPEND_RPL], w[KV_APPEND_RPL], ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < KV_APPEND_RPL; k++) {
+    const int c = lane + 64 * k;
+    v[k] = c < a.dim ? u[c] : 0.f;
+    w[k] = nw && c < a.dim ? nw[c] : 1.f;
+  }
+#pragma unroll
+  for (int k = 0; k < KV_APPEND_RPL; k++) ss = fmaf(v[k], v[k], ss);
+  const float r = 1.0f / sqrtf(wave_sum(ss) / (float)a.dim + a.eps);
+  if (!key) {
+#pragma unroll
+    for (int k = 0; k < KV_APPEND_RPL; k++) { const int c = lane + 64 * k; if (c < a.dim) u[c] = v[k] * r * w[k]; }
+    return;
+  }
+  const int pos = m.tok_pos[t], page = m.tbl[(size_t)m.tok_row[t] * m.tbl_stride + (pos >> m.page_shift)], off = pos & ((1 << m.page_shift) - 1), kd = a.kv_heads * a.dim;
+  const size_t slot = (((size_t)page << m.page_shift) + (size_t)off) * kd;
+#pragma unroll
+  for (int k = 0; k < KV_APPEND_RPL; k++) {
+    const int c = lane + 64 * k, ch = (hd - a.heads) * a.dim + c;
+    if (c >= a.dim) continue;
+    const elem_t<DT> sv = f32_to_elem<DT>(v[k]);
+    reinterpret_cast<elem_t<DT>*>(a.poolK)[slot + ch] = f32_to_elem<DT>(v[k] * r * w[k]);
+    reinterpret_cast<elem_t<DT>*>(a.poolV)[slot + ch] = sv;
+    if (a.poolVT) reinterpret_cast<elem_t<DT>*>(a.poolVT)[((((size_t)page * kd) + ch) << m.page_shift) + (size_t)off] = sv;
   }
 }
 
@@ -209,7 +243,8 @@ struct GqaAttnArgs {
   int mask_kind, mask_size;            // MASK_*
   float softcap; int dist_bias;        // softcap <= 0: none
   const float* sinks;                  // [heads]: a sink per head (instead of `sink`; nullptr: none)
-  const float* dist_tab; int dist_len; // [heads][dist_len]: added to the score by distance i - j, the last entry for every larger one (nullptr: none)
+  const float* dist_tab; int dist_len; // [heads][dist_len]: added to the score by distance n = i - j, at index max(dist_len - 1 - DIST_PAD - n, 0): far distances come first, every
+                                       // distance beyond the table takes its first entry, and DIST_PAD entries follow distance 0 (nullptr: none)
   int gate_per_head;                   // 1: one gate pre-activation per head, at gate + t * ldg + h
   float out_scale;                     // factor on the output
 };
@@ -255,7 +290,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(StepMeta m, GqaAttnArgs a
     s = wave_sum(s) * a.scale;
     if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
     s = fmaf(-slope, (float)(nkeys - 1 - j), s);
-    if (dist) s += dist[min(nkeys - 1 - j, a.dist_len - 1)];
+    if (dist) s += dist[max(a.dist_len - 1 - DIST_PAD - (nkeys - 1 - j), 0)];
     const float mn = fmaxf(mx, s);
     const float corr = expf(mx - mn), p = expf(s - mn);      // mx = -inf on a wave's first key: corr = 0
     l = fmaf(l, corr, p);

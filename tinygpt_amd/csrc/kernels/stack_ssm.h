@@ -278,17 +278,18 @@ __global__ __launch_bounds__(256) void part_norm_gate_kernel(PartNormArgs a) {
   float* __restrict__ out = a.out + t * a.ldo + c0;
   float ss = 0.f;
   if (a.n <= 256 * PART_REG) {
-    float u[PART_REG];
+    float u[PART_REG], g[PART_REG], wk[PART_REG];      // all loads first
 #pragma unroll
     for (int k = 0; k < PART_REG; k++) {
       const int c = threadIdx.x + 256 * k;
-      u[k] = c < a.n ? y[c] * silu_f(z[c]) : 0.f;
-      ss = fmaf(u[k], u[k], ss);
+      u[k] = c < a.n ? y[c] : 0.f; g[k] = c < a.n ? z[c] : 0.f; wk[k] = c < a.n ? w[c] : 0.f;
     }
+#pragma unroll
+    for (int k = 0; k < PART_REG; k++) { u[k] *= silu_f(g[k]); ss = fmaf(u[k], u[k], ss); }
     ss = block_sum_256(ss, s4);
     const float r = a.scale / sqrtf(ss / (float)a.n + a.eps);
 #pragma unroll
-    for (int k = 0; k < PART_REG; k++) { const int c = threadIdx.x + 256 * k; if (c < a.n) out[c] = u[k] * r * w[c]; }
+    for (int k = 0; k < PART_REG; k++) { const int c = threadIdx.x + 256 * k; if (c < a.n) out[c] = u[k] * r * wk[k]; }
     return;
   }
   for (int c = threadIdx.x; c < a.n; c += 256) { const float u = y[c] * silu_f(z[c]); ss = fmaf(u, u, ss); }

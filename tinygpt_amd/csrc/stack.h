@@ -57,7 +57,7 @@ struct StackLayerW {
   //   mamba1:   w_in = [x | z] rows, conv_w / conv_b the filters, w_w1 the product for [dt | B | C], w_w2 / w0 the step sizes' product and bias, decay2 =
   //             -exp(A_log) log2(e) [inner][state], d_skip; mS the state [slots][inner][state], conv_state the tails of the raw x columns
   //   parallel: w_in = [left q | k | right in (z | x | B | C | dt) | left gate] rows, b_in the biases of q and k, q_norm / k_norm, sink, dist the distance bias
-  //             expanded to [heads][dist_len]; w_o = [left | right] output projections side by side [width][heads * vdim + d_heads * d_vdim]; conv_w / conv_b,
+  //             by head and distance (GqaAttnArgs::dist_tab); w_o = [left | right] output projections side by side [width][heads * vdim + d_heads * d_vdim]; conv_w / conv_b,
   //             a_log, dt_bias, d_skip, head_w (the weight of the part norm) of the right half, mS its state [slots][d_heads][d_dim][d_vdim]
   float *conv_b = nullptr, *d_skip = nullptr, *decay2 = nullptr, *q_norm = nullptr, *k_norm = nullptr, *dist = nullptr;
   int dist_len = 0;
@@ -119,16 +119,22 @@ struct StackModel {
   int attn_mfma = 1;                   // option attn.mfma: 0 keeps every layer on the lane-per-channel attention kernels
   int gemv = 1;                        // option stack.gemv: 0 sends products of few rows through the matrix-core tiles as well
   int mlstm_narrow = -1;               // option mlstm.narrow: the matrix-memory scan's columns per wave (1: eight, 0: sixteen, -1: by the step's entries and heads)
+  int ssd_min = 64;                    // option ssd.min: portions from this many tokens on take the blocked form of the scalar-decay recurrence (0: never)
   int mix_groups = 0;                  // option attn.mix_groups: key / value heads per workgroup of the matrix-core sigmoid attention: 1; 2 where their accumulators fit, whatever the grid; 0: 2 while the halved grid fills the chip
   int gemm_wt = 0;                     // option stack.gemm_wt: force the product's tile (1: 64 x 64, 2: 128 x 128); 0 = by the number of tiles
 };
 
 // stack_gqa.hip
-namespace tgx { struct StepMeta; struct GqaMfmaArgs; struct MixMfmaArgs; }
+namespace tgx { struct StepMeta; struct GqaMfmaArgs; struct MixMfmaArgs; struct SsdArgs; }
 bool gqa_mfma_shapes_ok(int dt, int dim, int vdim, int page_shift, long long ldq);
 void launch_gqa_mfma(tgx_ctx* c, const tgx::StepMeta& m, const tgx::GqaMfmaArgs& a, dim3 grid, bool split);
 void launch_mix_mfma(tgx_ctx* c, const tgx::StepMeta& m, const tgx::MixMfmaArgs& a, dim3 grid);      // kernels/stack_mix_mfma.h
 size_t mix_mfma_wg_lds(int heads, int kv_heads);      // LDS bytes of one of its workgroups
+
+// stack_ssd.hip
+bool ssd_mfma_shapes_ok(int heads, int groups, int N, int E, long long ld);
+size_t ssd_gram_elems(int T, int S, int groups);
+void launch_ssd_mfma(tgx_ctx* c, const tgx::StepMeta& m, const tgx::SsdArgs& a, int S, int max_count);
 
 int stack_create(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int device_ordinal, tgx_ctx** out_ctx);
 int stack_upload(tgx_ctx* c, const char* name, const void* host, const int64_t* shape, int nd, int src_dtype);

@@ -19,6 +19,7 @@
 #include "kernels/stack_loop.h"
 #include "kernels/stack_mix_mfma.h"
 #include "kernels/stack_ssm.h"
+#include "kernels/stack_ssd_mfma.h"
 
 int upload_param_ext(tgx_ctx* c, ebyte* dst, const void* host, int64_t n, int src_dtype);      // abi.hip
 
@@ -357,7 +358,7 @@ struct GqaSpec {
   int mask_kind, mask_size; float softcap; int dist_bias;
   float q_temp_coef; int q_temp_every;
   float* out; long long ldo;
-  float qk_eps; const float *q_norm, *k_norm; int v_is_k;      // unit (or weighted) queries and keys; the key projections are the values
+  int v_is_k; float qk_eps; const float *q_norm, *k_norm;      // the key projections are the values; normed queries and keys (no rotation)
   const float* sinks; const float* dist; int dist_len;         // per-head sinks, distance table
   int gate_per_head;
   float out_scale = 1.0f;
@@ -369,8 +370,12 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
   ap.proj = sp.proj; ap.ldp = sp.ldp; ap.heads = H; ap.kv_heads = G; ap.dim = sp.dim; ap.vdim = sp.vdim; ap.rot_dims = sp.cs ? sp.rot_dims : 0; ap.rot_pairs = sp.rot_pairs;
   ap.cs = sp.cs; ap.poolK = sp.append ? sp.poolK : nullptr; ap.poolV = sp.poolV; ap.poolVT = sp.poolVT; ap.vfirst = sm->vfirst; ap.vmode = sp.vmode; ap.lam = sp.lam;
   ap.q_temp_coef = sp.q_temp_every > 0 ? sp.q_temp_coef : 0.f; ap.q_temp_every = sp.q_temp_every;
-  ap.qk_unit_eps = sp.qk_eps; ap.q_norm = sp.q_norm; ap.k_norm = sp.k_norm; ap.v_is_k = sp.v_is_k;
-  if (sp.append || ap.rot_dims > 0 || ap.q_temp_coef != 0.f || ap.qk_unit_eps > 0.f) TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::gqa_append_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, ap))
+  if (sp.v_is_k) {      // normed queries and keys, the keys' projections as values
+    tgx::KeyValueAppendArgs ka{};
+    ka.proj = sp.proj; ka.ldp = sp.ldp; ka.heads = H; ka.kv_heads = G; ka.dim = sp.dim; ka.q_norm = sp.q_norm; ka.k_norm = sp.k_norm; ka.eps = sp.qk_eps;
+    ka.poolK = sp.poolK; ka.poolV = sp.poolV; ka.poolVT = sp.poolVT;
+    TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::key_value_append_kernel<DT>, dim3(T, (H + G + 3) / 4), dim3(256), 0, c->stream, m, ka))
+  } else if (sp.append || ap.rot_dims > 0 || ap.q_temp_coef != 0.f) TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::gqa_append_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, ap))
   // the longest run of keys any workgroup walks: everything before the token, or the mask's span (plus the matrix-core kernel's tile alignment)
   const int span = sp.mask_kind == tgx::MASK_CAUSAL ? max_keys : std::min(max_keys, sp.mask_size + 96);
   if (sp.poolVT && sm->attn_mfma) {
@@ -1247,7 +1252,12 @@ int run_ssm_parallel(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T, 
   tgx::RecScanArgs ra{};
   ra.a = sm->rec_in + I + gn; ra.lda = ldr; ra.k = sm->rec_in + I; ra.ldk = ldr; ra.v = sm->rec_in; ra.ldv = ldr; ra.beta = sm->rec_in + C; ra.g = sm->rec_in + C + rH; ra.ldg = ldr;
   ra.skip = w.d_skip; ra.S = w.mS; ra.out = sm->hs; ra.ldo = I; ra.heads = rH; ra.kv_heads = ld.d_kv_heads; ra.dim = ld.d_dim; ra.vdim = ld.d_vdim;
-  launch_rec_scan(c, m, ra, tgx::REC_SSD, S);
+  if (sm->ssd_min > 0 && max_count >= sm->ssd_min && ssd_mfma_shapes_ok(rH, ld.d_kv_heads, ld.d_dim, ld.d_vdim, ldr)) {
+    if ((rc = ensure_part(c, ssd_gram_elems(T, S, ld.d_kv_heads)))) return rc;
+    tgx::SsdArgs da{};
+    da.row = sm->rec_in; da.ld = ldr; da.heads = rH; da.groups = ld.d_kv_heads; da.N = ld.d_dim; da.E = ld.d_vdim; da.gram = sm->part; da.skip = w.d_skip; da.S = w.mS; da.out = sm->hs; da.ldo = I;
+    launch_ssd_mfma(c, m, da, S, max_count);
+  } else launch_rec_scan(c, m, ra, tgx::REC_SSD, S);
   tgx::PartNormArgs pa{};
   pa.y = sm->hs; pa.ldy = I; pa.z = sm->proj + r0; pa.ldz = ldp; pa.w = w.head_w; pa.out = sm->o + lvd; pa.ldo = ldo; pa.n = I / ld.part_norms; pa.eps = sm->d.norm_eps; pa.scale = ld.right_scale;
   hipLaunchKernelGGL(tgx::part_norm_gate_kernel, dim3(T, ld.part_norms), dim3(256), 0, c->stream, pa);
@@ -1309,7 +1319,7 @@ int create_post_layers(tgx_ctx* c, const tgx_layer_desc* layers) {
           (rc = dev_alloc(c, &w.k_norm, (size_t)l.dim)) || (rc = dev_alloc(c, &w.sink, H)) || (rc = dev_alloc(c, &w.conv_w, C * (size_t)l.conv_taps)) || (rc = dev_alloc(c, &w.conv_b, C)) ||
           (rc = dev_alloc(c, &w.a_log, rH)) || (rc = dev_alloc(c, &w.dt_bias, rH)) || (rc = dev_alloc(c, &w.d_skip, rH)) || (rc = dev_alloc(c, &w.head_w, I))) return rc;
       HIP_OK(c, hipMemset(w.b_in, 0, nin * 4));
-      w.dist_len = std::min(l.bias_max, d.max_ctx - 1) + 1;      // distances 0 .. bias_max; from there on every distance takes the last row
+      w.dist_len = std::min(l.bias_max, d.max_ctx - 1) + 1 + 2 * tgx::DIST_PAD;      // distances 0 .. bias_max; from there on every distance takes the last row
       if ((rc = dev_alloc(c, &w.dist, H * (size_t)w.dist_len))) return rc;
       need(p, {"mix.left.q", "mix.left.q.b", "mix.left.q.norm", "mix.left.k", "mix.left.k.b", "mix.left.k.norm", "mix.left.rel", "mix.left.sink", "mix.left.g", "mix.left.o",
                "mix.right.in", "mix.right.conv", "mix.right.conv.b", "mix.right.dt_bias", "mix.right.A_log", "mix.right.D", "mix.right.norm", "mix.right.o"});
@@ -1414,9 +1424,9 @@ int upload_post(tgx_ctx* c, const char* name, const void* host, const int64_t* s
       if (l.bias_max <= B / 2) return set_err(c, TGX_ERR_INVALID, "%s: bias_max %d within the %d exact rows of the table", name, l.bias_max, B / 2);
       const std::vector<float> v = to_f32(host, (int64_t)B * H, src_dtype);
       std::vector<float> t((size_t)H * w.dist_len);
-      for (int n = 0; n < w.dist_len; n++) {
+      for (int n = 0; n < w.dist_len - tgx::DIST_PAD; n++) {
         const int b = distance_bucket(n, B, l.bias_max);
-        for (int64_t h = 0; h < H; h++) t[(size_t)h * w.dist_len + n] = v[(size_t)b * H + h];
+        for (int64_t h = 0; h < H; h++) t[(size_t)h * w.dist_len + (w.dist_len - 1 - tgx::DIST_PAD - n)] = v[(size_t)b * H + h];
       }
       return done(upload_f32(c, w.dist, t.data(), (int64_t)t.size(), TGX_F32));
     }
