@@ -55,98 +55,126 @@ __global__ __launch_bounds__(256) void ssd_gram_kernel(StepMeta m, SsdArgs a) {
 // row (r & 3) + 8 (r >> 2) + 4 (lane / 32), column lane % 32.  Register r of the two half-waves is at the same time a B operand whose two contraction slots are those
 // two rows, so S^T C needs no transposition: its A operand takes C's channels in that order.  A wave contributes its rows' share of S^T C and the share of sixteen
 // keys j of the block's own product; the four waves' shares are added up in LDS.  Grid: (entries, heads, E / 32).
+// Operands travel straight from memory to registers (every wave reads its own state rows only): B of a block is asked for at the block's start and used at its end,
+// C and the Gram rows of the next block replace the present ones as soon as these are used up, so nothing is held twice.  Rows past the
+// entry's end are clamped to its last one (what is read there twice meets dt = 0 or is not stored).
 template <int NW>
-__global__ __launch_bounds__(256, 1) void ssd_block_kernel(StepMeta m, SsdArgs a) {
+__global__ __launch_bounds__(256, NW == 1 ? 2 : 1) void ssd_block_kernel(StepMeta m, SsdArgs a) {
   constexpr int Q = SSD_BLOCK;
   constexpr double LOG2E = 1.4426950408889634;
   __shared__ float s_x[2][Q][32];
   __shared__ double s_cs[2][Q];        // base-2 logarithms, summed from the block's start
-  __shared__ float s_dt[2][Q];
+  __shared__ float s_dt[2][Q], s_end[2][Q];      // dt_j, exp(cs_64 - cs_j) dt_j
   __shared__ float s_part[4][Q][33];
-  const int e = blockIdx.x, h = blockIdx.y, e0 = blockIdx.z * 32, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, half = lane >> 5, l31 = lane & 31;
+  const int e = blockIdx.x, h = blockIdx.y, e0 = blockIdx.z * 32, tid = threadIdx.x, lane = tid & 63, wv = __builtin_amdgcn_readfirstlane(tid >> 6), half = lane >> 5, l31 = lane & 31;
   const int start = m.ent_start[e], cnt = m.ent_count[e], slot = m.ent_row[e], grp = h / (a.heads / a.groups);
   const bool fresh = m.tok_pos[start] == 0;
-  const float* base = a.row + (size_t)start * a.ld;
-  const size_t oB = (size_t)a.heads * a.E + (size_t)grp * a.N, oC = oB + (size_t)a.groups * a.N, oD = (size_t)a.heads * a.E + 2 * (size_t)a.groups * a.N + h, oL = oD + 2 * (size_t)a.heads;
+  const int ld = (int)a.ld, oX = h * a.E + e0, oB = a.heads * a.E + grp * a.N, oC = oB + a.groups * a.N, oD = a.heads * a.E + 2 * a.groups * a.N + h, oL = oD + 2 * a.heads;
+  const float* base = a.row + (size_t)start * ld;
   const float* gram = a.gram + ((size_t)ssd_first_block(start, e) * a.groups + grp) * (Q * Q);
   float* Sg = a.S + ((size_t)slot * a.heads + h) * (size_t)a.N * a.E;
   const bool colok = e0 + l31 < a.E;
+  const int xcol = colok ? l31 : 0, n0 = 32 * wv * NW;
   f32x16 S[NW];
 #pragma unroll
   for (int w = 0; w < NW; w++)
 #pragma unroll
     for (int r = 0; r < 16; r++) {
-      const int n = 32 * (wv * NW + w) + (r & 3) + 8 * (r >> 2) + 4 * half;
+      const int n = n0 + 32 * w + (r & 3) + 8 * (r >> 2) + 4 * half;
       S[w][r] = (!fresh && n < a.N && colok) ? Sg[(size_t)n * a.E + e0 + l31] : 0.f;
     }
-  // operands of one block, fetched a block ahead: B[n][j] with j = kk + 32 half (the state's product), C[i][n] four channels at a time, the Gram rows of this wave's
-  // sixteen keys j = 16 wv + 8 half + 0 .. 7, the value columns, step sizes and log decays
-  struct Ops { float B[NW][32]; f32x4 C[NW][2][4]; f32x4 G[2][2]; float x[8]; float dt, la; };
-  Ops cur, nxt;
-  auto fetch = [&](Ops& o, int b) {
-    const int t0 = b * Q, left = cnt - t0;
+  auto at = [](const float* p, unsigned int bytes) -> const float* { return reinterpret_cast<const float*>(reinterpret_cast<const char*>(p) + bytes); };
+  // byte offset of row t0 + k of a block with `left` rows, clamped to its last one (ld < 2^21 floats: the factors fit 24 bits); the constant k stays out of registers
+  auto row_off = [&](int t0, int k, int left) -> unsigned int { return (unsigned int)(4 * (__mul24(t0, ld) + __mul24(min(k, left - 1 - t0), ld))); };
+  float B[NW][32], x[8], dt = 0.f, la = 0.f;      // B[n][j]: j = kk + 32 half
+  f32x4 C[NW][2][4], G[2][2];                     // C[i][n]: four channels at a time; the Gram rows of this wave's sixteen keys j = 16 wv + 8 half + 0 .. 7
+  // (what stands in state rows beyond N is finite and meets a factor of zero)
+  auto fetch_B = [&](int b) {
+    const float* p = base + (size_t)b * Q * ld + oB;
+    const int left = cnt - b * Q;
 #pragma unroll
     for (int w = 0; w < NW; w++) {
-      const int n = 32 * (wv * NW + w) + l31;
+      const int n = min(n0 + 32 * w + l31, a.N - 1);
 #pragma unroll
-      for (int kk = 0; kk < 32; kk++) { const int j = kk + 32 * half; o.B[w][kk] = (j < left && n < a.N) ? base[(size_t)(t0 + j) * a.ld + oB + n] : 0.f; }
+      for (int kk = 0; kk < 32; kk++) B[w][kk] = *at(p, row_off(32 * half, kk, left) + 4 * n);
+    }
+  };
+  auto fetch_C = [&](int b) {
+    const float* p = base + (size_t)b * Q * ld + oC;
+    const int left = cnt - b * Q;
+#pragma unroll
+    for (int w = 0; w < NW; w++)
 #pragma unroll
       for (int it = 0; it < 2; it++)
 #pragma unroll
         for (int q = 0; q < 4; q++) {
-          const int i = 32 * it + l31, nc = 32 * (wv * NW + w) + 8 * q + 4 * half;
-          o.C[w][it][q] = (i < left && nc < a.N) ? *reinterpret_cast<const f32x4*>(base + (size_t)(t0 + i) * a.ld + oC + nc) : f32x4{0.f, 0.f, 0.f, 0.f};
+          const int n = n0 + 32 * w + 8 * q + 4 * half;
+          C[w][it][q] = *reinterpret_cast<const f32x4*>(at(p, row_off(l31, 32 * it, left) + 4 * min(n, a.N - 4)));
         }
-    }
-    const float* G = gram + (size_t)b * a.groups * (Q * Q);
+  };
+  auto fetch_G = [&](int b) {
+    const float* p = gram + (size_t)b * a.groups * (Q * Q);
 #pragma unroll
     for (int it = 0; it < 2; it++)
+      if (16 * wv <= 32 * it + 31)
 #pragma unroll
-      for (int q = 0; q < 2; q++) {
-        const int j = 16 * wv + 8 * half + 4 * q;
-        o.G[it][q] = j <= 32 * it + 31 ? *reinterpret_cast<const f32x4*>(G + (32 * it + l31) * Q + j) : f32x4{0.f, 0.f, 0.f, 0.f};
-      }
-#pragma unroll
-    for (int u = 0; u < 8; u++) { const int t = (tid >> 5) + 8 * u; o.x[u] = (t < left && colok) ? base[(size_t)(t0 + t) * a.ld + (size_t)h * a.E + e0 + l31] : 0.f; }
-    if (wv == 0) { o.dt = lane < left ? base[(size_t)(t0 + lane) * a.ld + oD] : 0.f; o.la = lane < left ? base[(size_t)(t0 + lane) * a.ld + oL] : 0.f; }
+        for (int q = 0; q < 2; q++) G[it][q] = *reinterpret_cast<const f32x4*>(at(p, 4u * (unsigned int)((32 * it + l31) * Q + 16 * wv + 8 * half + 4 * q)));
   };
-  auto stage = [&](const Ops& o, int buf) {
+  auto fetch_x = [&](int b) {
+    const float* p = base + (size_t)b * Q * ld;
+    const int left = cnt - b * Q;
 #pragma unroll
-    for (int u = 0; u < 8; u++) s_x[buf][(tid >> 5) + 8 * u][l31] = o.x[u];
+    for (int u = 0; u < 8; u++) x[u] = *at(p, row_off(tid >> 5, 8 * u, left) + 4 * (oX + xcol));
+    if (wv == 0) { const unsigned int off = row_off(lane, 0, left); dt = *at(p + oD, off); la = *at(p + oL, off); }
+  };
+  auto stage = [&](int b) {
+    const int buf = b & 1, left = cnt - b * Q;
+#pragma unroll
+    for (int u = 0; u < 8; u++) s_x[buf][(tid >> 5) + 8 * u][l31] = x[u];
     if (wv == 0) {
-      double v = (double)o.la * LOG2E;
+      double v = lane < left ? (double)la * LOG2E : 0.0;
+      const float d = lane < left ? dt : 0.f;
 #pragma unroll
-      for (int d = 1; d < 64; d <<= 1) { const double p = __shfl_up(v, d, 64); if (lane >= d) v += p; }
-      s_cs[buf][lane] = v; s_dt[buf][lane] = o.dt;
+      for (int o = 1; o < 64; o <<= 1) { const double p = __shfl_up(v, o, 64); if (lane >= o) v += p; }
+      const double end = __shfl(v, 63, 64);
+      s_cs[buf][lane] = v; s_dt[buf][lane] = d; s_end[buf][lane] = d * __builtin_amdgcn_exp2f((float)(end - v));
     }
   };
   const float Dh = a.skip[h];
   const int nblk = (cnt + Q - 1) / Q;
-  fetch(cur, 0);
-  stage(cur, 0);
+  fetch_x(0); fetch_C(0); fetch_G(0);
+  stage(0);
   for (int b = 0; b < nblk; b++) {
     const int buf = b & 1, t0 = b * Q;
+    const bool more = b + 1 < nblk;
     __syncthreads();      // the block's columns and sums stand; the shares of the block before have been read
-    if (b + 1 < nblk) fetch(nxt, b + 1);
+    fetch_B(b);
+    if (more) fetch_x(b + 1);
+    __builtin_amdgcn_sched_barrier(0);      // (the phases stay apart: operands of a later one must not take registers early)
     f32x16 acc[2];
 #pragma unroll
     for (int it = 0; it < 2; it++)
 #pragma unroll
       for (int r = 0; r < 16; r++) acc[it][r] = 0.f;
     double csi[2];
+    float ei[2];
 #pragma unroll
-    for (int it = 0; it < 2; it++) csi[it] = s_cs[buf][32 * it + l31];
+    for (int it = 0; it < 2; it++) { csi[it] = s_cs[buf][32 * it + l31]; ei[it] = __builtin_amdgcn_exp2f((float)csi[it]); }
     // exp(cs_i) S_in^T C_i over this wave's state rows
 #pragma unroll
-    for (int it = 0; it < 2; it++) {
-      const float ei = __builtin_amdgcn_exp2f((float)csi[it]);
+    for (int w = 0; w < NW; w++)
+      if (n0 + 32 * w < a.N)      // (wave-uniform)
 #pragma unroll
-      for (int w = 0; w < NW; w++)
-        if (32 * (wv * NW + w) < a.N)      // (wave-uniform)
+        for (int r = 0; r < 16; r++) {
+          const bool in = n0 + 32 * w + 8 * (r >> 2) + 4 * half < a.N;
 #pragma unroll
-          for (int r = 0; r < 16; r++) acc[it] = __builtin_amdgcn_mfma_f32_32x32x2f32(cur.C[w][it][r >> 2][r & 3] * ei, S[w][r], acc[it], 0, 0, 0);
-    }
+          for (int it = 0; it < 2; it++) acc[it] = __builtin_amdgcn_mfma_f32_32x32x2f32(C[w][it][r >> 2][r & 3] * (in ? ei[it] : 0.f), S[w][r], acc[it], 0, 0, 0);
+        }
+    if (more) fetch_C(b + 1);
+    __builtin_amdgcn_sched_barrier(0);
     // the block's own tokens: this wave's sixteen keys
+    int ahead = l31 - 16 * wv - 8 * half;      // key k of this lane lies ahead of row 32 it + l31 when k > ahead + 32 it
+    asm volatile("" : "+v"(ahead));            // (not hoisted into sixteen lane masks)
 #pragma unroll
     for (int k = 0; k < 8; k++) {
       const int j = 16 * wv + 8 * half + k;
@@ -154,46 +182,47 @@ __global__ __launch_bounds__(256, 1) void ssd_block_kernel(StepMeta m, SsdArgs a
       const float xj = s_x[buf][j][l31] * s_dt[buf][j];
 #pragma unroll
       for (int it = 0; it < 2; it++) {
-        if (16 * wv > 32 * it + 31) continue;      // (wave-uniform: all of the wave's keys lie behind these rows)
-        const float mij = j <= 32 * it + l31 ? cur.G[it][k >> 2][k & 3] * __builtin_amdgcn_exp2f((float)(csi[it] - csj)) : 0.f;
+        // (for two of the waves all keys lie ahead of the first 32 rows: they multiply zeros while the others, whom they would wait for, do not)
+        const float mij = k <= ahead + 32 * it ? G[it][k >> 2][k & 3] * __builtin_amdgcn_exp2f((float)(csi[it] - csj)) : 0.f;
         acc[it] = __builtin_amdgcn_mfma_f32_32x32x2f32(mij, xj, acc[it], 0, 0, 0);
       }
     }
+    if (more) fetch_G(b + 1);
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
     for (int it = 0; it < 2; it++)
 #pragma unroll
       for (int r = 0; r < 16; r++) s_part[wv][32 * it + (r & 3) + 8 * (r >> 2) + 4 * half][l31] = acc[it][r];
+    __builtin_amdgcn_sched_barrier(0);
     // S_out
-    const double cse = s_cs[buf][Q - 1];
-    const float ge = __builtin_amdgcn_exp2f((float)cse);
+    const float ge = __builtin_amdgcn_exp2f((float)s_cs[buf][Q - 1]);
 #pragma unroll
     for (int w = 0; w < NW; w++)
 #pragma unroll
       for (int r = 0; r < 16; r++) S[w][r] *= ge;
+    if (n0 < a.N)
 #pragma unroll
-    for (int kk = 0; kk < 32; kk++) {
-      const int j = kk + 32 * half;
-      const float xs = s_x[buf][j][l31] * s_dt[buf][j] * __builtin_amdgcn_exp2f((float)(cse - s_cs[buf][j]));
+      for (int kk = 0; kk < 32; kk++) {
+        const int j = kk + 32 * half;
+        const float xs = s_x[buf][j][l31] * s_end[buf][j];
 #pragma unroll
-      for (int w = 0; w < NW; w++)
-        if (32 * (wv * NW + w) < a.N) S[w] = __builtin_amdgcn_mfma_f32_32x32x2f32(cur.B[w][kk], xs, S[w], 0, 0, 0);
-    }
-    if (b + 1 < nblk) stage(nxt, buf ^ 1);
+        for (int w = 0; w < NW; w++) S[w] = __builtin_amdgcn_mfma_f32_32x32x2f32(B[w][kk], xs, S[w], 0, 0, 0);
+      }
+    __builtin_amdgcn_sched_barrier(0);
+    if (more) stage(b + 1);
     __syncthreads();
 #pragma unroll
     for (int u = 0; u < 8; u++) {
       const int t = (tid >> 5) + 8 * u;
       if (t0 + t < cnt && colok)
-        a.out[(size_t)(start + t0 + t) * a.ldo + (size_t)h * a.E + e0 + l31] =
-            fmaf(Dh, s_x[buf][t][l31], s_part[0][t][l31] + s_part[1][t][l31] + s_part[2][t][l31] + s_part[3][t][l31]);
+        a.out[(size_t)(start + t0 + t) * a.ldo + oX + l31] = fmaf(Dh, s_x[buf][t][l31], s_part[0][t][l31] + s_part[1][t][l31] + s_part[2][t][l31] + s_part[3][t][l31]);
     }
-    cur = nxt;
   }
 #pragma unroll
   for (int w = 0; w < NW; w++)
 #pragma unroll
     for (int r = 0; r < 16; r++) {
-      const int n = 32 * (wv * NW + w) + (r & 3) + 8 * (r >> 2) + 4 * half;
+      const int n = n0 + 32 * w + (r & 3) + 8 * (r >> 2) + 4 * half;
       if (n < a.N && colok) Sg[(size_t)n * a.E + e0 + l31] = S[w][r];
     }
 }

@@ -152,7 +152,7 @@ struct SelScanArgs {
 };
 template <int SPL, int LPC>
 __global__ __launch_bounds__(256) void selective_scan_kernel(StepMeta m, SelScanArgs a) {
-  constexpr int CPW = 256 / LPC, NP = SPL * LPC, TB = NP <= 64 ? 32 : 16, NX = (TB * CPW + 255) / 256, NB = TB * NP / 256 > 0 ? (TB * NP + 255) / 256 : 1;
+  constexpr int CPW = 256 / LPC, NP = SPL * LPC, TB = NP <= 32 ? 64 : NP <= 64 ? 32 : 16, NX = (TB * CPW + 255) / 256, NB = TB * NP / 256 > 0 ? (TB * NP + 255) / 256 : 1;
   typedef float f2 __attribute__((ext_vector_type(2)));
   __shared__ __attribute__((aligned(16))) f2 s_bc[TB][NP];
   __shared__ f2 s_dx[TB][CPW], s_xz[TB][CPW + 1];
