@@ -253,7 +253,7 @@ def test_one_far_key_stands_out(dim, dtype):
 
 @pytest.mark.parametrize("dtype", ["fp32", "bf16"])
 @pytest.mark.parametrize("dim", [8, 64])
-@pytest.mark.parametrize("buckets,bias_max", [(2, 2), (4, 17), (7, 40), (8, 64), (32, 120), (32, 17), (64, 700)])
+@pytest.mark.parametrize("buckets,bias_max", [(2, 2), (4, 17), (7, 40), (8, 64), (32, 130), (32, 17), (64, 700)])
 def test_distance_rows_one_by_one(buckets, bias_max, dim, dtype):
     """scores are zero and every row of the distance table is far from its neighbours: a distance that falls into a wrong row shows at once"""
     cfg = config([par(left={"heads": 2, "kv_heads": 1, "dim": dim, "mask": {"size": 150}, "scale": 1e-3, "bias_max": bias_max}, left_scale=1.0, right_scale=0.0)], width=16)

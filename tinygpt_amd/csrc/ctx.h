@@ -8,6 +8,7 @@
 //   skinny.hip       batched decode step / short prompts on the skinny MFMA GEMMs (kernels/skinny*.h)
 //   stack.hip        layered models (tgx_create_stack): ragged engine step, paged latent / key-value cache, slot state (kernels/stack*.h)
 //   stack_gqa.hip    their grouped-query attention on the matrix cores (kernels/stack_gqa_mfma.h)
+//   stack_ssd.hip    their blocked state-space recurrence on the matrix cores (kernels/stack_ssd_mfma.h)
 // One context = one GPU = one HIP stream; every call comes from one host thread.  There is NO CPU path in this library.
 #pragma once
 #include <hip/hip_runtime.h>
