@@ -27,11 +27,12 @@ extern "C" {
 
 /* 3 (round 5): per-row sequence lifecycle (tgx_reset_row / tgx_forward_row / tgx_sample_row / tgx_past_length_row); tgx_get_option added and
  * tgx_engine_read_stats + the options engine.*, pf.*, attn.fold_*, lmhead.fuse_finalize removed since 2. */
-#define TGX_ABI_VERSION 8   /* 4: layered models (tgx_create_stack, tgx_step_ragged); 5: Modepel (more mixers / feed-forward kinds in tgx_layer_desc);
+#define TGX_ABI_VERSION 9   /* 4: layered models (tgx_create_stack, tgx_step_ragged); 5: Modepel (more mixers / feed-forward kinds in tgx_layer_desc);
                              * 6: Vitudra (masks, score bias and cap, shared key / value layers, two recurrent mixers, parallel sublayers);
                              * 7: Zaluvik (layer norms around every sublayer, a looped span of layers, un-normalised sigmoid attention with mixed heads,
                              *    windowed latent attention with a shared rotated key part, sigmoid group-limited router);
-                             * 8: Nusovik (norms on the sublayers' outputs only, two state-space mixers, bucketed distance bias, per-head sink and gate) */
+                             * 8: Nusovik (norms on the sublayers' outputs only, two state-space mixers, bucketed distance bias, per-head sink and gate);
+                             * 9: Keronex (several residual streams, pair embedding, retention, channel-decay delta rule, two-map attention, layers that share weights) */
 
 #if defined(__GNUC__)
 #define TGX_API __attribute__((visibility("default")))
@@ -67,8 +68,11 @@ typedef enum tgx_family {
   TGX_FAMILY_ZALUVIK = 9,  /* a layered model: layer norms (weight and bias) before and after every sublayer, a span of layers run several times with the
                             * embedding output fed back in, windowed sigmoid attention whose weights are mixed across heads, windowed latent attention
                             * with a rotated key part all heads share, erf-gelu feed-forwards and sigmoid-routed experts; logits against the embedding table */
-  TGX_FAMILY_NUSOVIK = 10  /* a layered model: norms on the sublayers' outputs only; selective-scan layers and layers that run chunked attention (keys as values,
+  TGX_FAMILY_NUSOVIK = 10, /* a layered model: norms on the sublayers' outputs only; selective-scan layers and layers that run chunked attention (keys as values,
                             * bucketed distance bias, sinks) beside a scalar-decay state-space mixer; squared-relu feed-forwards */
+  TGX_FAMILY_KERONEX = 11  /* a layered model: several residual streams joined by learned mixes (hyper-connections), an embedding with a row per pair of tokens; retention,
+                            * two-map (differential) attention and a gated delta rule with a decay per key channel; sigmoid-routed squared-relu experts whose weight
+                            * multiplies their input; layers that use another layer's weights */
 } tgx_family;
 
 /* tinytorch::DType values the CLI accepts (examples/inference/main.cpp:82-88) */
@@ -172,8 +176,21 @@ typedef struct tgx_model_desc {
  *   parallel mixer            right_kind 1: the right half is a scalar-decay state-space mixer (state-space duality): d_heads heads of d_vdim values over d_kv_heads groups
  *                             of d_dim state numbers; convolution (with bias) and silu on x | B | C, dt = softplus(. + dt_bias), S <- exp(-exp(A_log) dt) S +
  *                             dt B x^T, y = S^T C + D x, then y * silu(z) RMS-normed in part_norms equal parts
- *   squared-relu feed-forward ff_act 2: down(max(up x, 0)^2) */
-typedef enum tgx_mixer { TGX_MIXER_LATENT_ATTENTION = 1, TGX_MIXER_ATTENTION = 2, TGX_MIXER_MLSTM = 3, TGX_MIXER_WKV = 4, TGX_MIXER_PARALLEL = 5, TGX_MIXER_MAMBA1 = 6 } tgx_mixer;
+ *   squared-relu feed-forward ff_act 2: down(max(up x, 0)^2)
+ * and, for TGX_FAMILY_KERONEX (`streams` copies x_1 .. x_n of the embedding output; a sublayer reads u = sum_s in[s] x_s through norm(u) = u / sqrt(mean(u^2) + norm_eps) *
+ * (1 + w), and leaves x_t <- sum_s mix[s][t] x_s + out[t] y in all streams at once; logits = head . norm(sum of the streams); streams 0: one stream, x <- x + y, without such
+ * tensors.  The embedding output is embed[token] * embed_scale + bigram[(token before * bigram_before + token * bigram_cur) mod bigram_buckets], row bigram_buckets for a
+ * sequence's first token; bigram_buckets 0: none.  Slots hold pages of the attention layers' key / value pools, one state per recurrent head, convolution tails and the last token):
+ *   attention                 maps 2: per head two queries and (per key / value head) two keys of `dim`, each map a causal softmax of its own over the same values;
+ *                             o = o_1 - lambda o_2, lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff; then o / sqrt(mean(o^2) + norm_eps) * (1 - diff) per head
+ *   retention                 S <- decays[head] S + k v^T, o = S^T q, k scaled by dim^(-1/2), rotary q and k; o / rms(o) * silu(gate)
+ *   channel delta             the gated delta rule with one decay per head and key channel, exp(-exp(A_log) softplus(W_a2 W_a1 h + dt_bias)); q and k of kv_heads heads;
+ *                             conv_taps taps and silu on q, k, v; o / rms(o) * w * sigmoid(W_g2 W_g1 h)
+ *   dense feed-forward        ff_act 3: down(gelu_tanh(gate h) * up h)
+ *   experts                   router_fn 1 (sigmoid scores) with router_norm 0; expert_act 1: down(max(up h, 0)^2), also in the shared expert; router_in 1: an expert reads
+ *                             its weight times h
+ *   shared weights            weights_of j + 1: the layer uses layer j's tensors with a cache or state of its own (every other field equals layer j's) */
+typedef enum tgx_mixer { TGX_MIXER_LATENT_ATTENTION = 1, TGX_MIXER_ATTENTION = 2, TGX_MIXER_MLSTM = 3, TGX_MIXER_WKV = 4, TGX_MIXER_PARALLEL = 5, TGX_MIXER_MAMBA1 = 6, TGX_MIXER_RETENTION = 7, TGX_MIXER_CHANNEL_DELTA = 8 } tgx_mixer;
 typedef enum tgx_mlp { TGX_MLP_NONE = 0, TGX_MLP_MOE = 1, TGX_MLP_DENSE = 2 } tgx_mlp;
 typedef enum tgx_mask { TGX_MASK_CAUSAL = 0, TGX_MASK_WINDOW = 1, TGX_MASK_CHUNK = 2 } tgx_mask;
 
@@ -224,7 +241,7 @@ typedef struct tgx_layer_desc {
   int32_t head_mix;  /* attention: 1 = weights mixed across heads by a [heads][heads] matrix      */
   int32_t gate_kind; /* output gate: 0 = the family's own, 1 = per channel, 2 = per head          */
   int32_t rot_dim;   /* latent attention: rotated query / key dimensions per head beside `dim` (0: none) */
-  int32_t ff_act;    /* dense feed-forward: 0 = the family's own, 1 = erf gelu without a gate, 2 (ABI 8) = squared relu without a gate */
+  int32_t ff_act;    /* dense feed-forward: 0 = the family's own, 1 = erf gelu without a gate, 2 (ABI 8) = squared relu without a gate, 3 (ABI 9) = tanh gelu with a gate */
   int32_t router_fn; /* experts: 0 = softmax scores + correction, 1 = sigmoid scores              */
   int32_t group_score; /* experts: a group counts as 0 = its largest, 1 = the sum of its two largest scores */
   int32_t router_norm; /* experts: 1 = weights divided by their sum + 1e-20                       */
@@ -237,10 +254,19 @@ typedef struct tgx_layer_desc {
   int32_t part_norms; /* state-space mixer: equal parts of its output norm                        */
   int32_t inner;     /* mamba1: channels                                                          */
   int32_t dt_rank;   /* mamba1: inner size of the step sizes' product                             */
+  /* ABI 9 (zero for the kinds that do not read them) */
+  int32_t maps;      /* attention: score maps per head over the same values (0, 1: one)           */
+  float diff;        /*            ... the constant part of the second map's weight                */
+  int32_t gate_rank; /* channel delta: inner size of the output gate's product (0: from the tensors; decay_rank: the decays') */
+  int32_t router_in; /* experts: 1 = a weight multiplies its expert's input instead of its output  */
+  int32_t expert_act; /* experts: 0 = the family's own, 1 = squared relu without a gate            */
+  int32_t weights_of; /* 1 + the layer whose tensors this one uses (0: its own)                    */
+  int32_t n_decays;  /* retention: entries of `decays` (= heads)                                   */
+  const float* decays; /*          ... one decay per head; read during tgx_create_stack only       */
 } tgx_layer_desc;
 
 typedef struct tgx_stack_desc {
-  int32_t family;         /* tgx_family (TGX_FAMILY_ZAKUSUN, TGX_FAMILY_MODEPEL, TGX_FAMILY_VITUDRA, TGX_FAMILY_ZALUVIK, TGX_FAMILY_NUSOVIK) */
+  int32_t family;         /* tgx_family (TGX_FAMILY_ZAKUSUN, TGX_FAMILY_MODEPEL, TGX_FAMILY_VITUDRA, TGX_FAMILY_ZALUVIK, TGX_FAMILY_NUSOVIK, TGX_FAMILY_KERONEX) */
   int32_t width;          /* residual width                                                        */
   int32_t layers;         /* entries of the tgx_layer_desc array                                   */
   int32_t vocab;
@@ -254,11 +280,16 @@ typedef struct tgx_stack_desc {
   int32_t canon_taps;     /* taps of the input convolution (>= 1)                                  */
   float logit_scale;      /* logits = embed . norm(x) * logit_scale                                */
   float residual_mult;    /* ABI 6, TGX_FAMILY_VITUDRA / ZALUVIK: the factor on what a sublayer adds to the stream */
-  /* ABI 7, TGX_FAMILY_ZALUVIK (embed_scale also TGX_FAMILY_NUSOVIK) */
+  /* ABI 7, TGX_FAMILY_ZALUVIK (embed_scale also TGX_FAMILY_NUSOVIK / KERONEX) */
   float embed_scale;      /* x = embed[token] * embed_scale                                         */
   int32_t loop_start;     /* layers loop_start .. loop_stop - 1 run loop_times times (an empty span: no loop) */
   int32_t loop_stop;
   int32_t loop_times;
+  /* ABI 9, TGX_FAMILY_KERONEX */
+  int32_t streams;        /* residual streams (0: one, without learned mixes)                       */
+  int32_t bigram_buckets; /* rows of the pair table without the first token's (0: no pair table)    */
+  int64_t bigram_before;  /* row = (token before * bigram_before + token * bigram_cur) mod bigram_buckets */
+  int64_t bigram_cur;
 } tgx_stack_desc;
 
 /* SamplerConfig (src/engine/Sampler.h:13-22).  Greedy iff temperature<=0 && top_k<=0 &&
@@ -289,7 +320,10 @@ TGX_API int tgx_create(const tgx_model_desc* desc, int device_ordinal, tgx_ctx**
  * TGX_FAMILY_ZALUVIK: "embed", "loop.in" (with a loop), "final.norm(.b)", "l<i>.norm1|norm1b|norm2|norm2b(.b)", attention "l<i>.mix.q|k|v|talk|pb|g|o", latent
  * attention "l<i>.mix.q|dkv|dkv.norm|uk|uv|g|o", dense "l<i>.mlp.up|down", experts "l<i>.mlp.router|e<j>.gate|up|down|shared.gate|up|down".
  * TGX_FAMILY_NUSOVIK: "embed", "head", "final.norm", "l<i>.norm1|norm2", "l<i>.mlp.up|down", mamba1 "l<i>.mix.in|conv(.b)|x|dt(.b)|A_log|D|o", parallel
- * "l<i>.mix.left.q(.b|.norm)|k(.b|.norm)|rel|sink|g|o", "l<i>.mix.right.in|conv(.b)|dt_bias|A_log|D|norm|o". */
+ * "l<i>.mix.left.q(.b|.norm)|k(.b|.norm)|rel|sink|g|o", "l<i>.mix.right.in|conv(.b)|dt_bias|A_log|D|norm|o".
+ * TGX_FAMILY_KERONEX: "embed", "bigram", "head", "final.norm", "l<i>.norm1|norm2", "l<i>.hc1|hc2.in|out|mix", attention "l<i>.mix.q|k|v|lq1|lk1|lq2|lk2|o", retention
+ * "l<i>.mix.q|k|v|g|o", channel delta "l<i>.mix.q|k|v(.conv)|b|A_log|a1|a2|dt_bias|norm|g1|g2|o", dense "l<i>.mlp.gate|up|down", experts
+ * "l<i>.mlp.router|e<j>.up|down|shared.up|down" (none for a layer with weights_of). */
 TGX_API int tgx_create_stack(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int device_ordinal, tgx_ctx** out_ctx);
 
 /* == SafeTensors::loadInternal -> Storage::copyOnDevice for ONE named tensor

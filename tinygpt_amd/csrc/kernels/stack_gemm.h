@@ -14,7 +14,7 @@
 
 namespace tgx {
 
-enum { SG_ACT_NONE = 0, SG_ACT_TANH = 1, SG_ACT_DECAY = 2, SG_ACT_GELU = 3, SG_ACT_SOFTPLUS = 4, SG_ACT_RELU2 = 5 };
+enum { SG_ACT_NONE = 0, SG_ACT_TANH = 1, SG_ACT_DECAY = 2, SG_ACT_GELU = 3, SG_ACT_SOFTPLUS = 4, SG_ACT_RELU2 = 5, SG_ACT_HEAD_DECAY = 6, SG_ACT_GELU_TANH = 7 };
 enum { SG_STORE = 0, SG_ADD = 1, SG_GATE = 2, SG_EXPERT_ACT = 3, SG_ROWSCALE = 4, SG_SILU_MUL = 5 };
 constexpr bool sg_dual(int epi) { return epi == SG_EXPERT_ACT || epi == SG_SILU_MUL; }
 struct StackGemmArgs {
@@ -27,7 +27,11 @@ struct StackGemmArgs {
   int M, N, K;
   float scale;                 // SG_STORE: C = act(acc * scale + bias); SG_ADD: C += acc * scale
   int act;                     // SG_STORE: SG_ACT_NONE, SG_ACT_TANH, SG_ACT_DECAY = exp(-exp(v)) (a decay in (0, 1) from a log-log pre-activation),
-                               //           SG_ACT_GELU = v (1 + erf(v / sqrt 2)) / 2, SG_ACT_SOFTPLUS = ln(1 + e^v), or SG_ACT_RELU2 = max(v, 0)^2
+                               //           SG_ACT_GELU = v (1 + erf(v / sqrt 2)) / 2, SG_ACT_SOFTPLUS = ln(1 + e^v), SG_ACT_RELU2 = max(v, 0)^2, or SG_ACT_HEAD_DECAY =
+                               //           exp(-exp(a_log[n / head_cols]) ln(1 + e^v)) (a decay per channel whose rate has a factor per head)
+                               // SG_SILU_MUL: SG_ACT_GELU_TANH takes the tanh form of gelu instead of silu
+  const float* a_log; int head_cols;
+  const float* in_w; const int* in_rows;         // SG_STORE: row m's product is first multiplied by in_w[in_rows[m]] (a router weight on its expert's input; nullptr: none)
   const float* bias;           // SG_STORE: [N] per z (column z * c_zoff + n), nullptr: none
   int gate_col0, gate_heads;   // SG_STORE: columns [gate_col0, + gate_heads) leave as log input gates cap tanh(v / cap), the next gate_heads columns as log forget gates
   float gate_cap;              //           logsigmoid(cap tanh(v / cap)) (the two gate rows of a matrix-memory layer's input product); gate_heads 0: none
@@ -53,11 +57,15 @@ __device__ __forceinline__ float store_value(const StackGemmArgs& a, float v, si
   else if (a.act == SG_ACT_DECAY) o = expf(-expf(o));
   else if (a.act == SG_ACT_SOFTPLUS) o = o > 20.f ? o : log1pf(expf(o));
   else if (a.act == SG_ACT_RELU2) { o = fmaxf(o, 0.f); o *= o; }
+  else if (a.act == SG_ACT_HEAD_DECAY) o = expf(-expf(a.a_log[n / a.head_cols]) * (o > 20.f ? o : log1pf(expf(o))));
   else if (a.act == SG_ACT_GELU) o = 0.5f * o * (1.0f + erff(o * 0.70710678118654752f));
   return o;
 }
 // the plain gated expert: silu(gate) * up
 __device__ __forceinline__ float silu_mul(float gate, float up) { return gate / (1.0f + expf(-gate)) * up; }
+__device__ __forceinline__ float gelu_tanh(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * fmaf(0.044715f * z * z, z, z))); }
+// the product of a gated feed-forward's two halves: silu or (act SG_ACT_GELU_TANH) the tanh gelu of the gate
+__device__ __forceinline__ float gate_mul(const StackGemmArgs& a, float gate, float up) { return a.act == SG_ACT_GELU_TANH ? gelu_tanh(gate) * up : silu_mul(gate, up); }
 
 template <int DT, int EPI, bool DUAL, int WT, bool VEC>
 __global__ __launch_bounds__(256) void stack_gemm_kernel(const StackGemmArgs a) {
@@ -236,16 +244,17 @@ __global__ __launch_bounds__(256) void stack_gemm_kernel(const StackGemmArgs a) 
       if (m >= mend) continue;
       const size_t crow = a.c_rows ? (size_t)a.c_rows[m] : (size_t)m;
       float* cp = a.C + crow * a.ldc + (size_t)z * a.c_zoff;
+      const float in_w = EPI == SG_STORE && a.in_w ? a.in_w[a.in_rows[m]] : 1.f;
 #pragma unroll
       for (int j = 0; j < WT; j++) {
         const int n = n0 + wn * (32 * WT) + j * 32 + (lane & 31);
         if (n >= a.N) continue;
         const float v = acc[0][i][j][r];
-        if constexpr (EPI == SG_STORE) cp[n] = store_value(a, v, (size_t)z * a.c_zoff + n, n);
+        if constexpr (EPI == SG_STORE) cp[n] = store_value(a, a.in_w ? v * in_w : v, (size_t)z * a.c_zoff + n, n);
         else if constexpr (EPI == SG_ADD) cp[n] = fmaf(v, a.scale, cp[n]);
         else if constexpr (EPI == SG_GATE) cp[n] = v / (1.0f + expf(-a.G[crow * a.ldg + a.g_col0 + (a.g_per_z ? (size_t)z : (size_t)z * a.c_zoff + n)]));
         else if constexpr (EPI == SG_EXPERT_ACT) cp[n] = expert_act(v, acc[NB - 1][i][j][r], a.limit);
-        else if constexpr (EPI == SG_SILU_MUL) cp[n] = silu_mul(v, acc[NB - 1][i][j][r]);
+        else if constexpr (EPI == SG_SILU_MUL) cp[n] = gate_mul(a, v, acc[NB - 1][i][j][r]);
         else cp[n] = v * a.rw[crow];
       }
     }
@@ -334,16 +343,17 @@ __global__ __launch_bounds__(256) void stack_gemv_kernel(const StackGemmArgs a) 
     if (m >= mend) break;
     const size_t crow = a.c_rows ? (size_t)a.c_rows[m] : (size_t)m;
     float* cp = a.C + crow * a.ldc + (size_t)z * a.c_zoff;
+    const float in_w = EPI == SG_STORE && a.in_w ? a.in_w[a.in_rows[m]] : 1.f;
 #pragma unroll
     for (int j = 0; j < NC; j++) {
       const int n = n0 + j;
       if (n >= a.N) break;
       const float v = acc[0][j][r];
-      if constexpr (EPI == SG_STORE) cp[n] = store_value(a, v, (size_t)z * a.c_zoff + n, n);
+      if constexpr (EPI == SG_STORE) cp[n] = store_value(a, a.in_w ? v * in_w : v, (size_t)z * a.c_zoff + n, n);
       else if constexpr (EPI == SG_ADD) cp[n] = fmaf(v, a.scale, cp[n]);
       else if constexpr (EPI == SG_GATE) cp[n] = v / (1.0f + expf(-a.G[crow * a.ldg + a.g_col0 + (a.g_per_z ? (size_t)z : (size_t)z * a.c_zoff + n)]));
       else if constexpr (EPI == SG_EXPERT_ACT) cp[n] = expert_act(v, acc[NB - 1][j][r], a.limit);
-      else if constexpr (EPI == SG_SILU_MUL) cp[n] = silu_mul(v, acc[NB - 1][j][r]);
+      else if constexpr (EPI == SG_SILU_MUL) cp[n] = gate_mul(a, v, acc[NB - 1][j][r]);
       else cp[n] = v * a.rw[crow];
     }
   }

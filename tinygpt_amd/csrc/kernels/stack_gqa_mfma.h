@@ -27,6 +27,7 @@ struct GqaMfmaArgs {
   float* out; long long ldo;           // [T][heads * vdim]
   float* part; int nsplit, keys_per;   // keys_per: a multiple of 64
   int heads, kv_heads, dim, vdim, terms;
+  int maps = 1;                        // score maps over the same values (GqaAttnArgs)
   float scale, sink; int has_sink;
   int mask_kind, mask_size;            // MASK_* (stack_meta.h): a row sees the keys [first_key(position), position]
   float softcap; int dist_bias;        // score shaping as in gqa_attn_kernel (softcap <= 0: none)
@@ -45,7 +46,8 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
   __shared__ float s_part[4][32][65];
   __shared__ __attribute__((aligned(16))) bf16_t s_ph[32][72], s_pl[32][72];
   __shared__ float s_corr[32], s_l[32];
-  const int e = blockIdx.y / a.kv_heads, kvh = blockIdx.y - e * a.kv_heads, Gq = a.heads / a.kv_heads;
+  const int e = blockIdx.y / a.kv_heads, kvh = blockIdx.y - e * a.kv_heads, Gq = a.heads / a.kv_heads, vh = kvh / a.maps;
+  auto head = [&](int r) -> int { return (vh * Gq + r % Gq) * a.maps + kvh - vh * a.maps; };      // the query head of row r: the group's heads, this workgroup's map of each
   const int cnt = m.ent_count[e], start = m.ent_start[e], slot = m.ent_row[e];
   const int nrows = cnt * Gq, r0 = blockIdx.x * 32;
   if (r0 >= nrows) return;
@@ -55,7 +57,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
   const int klo = first_key(past + r0 / Gq, a.mask_kind, a.mask_size) & ~63;      // the tile's first row sees the oldest key; whole key tiles
   int k0 = klo, k1 = kmax;
   if (SPLIT) { k0 = min(kmax, klo + (int)blockIdx.z * a.keys_per); k1 = min(kmax, k0 + a.keys_per); }
-  const int page = 1 << m.page_shift, kd = a.kv_heads * a.dim, vd = a.kv_heads * a.vdim;
+  const int page = 1 << m.page_shift, kd = a.kv_heads * a.dim, vd = a.kv_heads / a.maps * a.vdim;
   const bf16_t* poolK = reinterpret_cast<const bf16_t*>(a.poolK) + (size_t)kvh * a.dim;
   const bf16_t* poolVT = reinterpret_cast<const bf16_t*>(a.poolVT);
 
@@ -63,7 +65,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
   bf16x8 qh[KS], ql[KS];
   {
     const int r = r0 + l31, rc = min(r, nrows - 1);
-    const float* qp = a.q + (size_t)(start + rc / Gq) * a.ldq + (size_t)(kvh * Gq + rc % Gq) * a.dim + wv * RQ + 8 * half;
+    const float* qp = a.q + (size_t)(start + rc / Gq) * a.ldq + (size_t)head(rc) * a.dim + wv * RQ + 8 * half;
 #pragma unroll
     for (int kk = 0; kk < KS; kk++) {
       const f32x4 v0 = *reinterpret_cast<const f32x4*>(qp + 16 * kk), v1 = *reinterpret_cast<const f32x4*>(qp + 16 * kk + 4);
@@ -88,10 +90,10 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
   const bool svalid = sr < nrows;
   const int skeys = svalid ? past + sr / Gq + 1 : 0;
   const int slo = first_key(skeys - 1, a.mask_kind, a.mask_size);
-  const float slope2 = a.dist_bias && svalid ? distance_slope(kvh * Gq + sr % Gq, a.heads) * LOG2E : 0.f;
-  const float* dist = a.dist_tab && svalid ? a.dist_tab + (size_t)(kvh * Gq + sr % Gq) * a.dist_len : nullptr;
+  const float slope2 = a.dist_bias && svalid ? distance_slope(head(sr), a.heads) * LOG2E : 0.f;
+  const float* dist = a.dist_tab && svalid ? a.dist_tab + (size_t)head(sr) * a.dist_len : nullptr;
   const bool sinked = (a.has_sink || a.sinks) && svalid && (!SPLIT || blockIdx.z == 0);
-  float m_s = sinked ? (a.sinks ? a.sinks[kvh * Gq + sr % Gq] : a.sink) * LOG2E : -INFINITY, l_s = sinked ? 1.f : 0.f;      // the running maximum in base-2 units
+  float m_s = sinked ? (a.sinks ? a.sinks[head(sr)] : a.sink) * LOG2E : -INFINITY, l_s = sinked ? 1.f : 0.f;      // the running maximum in base-2 units
 
   auto key_rows = [&](int kt) -> const bf16_t* {
     const size_t pg = (size_t)m.tbl[(size_t)slot * m.tbl_stride + (kt >> m.page_shift)];
@@ -110,7 +112,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
 #pragma unroll
     for (int t = 0; t < NT; t++) {
       const int col = min(wv * 32 * NT + 32 * t + l31, a.vdim - 1);
-      const bf16_t* tp = poolVT + ((pg * vd + (size_t)(kvh * a.vdim + col)) << m.page_shift) + off + 8 * half;
+      const bf16_t* tp = poolVT + ((pg * vd + (size_t)(vh * a.vdim + col)) << m.page_shift) + off + 8 * half;
 #pragma unroll
       for (int kk = 0; kk < 4; kk++) bt[t][kk] = *reinterpret_cast<const u32x4*>(tp + 16 * kk);
     }
@@ -202,7 +204,7 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
     }
   }
   auto rec_of = [&](int gr) -> float* {      // the split record of row gr: indexed by (token, head) like the lane kernel's
-    return a.part + (((size_t)(start + gr / Gq) * a.heads + (size_t)(kvh * Gq + gr % Gq)) * a.nsplit + blockIdx.z) * (size_t)(a.vdim + 2);
+    return a.part + (((size_t)(start + gr / Gq) * a.heads + (size_t)head(gr)) * a.nsplit + blockIdx.z) * (size_t)(a.vdim + 2);
   };
   if ((lane & 7) == 0) {
     s_l[srow] = l_s;
@@ -217,9 +219,9 @@ __global__ __launch_bounds__(256) void gqa_attn_mfma_kernel(StepMeta m, GqaMfmaA
       if (gr >= nrows || col >= a.vdim) continue;
       if (SPLIT) rec_of(gr)[2 + col] = acc[t][r];
       else {
-        const size_t tok = (size_t)(start + gr / Gq), hc = (size_t)(kvh * Gq + gr % Gq) * a.vdim + col;
+        const size_t tok = (size_t)(start + gr / Gq), hc = (size_t)head(gr) * a.vdim + col;
         float v = s_l[ri] > 0.f ? acc[t][r] / s_l[ri] : 0.f;
-        if (a.gate) v = v / (1.0f + expf(-a.gate[tok * a.ldg + (a.gate_per_head ? (size_t)(kvh * Gq + gr % Gq) : hc)]));
+        if (a.gate) v = v / (1.0f + expf(-a.gate[tok * a.ldg + (a.gate_per_head ? (size_t)head(gr) : hc)]));
         a.out[tok * a.ldo + hc] = v * a.out_scale;
       }
     }

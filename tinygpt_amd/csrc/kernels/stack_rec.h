@@ -4,11 +4,13 @@
 //   offset_norm_kernel      rows / sqrt(mean(row^2) + eps) * (offset + w): an RMS norm whose weight is stored as its distance from `offset`
 //   token_shift_kernel      the n mixes h + (h_before - h) * mu_s of a token-shift layer, and the slot's last row
 //   delta_prep_kernel       causal depth-wise convolution + silu on the q | k | v projections of a gated-delta-rule layer (tails per slot), unit q and k per
-//                           head, beta = sigmoid, decay = exp(-exp(A_log) * softplus(a + dt_bias))
+//                           head, beta = sigmoid, decay = exp(-exp(A_log) * softplus(a + dt_bias)) (where the layer has one decay per head)
 //   rec_scan_kernel         the recurrence over an entry's tokens with the head's matrix state in registers:
 //                             REC_WKV     o = (S + diag(u) k v^T)^T r;  S <- diag(w) S + k v^T
 //                             REC_DELTA   S <- g S;  S += k (beta (v - S^T k))^T;  o = S^T q
-//                             REC_SSD     S <- g S + k (beta v)^T;  o = S^T q + skip v (a scalar-decay state-space recurrence)
+//                             REC_SSD     S <- g S + k (beta v)^T;  o = S^T q + skip v (a scalar-decay state-space recurrence; with `fixed`, a retention:
+//                                         the decay is a number per head and beta one number)
+//                             REC_CDELTA  S <- diag(w) S;  S += k (beta (v - S^T k))^T;  o = S^T q (the delta rule with one decay per head and key channel)
 // A sequence whose first token has position 0 starts from zero state whatever its slot held.
 #pragma once
 #include "stack.h"
@@ -52,13 +54,14 @@ __global__ __launch_bounds__(256) void token_shift_kernel(StepMeta m, TokenShift
 // ---- inputs of a gated-delta-rule layer.  proj row = [.. | q (G D) | k (G D) | v (H E) | b (H) | a (H) | ..] from column col0; the C = 2 G D + H E
 // convolved channels take taps weights each (last = the current token's); the taps - 1 rows before come from the step's own rows, the slot's tails (raw
 // projections, double-buffered by step parity like the other per-slot rows) or are zero before the sequence's start.
-// out row = [q | k | v | beta | decay]: q, k unit vectors per head (x / sqrt(sum x^2 + unit_eps)), q times q_scale.
+// out row = [q | k | v | beta | decay]: q, k unit vectors per head (x / sqrt(sum x^2 + unit_eps)), q times q_scale.  The b columns stand at b_col (from col0); a layer
+// without a_log has no scalar decays (neither a columns nor decay outputs).
 // Grid: (tokens, 2 G + H + 1): one workgroup per q head, k head (D <= 256 channels, one per thread, and their norm), v head, and one for the H gates.
 constexpr int DELTA_MAX_TAPS = 64;      // (bounds the per-slot tails, not the kernel: it loops over the taps)
 struct DeltaPrepArgs {
-  const float* proj; long long ldp; int col0;
+  const float* proj; long long ldp; int col0, b_col;
   const float* cw;       // [C][taps]
-  const float* a_log;    // [H]
+  const float* a_log;    // [H] (nullptr: no scalar decays)
   const float* dt_bias;  // [H]
   float* out; long long ldo;
   float* state;          // [2][slots][taps - 1][C] (nullptr when taps == 1)
@@ -74,9 +77,10 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(StepMeta m, DeltaPrepAr
   float* __restrict__ o = a.out + (size_t)t * a.ldo;
   if (u == G2 + a.heads) {
     for (int h = threadIdx.x; h < a.heads; h += 256) {
-      const float zb = pr[C + h], za = pr[C + a.heads + h] + a.dt_bias[h];
+      o[C + h] = 1.0f / (1.0f + expf(-pr[a.b_col + h]));
+      if (!a.a_log) continue;
+      const float za = pr[a.b_col + a.heads + h] + a.dt_bias[h];
       const float sp = za > 20.f ? za : log1pf(expf(za));
-      o[C + h] = 1.0f / (1.0f + expf(-zb));
       o[C + a.heads + h] = expf(-expf(a.a_log[h]) * sp);
     }
     return;
@@ -116,15 +120,16 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(StepMeta m, DeltaPrepAr
 // inputs (up to three vectors of `dim`) and the workgroup's value columns are staged in LDS (the next block's travel in registers meanwhile), then every
 // lane updates its DPER rows of its column with no barrier inside the block: a wave owns 8 columns, its lanes = 8 columns x 8 row groups (the row groups
 // of a column are adjacent lanes), 8 DPER >= dim.  Sums over the key channels cross the row groups on the lane crossbar.
-enum { REC_WKV = 0, REC_DELTA = 1, REC_SSD = 2 };
+enum { REC_WKV = 0, REC_DELTA = 1, REC_SSD = 2, REC_CDELTA = 3 };
 struct RecScanArgs {
   const float* a; long long lda;     // per token and key head [dim]: the read vector (wkv: r, delta: q, ssd: C)
   const float* k; long long ldk;     //                               k (ssd: B)
-  const float* w; long long ldw;     //                               wkv: the decay per channel
+  const float* w; long long ldw;     //                               wkv: the decay per channel; cdelta: per (query) head and channel
   const float* v; long long ldv;     // per token and head [vdim]
-  const float* beta; const float* g; long long ldg;      // delta, ssd: per token and head
+  const float* beta; const float* g; long long ldg;      // delta, ssd: per token and head (cdelta: beta alone)
+  const float* fixed; float beta0;   // ssd: [heads] decays that hold for every token, with beta0 as every token's beta (nullptr: beta and g)
   const float* u;                    // wkv: [heads][dim] bonus
-  const float* skip;                 // ssd: [heads]
+  const float* skip;                 // ssd: [heads] (nullptr: none)
   float* S;                          // [slots][heads][dim][vdim]
   float* out; long long ldo;         // [T][heads * vdim]
   int heads, kv_heads, dim, vdim;
@@ -133,7 +138,7 @@ constexpr int REC_RG = 8, REC_COLS = 4 * (64 / REC_RG);      // row groups per c
 template <int DPER, int KIND>
 __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a) {
   constexpr int RG = REC_RG, CW = 64 / RG, CB = REC_COLS, LP = DPER + 4, DP = RG * DPER, TB = DP <= 128 ? 16 : 8;      // LP: a row group's LDS stride (the groups' reads fall into different banks)
-  constexpr int NQ = TB * DP / 256, NV = (TB * CB + 255) / 256, NA = KIND == REC_WKV ? 3 : 2;
+  constexpr int NQ = TB * DP / 256, NV = (TB * CB + 255) / 256, NA = KIND == REC_WKV || KIND == REC_CDELTA ? 3 : 2;
   __shared__ __attribute__((aligned(16))) float s_in[NA][TB][RG * LP];      // [0]: the read vector, [1]: k, [2]: the decay
   __shared__ float s_v[TB][CB], s_b[TB], s_g[TB];
   const int e = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, rg = lane % RG, cl = lane / RG;
@@ -143,7 +148,7 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
   const int kh = h / (a.heads / a.kv_heads), d0 = rg * DPER, l0 = rg * LP;
   const bool col = j < a.vdim;
   float* Sg = a.S + ((size_t)row * a.heads + h) * (size_t)a.dim * a.vdim;
-  const float skip = KIND == REC_SSD ? a.skip[h] : 0.f;
+  const float skip = KIND == REC_SSD && a.skip ? a.skip[h] : 0.f;
   float S[DPER], ub[KIND == REC_WKV ? DPER : 1];
 #pragma unroll
   for (int dd = 0; dd < DPER; dd++) {
@@ -162,14 +167,18 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
       const bool on = t < nb && d < a.dim;
       const size_t tok = (size_t)(start + t0 + min(t, nb - 1));
 #pragma unroll
-      for (int s = 0; s < NA; s++) rin[s][u] = on ? src[s][tok * lds[s] + (size_t)kh * a.dim + d] : 0.f;
+      for (int s = 0; s < NA; s++) rin[s][u] = on ? src[s][tok * lds[s] + (size_t)(KIND == REC_CDELTA && s == 2 ? h : kh) * a.dim + d] : 0.f;
     }
 #pragma unroll
     for (int u = 0; u < NV; u++) {
       const int i = tid + 256 * u, t = i / CB, c = i - t * CB;
       rv[u] = (t < nb && blockIdx.z * CB + c < a.vdim) ? a.v[(size_t)(start + t0 + t) * a.ldv + (size_t)h * a.vdim + blockIdx.z * CB + c] : 0.f;
     }
-    if (KIND != REC_WKV && tid < nb) { rb = a.beta[(size_t)(start + t0 + tid) * a.ldg + h]; rgt = a.g[(size_t)(start + t0 + tid) * a.ldg + h]; }
+    if (KIND != REC_WKV && tid < nb) {
+      const size_t at = (size_t)(start + t0 + tid) * a.ldg + h;
+      if (KIND == REC_SSD && a.fixed) { rb = a.beta0; rgt = a.fixed[h]; }
+      else { rb = a.beta[at]; if (KIND != REC_CDELTA) rgt = a.g[at]; }
+    }
   };
   fetch(0);
   for (int t0 = 0; t0 < cnt; t0 += TB) {
@@ -213,7 +222,7 @@ __global__ __launch_bounds__(256) void rec_scan_kernel(StepMeta m, RecScanArgs a
       } else {
         float pk = 0.f;
 #pragma unroll
-        for (int dd = 0; dd < DPER; dd++) { S[dd] *= k.g; pk = fmaf(S[dd], k.in[1][dd / 4][dd & 3], pk); }
+        for (int dd = 0; dd < DPER; dd++) { S[dd] *= KIND == REC_CDELTA ? k.in[NA - 1][dd / 4][dd & 3] : k.g; pk = fmaf(S[dd], k.in[1][dd / 4][dd & 3], pk); }
         pk = row_group_sum<RG>(pk);
         const float uj = k.b * (k.v - pk);
 #pragma unroll

@@ -119,6 +119,7 @@ struct GqaAppendArgs {
   int rot_pairs;             // 1: neighbours turn together
   float q_temp_coef; int q_temp_every;      // coef 0: no query temperature
   float qk_unit_eps;         // > 0: every q and k head is first divided by sqrt(mean(head^2) + qk_unit_eps) (no weight)
+  int maps = 1;              // key heads per value head (heads and kv_heads count every map: GqaAttnArgs)
   unsigned short *q_hi, *q_lo;      // [T][heads * dim] (nullptr: not kept): the finished queries as two 16-bit terms, the A operand of a matrix-core score product
 };
 template <int DT>
@@ -163,7 +164,7 @@ __global__ __launch_bounds__(256) void gqa_append_kernel(StepMeta m, GqaAppendAr
   __syncthreads();
   const int page = m.tbl[(size_t)m.tok_row[t] * m.tbl_stride + (pos >> m.page_shift)];
   const size_t slot = ((size_t)page << m.page_shift) + (size_t)(pos & ((1 << m.page_shift) - 1));
-  const int kd = a.kv_heads * a.dim, vd = a.kv_heads * a.vdim;
+  const int kd = a.kv_heads * a.dim, vd = a.kv_heads / a.maps * a.vdim;
   elem_t<DT>* kdst = reinterpret_cast<elem_t<DT>*>(a.poolK) + slot * kd;
   elem_t<DT>* vdst = reinterpret_cast<elem_t<DT>*>(a.poolV) + slot * vd;
   const float* ksrc = row + (size_t)a.heads * a.dim;
@@ -238,6 +239,8 @@ struct GqaAttnArgs {
   const float* gate; long long ldg;    // gate pre-activation of (t, h, c) at gate + t * ldg + h * vdim + c (nullptr: none)
   float* out; long long ldo;           // [T][heads * vdim]
   int heads, kv_heads, dim, vdim;
+  int maps = 1;                        // score maps over the same values (differential attention: 2): head h is map h % maps of query head h / maps, the keys hold maps rows of dim
+                                       // per value head; heads and kv_heads count every map, and every map leaves an output of its own
   float scale, sink; int has_sink;
   float* part; int nsplit, keys_per;   // split form: records (m, l, acc[vdim]) per (token, head, split); split z takes keys_per keys from first_key on
   int mask_kind, mask_size;            // MASK_*
@@ -261,7 +264,7 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(StepMeta m, GqaAttnArgs a
   extern __shared__ float s_acc[];      // [4][vdim]
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
   const int row = m.tok_row[t], nkeys = m.tok_pos[t] + 1;
-  const int kvh = h / (a.heads / a.kv_heads), kd = a.kv_heads * a.dim, vd = a.kv_heads * a.vdim;
+  const int vh = h / a.maps / (a.heads / a.kv_heads), kh = vh * a.maps + h % a.maps, kd = a.kv_heads * a.dim, vd = a.kv_heads / a.maps * a.vdim;
   int k0 = first_key(nkeys - 1, a.mask_kind, a.mask_size), k1 = nkeys;
   if (SPLIT) { k0 = min(nkeys, k0 + (int)blockIdx.z * a.keys_per); k1 = min(nkeys, k0 + a.keys_per); }
   const float slope = a.dist_bias ? distance_slope(h, a.heads) : 0.f;
@@ -272,8 +275,8 @@ __global__ __launch_bounds__(256) void gqa_attn_kernel(StepMeta m, GqaAttnArgs a
   const float* dist = a.dist_tab ? a.dist_tab + (size_t)h * a.dist_len : nullptr;
   const bool sink_here = (a.has_sink || a.sinks) && wv == 0 && (!SPLIT || blockIdx.z == 0);      // the sink enters once
   float mx = sink_here ? (a.sinks ? a.sinks[h] : a.sink) : -INFINITY, l = sink_here ? 1.f : 0.f;
-  const elem_t<DT>* pk = reinterpret_cast<const elem_t<DT>*>(a.poolK) + (size_t)kvh * a.dim;
-  const elem_t<DT>* pv = reinterpret_cast<const elem_t<DT>*>(a.poolV) + (size_t)kvh * a.vdim;
+  const elem_t<DT>* pk = reinterpret_cast<const elem_t<DT>*>(a.poolK) + (size_t)kh * a.dim;
+  const elem_t<DT>* pv = reinterpret_cast<const elem_t<DT>*>(a.poolV) + (size_t)vh * a.vdim;
   const int pmask = (1 << m.page_shift) - 1;
   for (int j = k0 + wv; j < k1; j += 4) {
     const int page = m.tbl[(size_t)row * m.tbl_stride + (j >> m.page_shift)];
@@ -483,7 +486,7 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(StepMeta m, MlstmArgs a
 }
 
 // out[t][h][c] = hs / sqrt(mean_c(hs^2) + eps) * w[h * w_hstride + c] * gate, gate = sigmoid(z) or silu(z) of the pre-activation z (w_hstride 0: one
-// weight vector for all heads).  One wave per (token, head): the seam behind every recurrent mixer (mLSTM, wkv, gated delta rule).
+// weight vector for all heads; w nullptr: none).  One wave per (token, head): the seam behind every recurrent mixer (mLSTM, wkv, gated delta rule, retention).
 struct HeadNormGateArgs { const float* hs; long long ldh; const float* w; int w_hstride; const float* gate; long long ldg; int silu_gate; float* out; long long ldo; int vdim; float eps; };
 __global__ __launch_bounds__(64) void head_norm_gate_kernel(HeadNormGateArgs a) {
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -494,7 +497,7 @@ __global__ __launch_bounds__(64) void head_norm_gate_kernel(HeadNormGateArgs a) 
   const float rinv = 1.0f / sqrtf(ss / (float)a.vdim + a.eps);
   for (int c = lane; c < a.vdim; c += 64) {
     const float g = a.gate[(size_t)t * a.ldg + (size_t)h * a.vdim + c], sg = 1.0f / (1.0f + expf(-g));
-    a.out[(size_t)t * a.ldo + (size_t)h * a.vdim + c] = r[c] * rinv * a.w[(size_t)h * a.w_hstride + c] * (a.silu_gate ? g * sg : sg);
+    a.out[(size_t)t * a.ldo + (size_t)h * a.vdim + c] = r[c] * rinv * (a.w ? a.w[(size_t)h * a.w_hstride + c] : 1.0f) * (a.silu_gate ? g * sg : sg);
   }
 }
 

@@ -17,7 +17,8 @@ struct SsdArgs {
   const float* row; long long ld;      // per token [x (heads E) | B (groups N) | C (groups N) | dt (heads) | decay (heads) | log decay (heads)]
   int heads, groups, N, E;             // N and heads E multiples of 4
   float* gram;                         // [blocks][groups][64][64]
-  const float* skip;                   // [heads]
+  const float* fixed; float dt0;       // [2][heads] decays and their logarithms that hold for every token, with dt0 as every token's dt (the rows then end behind C; nullptr: per token)
+  const float* skip;                   // [heads] (nullptr: none)
   float* S;                            // [slots][heads][N][E]
   float* out; long long ldo;           // [T][heads E]
 };
@@ -125,7 +126,7 @@ __global__ __launch_bounds__(256, NW == 1 ? 2 : 1) void ssd_block_kernel(StepMet
     const int left = cnt - b * Q;
 #pragma unroll
     for (int u = 0; u < 8; u++) x[u] = *at(p, row_off(tid >> 5, 8 * u, left) + 4 * (oX + xcol));
-    if (wv == 0) { const unsigned int off = row_off(lane, 0, left); dt = *at(p + oD, off); la = *at(p + oL, off); }
+    if (wv == 0 && !a.fixed) { const unsigned int off = row_off(lane, 0, left); dt = *at(p + oD, off); la = *at(p + oL, off); }
   };
   auto stage = [&](int b) {
     const int buf = b & 1, left = cnt - b * Q;
@@ -140,7 +141,8 @@ __global__ __launch_bounds__(256, NW == 1 ? 2 : 1) void ssd_block_kernel(StepMet
       s_cs[buf][lane] = v; s_dt[buf][lane] = d; s_end[buf][lane] = d * __builtin_amdgcn_exp2f((float)(end - v));
     }
   };
-  const float Dh = a.skip[h];
+  if (a.fixed) { dt = a.dt0; la = a.fixed[a.heads + h]; }
+  const float Dh = a.skip ? a.skip[h] : 0.f;
   const int nblk = (cnt + Q - 1) / Q;
   fetch_x(0); fetch_C(0); fetch_G(0);
   stage(0);

@@ -61,6 +61,17 @@ struct StackLayerW {
   //             a_log, dt_bias, d_skip, head_w (the weight of the part norm) of the right half, mS its state [slots][d_heads][d_dim][d_vdim]
   float *conv_b = nullptr, *d_skip = nullptr, *decay2 = nullptr, *q_norm = nullptr, *k_norm = nullptr, *dist = nullptr;
   int dist_len = 0;
+  // hyper-connected designs (Keronex).  norm1 / norm2 in front of the mixer and the feed-forward (distances from one), hc the two sublayers' stream weights
+  // [in (n) | out (n) | mix (n x n)] each; dense: w_gate / w_up / w_down; experts: w_router (fp32), w_up / w_down stacked, ws_up / ws_down the shared expert
+  //   attention:     w_in = [q (head, map) | k (key / value head, map) | v] rows, lambda the second map's weight (from lam_host at finalize)
+  //   retention:     w_in = [v | k | q | gate] rows, decays [2][heads]: the heads' decays and their logarithms; mS the state [slots][heads][dim][vdim]
+  //   channel delta: w_in = [q | k | v | decays' first product | gate's first product | b] rows (put together at finalize from w_in, w_w1, w_g1 and w_b), w_w2 / w_g2 the second
+  //                  products, conv_w, a_log, dt_bias [heads * dim], head_w the weight all heads share; mS the state, conv_state the tails of the raw q | k | v columns
+  int w_src = -1;               // the layer whose weights this one uses: every pointer but the caches and states is borrowed
+  float *hc = nullptr, *decays = nullptr;
+  ebyte *w_b = nullptr, *w_g1 = nullptr, *w_g2 = nullptr;
+  float lambda = 0.f;
+  std::vector<std::vector<float>> lam_host;
 };
 
 // one run of a layer (layer-norm designs): which layer's weights, whether the loop's input product comes first, and the run's own cache
@@ -85,7 +96,11 @@ struct StackModel {
   bool joint = false;                  // one offset-weight RMS norm per layer; mixer and feed-forward read it side by side; x += residual_mult * (their sum); a separate head
   bool affine = false;                 // layer norms (weight and bias) before and after every sublayer, x += residual_mult * norm(sublayer(norm(x))); a looped span; logits against the embedding table
   bool post = false;                   // RMS norms (with weight) behind the sublayers only, x += norm(sublayer(x)); scaled embedding rows plus a position vector; a separate head
-  bool latent() const { return !sandwich && !joint && !affine && !post; }      // the first layered design: grouped norms, input convolutions, depth average
+  bool hyper = false;                  // several residual streams joined by learned mixes, offset-weight RMS norms in front of the sublayers; pair embedding; a separate head
+  bool latent() const { return !sandwich && !joint && !affine && !post && !hyper; }      // the first layered design: grouped norms, input convolutions, depth average
+  int n_streams() const { return d.streams > 0 ? d.streams : 1; }
+  ebyte* pair = nullptr;               // hyper designs: [bigram_buckets + 1][width] (nullptr: none)
+  int* last_tok = nullptr;             // hyper designs: [2][slots], the slot's last token
   std::vector<StackRun> runs;          // affine designs: the layers in the order they run
   ebyte* w_loop = nullptr;             // [width][2 width]: the loop's input product on [x; x0]
   float* xcat = nullptr;               // step workspace [T][2 width]: the stream beside the embedding output

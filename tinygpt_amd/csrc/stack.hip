@@ -20,6 +20,7 @@
 #include "kernels/stack_mix_mfma.h"
 #include "kernels/stack_ssm.h"
 #include "kernels/stack_ssd_mfma.h"
+#include "kernels/stack_hyper.h"
 
 int upload_param_ext(tgx_ctx* c, ebyte* dst, const void* host, int64_t n, int src_dtype);      // abi.hip
 
@@ -186,9 +187,10 @@ int ensure_ws(tgx_ctx* c, int T) {
   } else if (sm->affine) {   // the seam's scratch row, the shared expert's row, the stream beside the embedding output
     if ((rc = dev_alloc(c, &sm->ytmp, n * W)) || (rc = dev_alloc(c, &sm->ysh, n * W)) || (rc = dev_alloc(c, &sm->xcat, 2 * n * W)) ||
         (rc = dev_alloc(c, &sm->qplanes, 2 * n * (size_t)std::max(1, sm->max_qd) + 8))) return rc;
-  } else if (sm->joint || sm->post) {    // the recurrent mixers' side buffers: un-normed outputs, token-shift mixes, low-rank inner products, the recurrences' inputs
+  } else if (sm->joint || sm->post || sm->hyper) {    // the recurrent mixers' side buffers: un-normed outputs, token-shift mixes, low-rank inner products, the recurrences' inputs
     if ((rc = dev_alloc(c, &sm->hs, n * (size_t)std::max(1, sm->max_hv))) || (rc = dev_alloc(c, &sm->mixed, n * (size_t)std::max(1, sm->max_shift))) ||
         (rc = dev_alloc(c, &sm->lora, n * (size_t)std::max(1, sm->max_lora))) || (rc = dev_alloc(c, &sm->rec_in, n * (size_t)std::max(1, sm->max_rec)))) return rc;
+    if (sm->hyper && ((rc = dev_alloc(c, &sm->xs, n * (size_t)sm->n_streams() * W)) || (rc = dev_alloc(c, &sm->ysh, n * W)))) return rc;
   } else if ((rc = dev_alloc(c, &sm->xs, (size_t)(sm->d.layers + 1) * n * W))) return rc;
   if ((rc = dev_alloc(c, &sm->x, n * W)) || (rc = dev_alloc(c, &sm->a, n * W)) ||
       (rc = dev_alloc(c, &sm->proj, n * (size_t)sm->max_in)) || (rc = dev_alloc(c, &sm->ql, n * (size_t)sm->max_hr)) || (rc = dev_alloc(c, &sm->lat, n * (size_t)sm->max_hr)) ||
@@ -362,12 +364,13 @@ struct GqaSpec {
   const float* sinks; const float* dist; int dist_len;         // per-head sinks, distance table
   int gate_per_head;
   float out_scale = 1.0f;
+  int maps = 1;                                                // score maps over the same values (heads and kv_heads count every map)
 };
 int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, int S, int max_keys, int max_count) {
   StackModel* sm = c->stack;
   const int H = sp.heads, G = sp.kv_heads;
   tgx::GqaAppendArgs ap{};
-  ap.proj = sp.proj; ap.ldp = sp.ldp; ap.heads = H; ap.kv_heads = G; ap.dim = sp.dim; ap.vdim = sp.vdim; ap.rot_dims = sp.cs ? sp.rot_dims : 0; ap.rot_pairs = sp.rot_pairs;
+  ap.proj = sp.proj; ap.ldp = sp.ldp; ap.heads = H; ap.kv_heads = G; ap.maps = sp.maps; ap.dim = sp.dim; ap.vdim = sp.vdim; ap.rot_dims = sp.cs ? sp.rot_dims : 0; ap.rot_pairs = sp.rot_pairs;
   ap.cs = sp.cs; ap.poolK = sp.append ? sp.poolK : nullptr; ap.poolV = sp.poolV; ap.poolVT = sp.poolVT; ap.vfirst = sm->vfirst; ap.vmode = sp.vmode; ap.lam = sp.lam;
   ap.q_temp_coef = sp.q_temp_every > 0 ? sp.q_temp_coef : 0.f; ap.q_temp_every = sp.q_temp_every;
   if (sp.v_is_k) {      // normed queries and keys, the keys' projections as values
@@ -382,7 +385,7 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
     // rows = (token, query head of the group) pairs of an entry and a key / value head in tiles of 32; few tiles and a long context: the keys are divided
     tgx::GqaMfmaArgs ma{};
     ma.q = sp.proj; ma.ldq = sp.ldp; ma.poolK = sp.poolK; ma.poolVT = sp.poolVT; ma.gate = sp.gate; ma.ldg = sp.ldg; ma.out = sp.out; ma.ldo = sp.ldo;
-    ma.heads = H; ma.kv_heads = G; ma.dim = sp.dim; ma.vdim = sp.vdim; ma.terms = c->act16 ? 1 : 2; ma.scale = sp.scale; ma.sink = sp.sink; ma.has_sink = sp.has_sink;
+    ma.heads = H; ma.kv_heads = G; ma.maps = sp.maps; ma.dim = sp.dim; ma.vdim = sp.vdim; ma.terms = c->act16 ? 1 : 2; ma.scale = sp.scale; ma.sink = sp.sink; ma.has_sink = sp.has_sink;
     ma.mask_kind = sp.mask_kind; ma.mask_size = sp.mask_size; ma.softcap = sp.softcap; ma.dist_bias = sp.dist_bias;
     ma.sinks = sp.sinks; ma.dist_tab = sp.dist; ma.dist_len = sp.dist_len; ma.gate_per_head = sp.gate_per_head; ma.out_scale = sp.out_scale;
     const int tiles = (max_count * (H / G) + 31) / 32;
@@ -410,7 +413,7 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
   }
   tgx::GqaAttnArgs aa{};
   aa.q = sp.proj; aa.ldq = sp.ldp; aa.poolK = sp.poolK; aa.poolV = sp.poolV; aa.gate = sp.gate; aa.ldg = sp.ldg; aa.out = sp.out; aa.ldo = sp.ldo;
-  aa.heads = H; aa.kv_heads = G; aa.dim = sp.dim; aa.vdim = sp.vdim; aa.scale = sp.scale; aa.sink = sp.sink; aa.has_sink = sp.has_sink;
+  aa.heads = H; aa.kv_heads = G; aa.maps = sp.maps; aa.dim = sp.dim; aa.vdim = sp.vdim; aa.scale = sp.scale; aa.sink = sp.sink; aa.has_sink = sp.has_sink;
   aa.mask_kind = sp.mask_kind; aa.mask_size = sp.mask_size; aa.softcap = sp.softcap; aa.dist_bias = sp.dist_bias;
   aa.sinks = sp.sinks; aa.dist_tab = sp.dist; aa.dist_len = sp.dist_len; aa.gate_per_head = sp.gate_per_head; aa.out_scale = sp.out_scale;
   int nsplit = 1;
@@ -595,6 +598,7 @@ void launch_rec_scan(tgx_ctx* c, const tgx::StepMeta& m, const tgx::RecScanArgs&
     else hipLaunchKernelGGL((tgx::rec_scan_kernel<32, KIND>), grid, dim3(256), 0, c->stream, m, a);
   };
   if (kind == tgx::REC_WKV) go(std::integral_constant<int, tgx::REC_WKV>{});
+  else if (kind == tgx::REC_CDELTA) go(std::integral_constant<int, tgx::REC_CDELTA>{});
   else if (kind == tgx::REC_SSD) go(std::integral_constant<int, tgx::REC_SSD>{});
   else go(std::integral_constant<int, tgx::REC_DELTA>{});
 }
@@ -667,7 +671,7 @@ int run_parallel(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T, int 
   // the right half: rec_in row = [q | k | v | beta | decay]
   const int ldr = rC + 2 * rH, nb = ld.conv_taps - 1;
   tgx::DeltaPrepArgs dp{};
-  dp.proj = sm->proj; dp.ldp = nin; dp.col0 = lq + lkv; dp.cw = w.conv_w; dp.a_log = w.a_log; dp.dt_bias = w.dt_bias; dp.out = sm->rec_in; dp.ldo = ldr;
+  dp.proj = sm->proj; dp.ldp = nin; dp.col0 = lq + lkv; dp.b_col = rC; dp.cw = w.conv_w; dp.a_log = w.a_log; dp.dt_bias = w.dt_bias; dp.out = sm->rec_in; dp.ldo = ldr;
   dp.state = nb > 0 ? w.conv_state : nullptr; dp.state_buf = (size_t)sm->d.max_seqs * nb * rC; dp.heads = rH; dp.kv_heads = rG; dp.dim = ld.d_dim; dp.vdim = ld.d_vdim; dp.taps = ld.conv_taps;
   dp.q_scale = 1.0f / sqrtf((float)ld.d_dim); dp.unit_eps = 1e-6f;
   hipLaunchKernelGGL(tgx::delta_prep_kernel, dim3(T, 2 * rG + rH + 1), dim3(256), 0, c->stream, m, dp);
@@ -1466,7 +1470,493 @@ int check_post_desc(const tgx_stack_desc& d, const tgx_layer_desc* layers) {
   return TGX_OK;
 }
 
+// ---- hyper-connected designs (Keronex): n residual streams.  A sublayer reads norm(sum_s in[s] x_s); behind it every stream takes the others' shares and the sublayer's
+// output (the seam kernel, which leaves the next sublayer's normed input at once).  A layer may use another layer's weights with a cache or state of its own.
+float* hyper_in(const StackModel* sm, const StackLayerW& w, int sub) { const size_t n = (size_t)sm->n_streams(); return w.hc + (size_t)sub * (2 * n + n * n); }      // [in (n) | out (n) | mix (n x n)]
+
+int run_two_map_attention(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T, int S, int max_keys, int max_count) {
+  StackModel* sm = c->stack;
+  const tgx_layer_desc& ld = w.d;
+  const int W = sm->d.width, M = ld.maps, H = ld.heads * M, G = ld.kv_heads * M, nin = H * ld.dim + G * ld.dim + ld.kv_heads * ld.vdim, ldp = pad4(nin), vd = ld.heads * ld.vdim;
+  // [q (head, map) | k (key / value head, map) | v] = h . w_in^T
+  tgx::StackGemmArgs g{};
+  g.A = sm->a; g.lda = W; g.B = w.w_in; g.ldb = W; g.C = sm->proj; g.ldc = ldp; g.M = T; g.N = nin; g.K = W; g.scale = 1.f;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  GqaSpec sp{};
+  sp.proj = sm->proj; sp.ldp = ldp; sp.heads = H; sp.kv_heads = G; sp.maps = M; sp.dim = ld.dim; sp.vdim = ld.vdim; sp.rot_dims = ld.rot_dims;
+  sp.cs = w.rot >= 0 ? sm->rot[(size_t)w.rot].cs : nullptr; sp.poolK = w.pool; sp.poolV = w.poolV; sp.poolVT = w.poolVT; sp.append = true; sp.scale = ld.scale;
+  sp.out = sm->hs; sp.ldo = (long long)H * ld.vdim;
+  int rc = run_gqa_core(c, m, sp, T, S, max_keys, max_count);
+  if (rc) return rc;
+  tgx::MapDifferenceArgs da{};
+  da.maps = sm->hs; da.out = sm->o; da.pairs = T * ld.heads; da.vdim = ld.vdim; da.lambda = w.lambda; da.eps = sm->d.norm_eps; da.scale = 1.0f - ld.diff;
+  hipLaunchKernelGGL(tgx::map_difference_kernel, dim3((da.pairs + 3) / 4), dim3(256), 0, c->stream, da);
+  sublayer_out(c, sm->o, vd, w.w_o, T);
+  return TGX_OK;
+}
+
+int run_retention(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T, int S, int max_count) {
+  StackModel* sm = c->stack;
+  const tgx_layer_desc& ld = w.d;
+  const int W = sm->d.width, H = ld.heads, qd = H * ld.dim, vd = H * ld.vdim, nin = 2 * qd + 2 * vd, ldp = pad4(nin);
+  // [v | k | q | gate] = h . w_in^T: the order of a state-space recurrence's row (x | B | C)
+  tgx::StackGemmArgs g{};
+  g.A = sm->a; g.lda = W; g.B = w.w_in; g.ldb = W; g.C = sm->proj; g.ldc = ldp; g.M = T; g.N = nin; g.K = W; g.scale = 1.f;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  if (w.rot >= 0) {      // q and k turn in place (2 H heads side by side)
+    tgx::GqaAppendArgs ap{};
+    ap.proj = sm->proj + vd; ap.ldp = ldp; ap.heads = 2 * H; ap.dim = ld.dim; ap.rot_dims = ld.rot_dims; ap.cs = sm->rot[(size_t)w.rot].cs;
+    TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::gqa_append_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, ap))
+  }
+  const float kscale = 1.0f / sqrtf((float)ld.dim);      // the keys' factor, applied to k v^T
+  if (sm->ssd_min > 0 && max_count >= sm->ssd_min && ssd_mfma_shapes_ok(H, H, ld.dim, ld.vdim, ldp)) {
+    int rc = ensure_part(c, ssd_gram_elems(T, S, H));
+    if (rc) return rc;
+    tgx::SsdArgs da{};
+    da.row = sm->proj; da.ld = ldp; da.heads = H; da.groups = H; da.N = ld.dim; da.E = ld.vdim; da.gram = sm->part; da.fixed = w.decays; da.dt0 = kscale; da.S = w.mS; da.out = sm->hs; da.ldo = vd;
+    launch_ssd_mfma(c, m, da, S, max_count);
+  } else {
+    tgx::RecScanArgs ra{};
+    ra.a = sm->proj + vd + qd; ra.lda = ldp; ra.k = sm->proj + vd; ra.ldk = ldp; ra.v = sm->proj; ra.ldv = ldp; ra.fixed = w.decays; ra.beta0 = kscale; ra.S = w.mS; ra.out = sm->hs; ra.ldo = vd;
+    ra.heads = H; ra.kv_heads = H; ra.dim = ld.dim; ra.vdim = ld.vdim;
+    launch_rec_scan(c, m, ra, tgx::REC_SSD, S);
+  }
+  tgx::HeadNormGateArgs oa{};
+  oa.hs = sm->hs; oa.ldh = vd; oa.gate = sm->proj + vd + 2 * qd; oa.ldg = ldp; oa.silu_gate = 1; oa.out = sm->o; oa.ldo = vd; oa.vdim = ld.vdim; oa.eps = sm->d.norm_eps;
+  hipLaunchKernelGGL(tgx::head_norm_gate_kernel, dim3(T, H), dim3(64), 0, c->stream, oa);
+  sublayer_out(c, sm->o, vd, w.w_o, T);
+  return TGX_OK;
+}
+
+// columns of a channel-delta layer's input product: [q | k | v (the convolved channels) | decays' inner row | gate's inner row | b], each part at a multiple of four
+struct ChannelDeltaCols {
+  int qk, C, HD, HE, a1, g1, b, n;
+  explicit ChannelDeltaCols(const tgx_layer_desc& l) {
+    qk = l.kv_heads * l.dim; HD = l.heads * l.dim; HE = l.heads * l.vdim; C = 2 * qk + HE; a1 = pad4(C); g1 = a1 + pad4(l.decay_rank); b = g1 + pad4(l.gate_rank); n = b + l.heads;
+  }
+};
+void run_channel_delta(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T, int S) {
+  StackModel* sm = c->stack;
+  const tgx_layer_desc& ld = w.d;
+  const ChannelDeltaCols k(ld);
+  const int W = sm->d.width, ldp = pad4(k.n), ldr = pad4(k.C + ld.heads), nb = ld.conv_taps - 1;
+  tgx::StackGemmArgs g{};
+  g.A = sm->a; g.lda = W; g.B = w.w_in; g.ldb = W; g.C = sm->proj; g.ldc = ldp; g.M = T; g.N = k.n; g.K = W; g.scale = 1.f;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  // the decays per head and key channel, the gate's pre-activation
+  g = tgx::StackGemmArgs{};
+  g.A = sm->proj + k.a1; g.lda = ldp; g.B = w.w_w2; g.ldb = ld.decay_rank; g.C = sm->mixed; g.ldc = k.HD; g.M = T; g.N = k.HD; g.K = ld.decay_rank; g.scale = 1.f; g.bias = w.dt_bias;
+  g.act = tgx::SG_ACT_HEAD_DECAY; g.a_log = w.a_log; g.head_cols = ld.dim;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  g = tgx::StackGemmArgs{};
+  g.A = sm->proj + k.g1; g.lda = ldp; g.B = w.w_g2; g.ldb = ld.gate_rank; g.C = sm->lora; g.ldc = k.HE; g.M = T; g.N = k.HE; g.K = ld.gate_rank; g.scale = 1.f;
+  launch_gemm(c, g, tgx::SG_STORE, 1);
+  // rec_in row = [q | k | v | beta]
+  tgx::DeltaPrepArgs dp{};
+  dp.proj = sm->proj; dp.ldp = ldp; dp.b_col = k.b; dp.cw = w.conv_w; dp.out = sm->rec_in; dp.ldo = ldr; dp.state = nb > 0 ? w.conv_state : nullptr;
+  dp.state_buf = (size_t)sm->d.max_seqs * nb * k.C; dp.heads = ld.heads; dp.kv_heads = ld.kv_heads; dp.dim = ld.dim; dp.vdim = ld.vdim; dp.taps = ld.conv_taps;
+  dp.q_scale = 1.0f / sqrtf((float)ld.dim); dp.unit_eps = 1e-6f;
+  hipLaunchKernelGGL(tgx::delta_prep_kernel, dim3(T, 2 * ld.kv_heads + ld.heads + 1), dim3(256), 0, c->stream, m, dp);
+  tgx::RecScanArgs ra{};
+  ra.a = sm->rec_in; ra.lda = ldr; ra.k = sm->rec_in + k.qk; ra.ldk = ldr; ra.v = sm->rec_in + 2 * (size_t)k.qk; ra.ldv = ldr; ra.beta = sm->rec_in + k.C; ra.ldg = ldr;
+  ra.w = sm->mixed; ra.ldw = k.HD; ra.S = w.mS; ra.out = sm->hs; ra.ldo = k.HE; ra.heads = ld.heads; ra.kv_heads = ld.kv_heads; ra.dim = ld.dim; ra.vdim = ld.vdim;
+  launch_rec_scan(c, m, ra, tgx::REC_CDELTA, S);
+  tgx::HeadNormGateArgs oa{};
+  oa.hs = sm->hs; oa.ldh = k.HE; oa.w = w.head_w; oa.w_hstride = 0; oa.gate = sm->lora; oa.ldg = k.HE; oa.out = sm->o; oa.ldo = k.HE; oa.vdim = ld.vdim; oa.eps = sm->d.norm_eps;
+  hipLaunchKernelGGL(tgx::head_norm_gate_kernel, dim3(T, ld.heads), dim3(64), 0, c->stream, oa);
+  sublayer_out(c, sm->o, k.HE, w.w_o, T);
+}
+
+// the feed-forward into yd (one row per token, or `top` rows for experts) and ysh (the shared expert's row)
+void run_hyper_ff(tgx_ctx* c, StackLayerW& w, int T) {
+  StackModel* sm = c->stack;
+  const tgx_layer_desc& ld = w.d;
+  const int W = sm->d.width;
+  tgx::StackGemmArgs g{};
+  if (ld.mlp == TGX_MLP_DENSE) {      // down(gelu(gate h) * (up h))
+    g.A = sm->a; g.lda = W; g.B = w.w_gate; g.B2 = w.w_up; g.ldb = W; g.C = sm->yh; g.ldc = ld.ff; g.M = T; g.N = ld.ff; g.K = W; g.act = tgx::SG_ACT_GELU_TANH;
+    launch_gemm(c, g, tgx::SG_SILU_MUL, 1);
+    sublayer_out(c, sm->yh, ld.ff, w.w_down, T);
+    return;
+  }
+  const int E = ld.experts, top = ld.top, np = T * top;
+  g.A = sm->a; g.lda = W; g.B = w.w_router; g.ldb = W; g.C = sm->zr; g.ldc = E; g.M = T; g.N = E; g.K = W; g.scale = 1.f;
+  launch_gemm(c, g, tgx::SG_STORE, 1, 0, 0, 64, tgx::DT_F32);
+  tgx::RouterGroupArgs ra{};
+  ra.z = sm->zr; ra.ldz = E; ra.sel = sm->sel; ra.selw = sm->selw; ra.E = E; ra.top = top; ra.groups = 1; ra.keep = 1; ra.scale = 1.f; ra.sigmoid_scores = ld.router_fn == 1; ra.normalise = ld.router_norm;
+  hipLaunchKernelGGL(tgx::router_group_kernel, dim3(T), dim3(64), 0, c->stream, ra);
+  tgx::MoePlanArgs pa{};
+  pa.sel = sm->sel; pa.n_pairs = np; pa.E = E; pa.top = top; pa.tile_m = grouped_tile_rows(c, np, W, ld.ff); pa.E_tiles = E;
+  pa.off = sm->moe_off; pa.perm = sm->perm; pa.tok = sm->ptok; pa.tile_e = sm->tile_e; pa.tile_m0 = sm->tile_m0; pa.n_tiles = sm->n_tiles;
+  hipLaunchKernelGGL(tgx::moe_plan_kernel, dim3(1), dim3(1024), 0, c->stream, pa);
+  // yh[n] = max(up_e (w h), 0)^2 over the pairs grouped by expert: up_e is linear, so the weight multiplies its product
+  g = tgx::StackGemmArgs{};
+  g.A = sm->a; g.lda = W; g.a_rows = sm->ptok; g.B = w.w_up; g.ldb = W; g.b_zstride = (long long)ld.ff * W; g.C = sm->yh; g.ldc = ld.ff; g.scale = 1.f; g.act = tgx::SG_ACT_RELU2;
+  g.in_w = sm->selw; g.in_rows = sm->perm; g.z_off = sm->moe_off; g.tile_z = sm->tile_e; g.tile_m0 = sm->tile_m0; g.n_tiles = sm->n_tiles; g.M = np; g.N = ld.ff; g.K = W;
+  launch_gemm(c, g, tgx::SG_STORE, 1, np, E, pa.tile_m);
+  g = tgx::StackGemmArgs{};
+  g.A = sm->yh; g.lda = ld.ff; g.B = w.w_down; g.ldb = ld.ff; g.b_zstride = (long long)W * ld.ff; g.C = sm->yd; g.ldc = W; g.c_rows = sm->perm; g.scale = 1.f;
+  g.z_off = sm->moe_off; g.tile_z = sm->tile_e; g.tile_m0 = sm->tile_m0; g.n_tiles = sm->n_tiles; g.M = np; g.N = W; g.K = ld.ff;
+  launch_gemm(c, g, tgx::SG_STORE, 1, np, E, pa.tile_m);
+  if (ld.shared_ff > 0) {
+    float* hsh = sm->yh + (((size_t)np * ld.ff + 3) & ~(size_t)3);
+    g = tgx::StackGemmArgs{};
+    g.A = sm->a; g.lda = W; g.B = w.ws_up; g.ldb = W; g.C = hsh; g.ldc = ld.shared_ff; g.M = T; g.N = ld.shared_ff; g.K = W; g.scale = 1.f; g.act = tgx::SG_ACT_RELU2;
+    launch_gemm(c, g, tgx::SG_STORE, 1);
+    g = tgx::StackGemmArgs{};
+    g.A = hsh; g.lda = ld.shared_ff; g.B = w.ws_down; g.ldb = ld.shared_ff; g.C = sm->ysh; g.ldc = W; g.M = T; g.N = W; g.K = ld.shared_ff; g.scale = 1.f;
+    launch_gemm(c, g, tgx::SG_STORE, 1);
+  }
+}
+
+void hyper_seam(tgx_ctx* c, const StackLayerW& w, int sub, const float* next_in, const float* next_norm, int T, int top, bool shared) {
+  StackModel* sm = c->stack;
+  const int n = sm->n_streams();
+  const float* hc = hyper_in(sm, w, sub);
+  tgx::HyperSeamArgs sa{};
+  sa.xs = sm->xs; sa.y = sm->yd; sa.top = top; sa.ysh = shared ? sm->ysh : nullptr; sa.w_out = hc + n; sa.mix = hc + 2 * n; sa.n = n; sa.W = sm->d.width;
+  sa.in.w_in = next_in; sa.in.w_norm = next_norm; sa.in.out = next_in ? sm->a : sm->x; sa.in.eps = sm->d.norm_eps;
+  if (n <= 1) hipLaunchKernelGGL(tgx::hyper_seam_kernel<1>, dim3(T), dim3(256), 0, c->stream, sa);
+  else if (n <= 2) hipLaunchKernelGGL(tgx::hyper_seam_kernel<2>, dim3(T), dim3(256), 0, c->stream, sa);
+  else if (n <= 4) hipLaunchKernelGGL(tgx::hyper_seam_kernel<4>, dim3(T), dim3(256), 0, c->stream, sa);
+  else if (n <= 8) hipLaunchKernelGGL(tgx::hyper_seam_kernel<8>, dim3(T), dim3(256), 0, c->stream, sa);
+  else hipLaunchKernelGGL(tgx::hyper_seam_kernel<16>, dim3(T), dim3(256), 0, c->stream, sa);
+}
+
+int run_layers_hyper(tgx_ctx* c, const MetaPtrs& mp, int T, int S, int max_keys, int max_count) {
+  StackModel* sm = c->stack;
+  const tgx::StepMeta m = step_meta(sm, mp, T, S);
+  const tgx_stack_desc& d = sm->d;
+  tgx::PairEmbedArgs ea{};
+  ea.embed = c->embed; ea.pair = sm->pair; ea.last = sm->last_tok; ea.slots = d.max_seqs; ea.buckets = d.bigram_buckets; ea.mul_before = d.bigram_before; ea.mul = d.bigram_cur;
+  ea.scale = d.embed_scale; ea.xs = sm->xs; ea.n = sm->n_streams(); ea.W = d.width;
+  ea.in.w_in = hyper_in(sm, sm->L[0], 0); ea.in.w_norm = sm->L[0].norm1; ea.in.out = sm->a; ea.in.eps = d.norm_eps;
+  TGX_DT_SWITCH(c->dt, hipLaunchKernelGGL(tgx::pair_embed_kernel<DT>, dim3(T), dim3(256), 0, c->stream, m, ea))
+  for (int li = 0; li < d.layers; li++) {
+    StackLayerW& w = sm->L[(size_t)li];
+    const tgx_layer_desc& ld = w.d;
+    int rc = TGX_OK;
+    if (ld.mixer == TGX_MIXER_ATTENTION) rc = run_two_map_attention(c, m, w, T, S, max_keys, max_count);
+    else if (ld.mixer == TGX_MIXER_RETENTION) rc = run_retention(c, m, w, T, S, max_count);
+    else run_channel_delta(c, m, w, T, S);
+    if (rc) return rc;
+    const bool last = li + 1 == d.layers, ff = ld.mlp != TGX_MLP_NONE;
+    const StackLayerW* nx = last ? nullptr : &sm->L[(size_t)li + 1];
+    const float *next_in = nx ? hyper_in(sm, *nx, 0) : nullptr, *next_norm = nx ? nx->norm1 : nullptr;
+    hyper_seam(c, w, 0, ff ? hyper_in(sm, w, 1) : next_in, ff ? w.norm2 : next_norm, T, 1, false);
+    if (!ff) continue;
+    run_hyper_ff(c, w, T);
+    hyper_seam(c, w, 1, next_in, next_norm, T, ld.mlp == TGX_MLP_MOE ? ld.top : 1, ld.mlp == TGX_MLP_MOE && ld.shared_ff > 0);
+  }
+  return TGX_OK;
+}
+
+// the layer whose tensors layer i uses (checked at creation: an earlier or later layer of the same description that ends at one with tensors of its own)
+int weights_layer(const tgx_layer_desc* layers, int n, int i) {
+  for (int hops = 0; hops <= n; hops++) {
+    if (i < 0 || i >= n) return -1;
+    if (!layers[i].weights_of) return i;
+    i = layers[i].weights_of - 1;
+  }
+  return -1;
+}
+
+// parameter storage of a hyper-connected design (Keronex)
+int create_hyper_layers(tgx_ctx* c, const tgx_layer_desc* layers) {
+  StackModel* sm = c->stack;
+  const tgx_stack_desc& d = sm->d;
+  const size_t W = (size_t)d.width, es = c->esz, n = (size_t)sm->n_streams();
+  int rc;
+  if ((rc = dev_alloc(c, &sm->head, (size_t)d.vocab * W * es)) || (rc = dev_alloc(c, &sm->last_tok, 2 * (size_t)d.max_seqs))) return rc;
+  HIP_OK(c, hipMemset(sm->last_tok, 0, 2 * (size_t)d.max_seqs * 4));
+  sm->missing.insert("head");
+  if (d.bigram_buckets > 0) {
+    if ((rc = dev_alloc(c, &sm->pair, ((size_t)d.bigram_buckets + 1) * W * es))) return rc;
+    sm->missing.insert("bigram");
+  }
+  sm->max_top = 1; sm->max_E = 1; sm->max_ff = 1;      // the sublayers' outputs and the dense feed-forward use the expert buffers with one row per token
+  auto need = [&](const std::string& p, std::initializer_list<const char*> names) { for (const char* s : names) sm->missing.insert(p + s); };
+  for (int i = 0; i < d.layers; i++) {
+    StackLayerW& w = sm->L[(size_t)i];
+    w.d = layers[i];
+    const tgx_layer_desc& l = w.d;
+    w.d.decays = nullptr;                                 // (read below, while the caller's array stands)
+    w.w_src = l.weights_of ? weights_layer(layers, d.layers, i) : -1;
+    const std::string p = "l" + std::to_string(i) + ".";
+    const size_t H = (size_t)l.heads, qd = H * l.dim, vd = H * l.vdim;
+    if (l.mixer != TGX_MIXER_CHANNEL_DELTA && l.rot_dims > 0) {
+      for (size_t r = 0; r < sm->rot.size(); r++) if (sm->rot[r].dims == l.rot_dims && sm->rot[r].base == l.rot_base) w.rot = (int)r;
+      if (w.rot < 0) { w.rot = (int)sm->rot.size(); sm->rot.push_back(RotTable{l.rot_dims, l.rot_base, 1.f, nullptr}); }
+    }
+    if (w.w_src >= 0) continue;                           // (the sizes below are those of the layer it borrows from)
+    if ((rc = dev_alloc(c, &w.norm1, W)) || (rc = dev_alloc(c, &w.hc, 2 * (2 * n + n * n))) || (rc = dev_alloc(c, &w.w_o, W * vd * es))) return rc;
+    need(p, {"norm1", "mix.q", "mix.k", "mix.v", "mix.o"});
+    if (d.streams > 0) need(p, {"hc1.in", "hc1.out", "hc1.mix"});
+    else {                                                // the plain residual: read the stream, add the output
+      const std::vector<float> one(2 * 3, 1.f);
+      HIP_OK(c, hipMemcpy(w.hc, one.data(), one.size() * 4, hipMemcpyHostToDevice));
+    }
+    sm->max_hv = std::max(sm->max_hv, (int)(vd * std::max(1, l.maps)));
+    if (l.mixer == TGX_MIXER_ATTENTION) {
+      const size_t nin = (size_t)l.maps * (H + l.kv_heads) * l.dim + (size_t)l.kv_heads * l.vdim;
+      if ((rc = dev_alloc(c, &w.w_in, nin * W * es))) return rc;
+      need(p, {"mix.lq1", "mix.lk1", "mix.lq2", "mix.lk2"});
+      w.lam_host.assign(4, std::vector<float>());
+      sm->max_in = std::max(sm->max_in, pad4((int)nin));
+    } else if (l.mixer == TGX_MIXER_RETENTION) {
+      const size_t nin = 2 * qd + 2 * vd;
+      if ((rc = dev_alloc(c, &w.w_in, nin * W * es)) || (rc = dev_alloc(c, &w.decays, 2 * H))) return rc;
+      std::vector<float> dec(2 * H);
+      for (size_t h = 0; h < H; h++) { dec[h] = layers[i].decays[h]; dec[H + h] = (float)log((double)layers[i].decays[h]); }
+      HIP_OK(c, hipMemcpy(w.decays, dec.data(), dec.size() * 4, hipMemcpyHostToDevice));
+      need(p, {"mix.g"});
+      sm->max_in = std::max(sm->max_in, pad4((int)nin));
+    } else {      // the input product is put together at finalize, when the inner sizes of the low-rank products are known
+      const size_t C = 2 * (size_t)l.kv_heads * l.dim + vd;
+      if ((rc = dev_alloc(c, &w.w_in, C * W * es)) || (rc = dev_alloc(c, &w.w_b, H * W * es)) || (rc = dev_alloc(c, &w.conv_w, C * (size_t)l.conv_taps)) || (rc = dev_alloc(c, &w.a_log, H)) ||
+          (rc = dev_alloc(c, &w.dt_bias, qd)) || (rc = dev_alloc(c, &w.head_w, (size_t)l.vdim))) return rc;
+      if (l.decay_rank > 0 && ((rc = dev_alloc(c, &w.w_w1, (size_t)l.decay_rank * W * es)) || (rc = dev_alloc(c, &w.w_w2, qd * l.decay_rank * es)))) return rc;
+      if (l.gate_rank > 0 && ((rc = dev_alloc(c, &w.w_g1, (size_t)l.gate_rank * W * es)) || (rc = dev_alloc(c, &w.w_g2, vd * l.gate_rank * es)))) return rc;
+      need(p, {"mix.q.conv", "mix.k.conv", "mix.v.conv", "mix.b", "mix.A_log", "mix.norm", "mix.a1", "mix.a2", "mix.dt_bias", "mix.g1", "mix.g2"});
+      sm->max_rec = std::max(sm->max_rec, pad4((int)(C + H))); sm->max_shift = std::max(sm->max_shift, (int)qd); sm->max_lora = std::max(sm->max_lora, (int)vd);
+    }
+    if (l.mlp == TGX_MLP_NONE) continue;
+    if ((rc = dev_alloc(c, &w.norm2, W))) return rc;
+    need(p, {"norm2"});
+    if (d.streams > 0) need(p, {"hc2.in", "hc2.out", "hc2.mix"});
+    if (l.mlp == TGX_MLP_DENSE) {
+      const size_t F = (size_t)l.ff;
+      if ((rc = dev_alloc(c, &w.w_gate, F * W * es)) || (rc = dev_alloc(c, &w.w_up, F * W * es)) || (rc = dev_alloc(c, &w.w_down, W * F * es))) return rc;
+      need(p, {"mlp.gate", "mlp.up", "mlp.down"});
+      sm->max_ff = std::max(sm->max_ff, l.ff);
+      continue;
+    }
+    const size_t E = (size_t)l.experts, F = (size_t)l.ff, SF = (size_t)l.shared_ff;
+    if ((rc = dev_alloc(c, &w.w_router, E * W)) || (rc = dev_alloc(c, &w.w_up, E * F * W * es)) || (rc = dev_alloc(c, &w.w_down, E * W * F * es))) return rc;
+    need(p, {"mlp.router"});
+    for (int e = 0; e < l.experts; e++)
+      for (const char* s : {".up", ".down"}) sm->missing.insert(p + "mlp.e" + std::to_string(e) + s);
+    if (SF > 0) {
+      if ((rc = dev_alloc(c, &w.ws_up, SF * W * es)) || (rc = dev_alloc(c, &w.ws_down, W * SF * es))) return rc;
+      need(p, {"mlp.shared.up", "mlp.shared.down"});
+    }
+    sm->max_top = std::max(sm->max_top, l.top); sm->max_ff = std::max(sm->max_ff, l.ff); sm->max_E = std::max(sm->max_E, l.experts); sm->max_sff = std::max(sm->max_sff, l.shared_ff);
+  }
+  sm->max_sff += sm->max_sff > 0 ? 4 : 0;      // (the shared expert's rows start at a multiple of four)
+  return TGX_OK;
+}
+
+// tensors of a hyper-connected design by checkpoint name
+int upload_hyper(tgx_ctx* c, const char* name, const void* host, const int64_t* shape, int nd, int src_dtype) {
+  StackModel* sm = c->stack;
+  const tgx_stack_desc& d = sm->d;
+  const int64_t W = d.width, n = sm->n_streams();
+  const bool probe = nd < 0;
+  auto bad_shape = [&]() { return set_err(c, TGX_ERR_SHAPE, "shape not equal for tensor: %s", name); };
+  auto is = [&](int64_t a, int64_t b) { return b < 0 ? (nd == 1 && shape[0] == a) : (nd == 2 && shape[0] == a && shape[1] == b); };
+  auto done = [&](int rc) { if (!rc) sm->missing.erase(name); return rc; };
+  auto mat = [&](ebyte* dst, int64_t row0, int64_t rows, int64_t cols) {
+    if (probe) return (int)TGX_ERR_SHAPE;
+    if (!is(rows, cols)) return bad_shape();
+    return done(upload_param_ext(c, dst + (size_t)(row0 * cols) * c->esz, host, rows * cols, src_dtype));
+  };
+  auto vec = [&](float* dst, int64_t len, int64_t n2 = -1) {      // an fp32 vector, or (n2 >= 0) an fp32 matrix [len][n2]
+    if (probe) return (int)TGX_ERR_SHAPE;
+    if (!is(len, n2)) return bad_shape();
+    return done(upload_f32(c, dst, host, n2 < 0 ? len : len * n2, src_dtype));
+  };
+  if (!strcmp(name, "embed")) return mat(c->embed, 0, d.vocab, W);
+  if (!strcmp(name, "head")) return mat(sm->head, 0, d.vocab, W);
+  if (!strcmp(name, "final.norm")) return vec(sm->final_norm, W);
+  if (sm->pair && !strcmp(name, "bigram")) return mat(sm->pair, 0, (int64_t)d.bigram_buckets + 1, W);
+  int li = -1;
+  char rest[128] = {0};
+  if (sscanf(name, "l%d.%127s", &li, rest) != 2 || li < 0 || li >= d.layers || sm->L[(size_t)li].w_src >= 0) return set_err(c, TGX_ERR_NAME, "Unexpected key: %s", name);
+  StackLayerW& w = sm->L[(size_t)li];
+  tgx_layer_desc& l = w.d;
+  const int64_t H = l.heads, G = l.kv_heads, qd = H * l.dim, vd = H * l.vdim;
+  const bool ff = l.mlp != TGX_MLP_NONE;
+  if (!strcmp(rest, "norm1")) return vec(w.norm1, W);
+  if (ff && !strcmp(rest, "norm2")) return vec(w.norm2, W);
+  if (d.streams > 0 && !strncmp(rest, "hc", 2) && (rest[2] == '1' || (ff && rest[2] == '2')) && rest[3] == '.') {
+    float* hc = hyper_in(sm, w, rest[2] - '1');
+    if (!strcmp(rest + 4, "in")) return vec(hc, n);
+    if (!strcmp(rest + 4, "out")) return vec(hc + n, n);
+    if (!strcmp(rest + 4, "mix")) return vec(hc + 2 * n, n, n);
+  }
+  if (!strcmp(rest, "mix.o")) return mat(w.w_o, 0, W, vd);
+  if (l.mixer == TGX_MIXER_ATTENTION) {
+    const int64_t mq = l.maps * qd, mk = l.maps * G * l.dim;
+    if (!strcmp(rest, "mix.q")) return mat(w.w_in, 0, mq, W);
+    if (!strcmp(rest, "mix.k")) return mat(w.w_in, mq, mk, W);
+    if (!strcmp(rest, "mix.v")) return mat(w.w_in, mq + mk, G * l.vdim, W);
+    static const char* const lam[4] = {"mix.lq1", "mix.lk1", "mix.lq2", "mix.lk2"};      // one number per layer comes of them at finalize
+    for (int k = 0; k < 4; k++)
+      if (!strcmp(rest, lam[k])) {
+        if (probe) return TGX_ERR_SHAPE;
+        if (!is(l.dim, -1)) return bad_shape();
+        w.lam_host[(size_t)k] = to_f32(host, l.dim, src_dtype);
+        return done(TGX_OK);
+      }
+  } else if (l.mixer == TGX_MIXER_RETENTION) {
+    if (!strcmp(rest, "mix.v")) return mat(w.w_in, 0, vd, W);
+    if (!strcmp(rest, "mix.k")) return mat(w.w_in, vd, qd, W);
+    if (!strcmp(rest, "mix.q")) return mat(w.w_in, vd + qd, qd, W);
+    if (!strcmp(rest, "mix.g")) return mat(w.w_in, vd + 2 * qd, vd, W);
+  } else {
+    const int64_t GD = G * l.dim;
+    if (!strcmp(rest, "mix.q")) return mat(w.w_in, 0, GD, W);
+    if (!strcmp(rest, "mix.k")) return mat(w.w_in, GD, GD, W);
+    if (!strcmp(rest, "mix.v")) return mat(w.w_in, 2 * GD, vd, W);
+    if (!strcmp(rest, "mix.b")) return mat(w.w_b, 0, H, W);
+    if (!strcmp(rest, "mix.q.conv")) return vec(w.conv_w, GD, l.conv_taps);
+    if (!strcmp(rest, "mix.k.conv")) return vec(w.conv_w + (size_t)GD * l.conv_taps, GD, l.conv_taps);
+    if (!strcmp(rest, "mix.v.conv")) return vec(w.conv_w + (size_t)2 * GD * l.conv_taps, vd, l.conv_taps);
+    if (!strcmp(rest, "mix.A_log")) return vec(w.a_log, H);
+    if (!strcmp(rest, "mix.dt_bias")) return vec(w.dt_bias, qd);
+    if (!strcmp(rest, "mix.norm")) return vec(w.head_w, l.vdim);
+    const bool a = !strcmp(rest, "mix.a1") || !strcmp(rest, "mix.a2"), gt = !strcmp(rest, "mix.g1") || !strcmp(rest, "mix.g2");
+    if (a || gt) {      // the inner size is the tensors' own where the description leaves it open
+      if (probe) return TGX_ERR_SHAPE;
+      if (nd != 2) return bad_shape();
+      const bool first = rest[5] == '1';
+      const int64_t rows = a ? qd : vd, R = first ? shape[0] : shape[1];
+      int32_t& rank = a ? l.decay_rank : l.gate_rank;
+      ebyte*& m1 = a ? w.w_w1 : w.w_g1;
+      ebyte*& m2 = a ? w.w_w2 : w.w_g2;
+      if (rank <= 0) {
+        if (R <= 0 || R > 65536) return bad_shape();
+        int rc;
+        if ((rc = dev_alloc(c, &m1, (size_t)(R * W) * c->esz)) || (rc = dev_alloc(c, &m2, (size_t)(rows * R) * c->esz))) return rc;
+        rank = (int32_t)R;
+      }
+      return first ? mat(m1, 0, rank, W) : mat(m2, 0, rows, rank);
+    }
+  }
+  if (l.mlp == TGX_MLP_DENSE) {
+    if (!strcmp(rest, "mlp.gate")) return mat(w.w_gate, 0, l.ff, W);
+    if (!strcmp(rest, "mlp.up")) return mat(w.w_up, 0, l.ff, W);
+    if (!strcmp(rest, "mlp.down")) return mat(w.w_down, 0, W, l.ff);
+  }
+  if (l.mlp == TGX_MLP_MOE) {
+    const int64_t E = l.experts, F = l.ff, SF = l.shared_ff;
+    if (!strcmp(rest, "mlp.router")) return vec(w.w_router, E, W);
+    if (SF > 0) {
+      if (!strcmp(rest, "mlp.shared.up")) return mat(w.ws_up, 0, SF, W);
+      if (!strcmp(rest, "mlp.shared.down")) return mat(w.ws_down, 0, W, SF);
+    }
+    int e = -1;
+    char leaf[32] = {0};
+    if (sscanf(rest, "mlp.e%d.%31s", &e, leaf) == 2 && e >= 0 && e < E) {
+      if (!strcmp(leaf, "up")) return mat(w.w_up, e * F, F, W);
+      if (!strcmp(leaf, "down")) return mat(w.w_down, e * W, W, F);
+    }
+  }
+  return set_err(c, TGX_ERR_NAME, "Unexpected key: %s", name);
+}
+
+// what a hyper-connected design's description may ask for
+int check_hyper_desc(const tgx_stack_desc& d, const tgx_layer_desc* layers) {
+  if (d.streams < 0 || d.streams > tgx::HYPER_MAX_STREAMS) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "%d residual streams (0 .. %d)", d.streams, tgx::HYPER_MAX_STREAMS);
+  if (d.bigram_buckets < 0 || d.bigram_before < 0 || d.bigram_cur < 0 || (d.bigram_buckets > 0 && (d.bigram_before > INT32_MAX || d.bigram_cur > INT32_MAX)))
+    return set_err(nullptr, TGX_ERR_INVALID, "pair table: %d buckets, factors %lld and %lld", d.bigram_buckets, (long long)d.bigram_before, (long long)d.bigram_cur);
+  for (int i = 0; i < d.layers; i++) {
+    const tgx_layer_desc& l = layers[i];
+    if (l.heads <= 0 || l.dim <= 0 || l.vdim <= 0 || l.kv_heads <= 0 || l.heads % l.kv_heads) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: %d heads over %d key heads of %d / %d", i, l.heads, l.kv_heads, l.dim, l.vdim);
+    if (l.mixer != TGX_MIXER_CHANNEL_DELTA && (l.rot_dims < 0 || l.rot_dims > l.dim || (l.rot_dims & 1) || (l.rot_dims > 0 && !(l.rot_base > 0.f))))
+      return set_err(nullptr, TGX_ERR_INVALID, "layer %d: %d rotated dimensions of %d (base %g)", i, l.rot_dims, l.dim, l.rot_base);
+    if (l.mixer == TGX_MIXER_ATTENTION) {
+      if (l.maps != 2 || l.dim > 64 * tgx::GQA_MAX_RPL || l.vdim > 64 * tgx::GQA_MAX_RPL) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: attention of %d maps, heads of %d / %d (two maps, up to %d)", i, l.maps, l.dim, l.vdim, 64 * tgx::GQA_MAX_RPL);
+    } else if (l.mixer == TGX_MIXER_RETENTION) {
+      if (l.dim > 256 || l.kv_heads != l.heads) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: retention: %d heads over %d of %d (1 .. 256)", i, l.heads, l.kv_heads, l.dim);
+      if (l.n_decays != l.heads || !l.decays) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: retention: %d decays for %d heads", i, l.n_decays, l.heads);
+      for (int h = 0; h < l.heads; h++) if (!(l.decays[h] > 0.f && l.decays[h] <= 1.f)) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: decay %g of head %d outside (0, 1]", i, l.decays[h], h);
+    } else if (l.mixer == TGX_MIXER_CHANNEL_DELTA) {
+      if (l.dim > 256 || l.conv_taps < 1 || l.conv_taps > tgx::DELTA_MAX_TAPS || l.decay_rank < 0 || l.gate_rank < 0)
+        return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: channel delta: key size %d (1 .. 256), %d taps (1 .. %d), ranks %d and %d", i, l.dim, l.conv_taps, tgx::DELTA_MAX_TAPS, l.decay_rank, l.gate_rank);
+    } else return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: mixer %d is not part of this family (retention, attention and channel_delta are)", i, l.mixer);
+    if (l.mlp != TGX_MLP_NONE && l.mlp != TGX_MLP_MOE && l.mlp != TGX_MLP_DENSE) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: feed-forward kind %d is not implemented", i, l.mlp);
+    if (l.mlp == TGX_MLP_DENSE && (l.ff <= 0 || l.ff_act != 3)) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: ff %d, activation %d", i, l.ff, l.ff_act);
+    if (l.mlp == TGX_MLP_MOE && (l.experts <= 0 || l.experts >= tgx::ROUTER_MAX_E || l.top <= 0 || l.top > l.experts || l.top > tgx::ROUTER_MAX_TOP || l.ff <= 0 || l.shared_ff < 0 || l.identity != 0 ||
+                                 l.groups > 1 || l.router_fn != 1 || !l.router_in || l.expert_act != 1))
+      return set_err(nullptr, TGX_ERR_UNSUPPORTED, "layer %d: experts %d (< %d), top %d (<= %d), ff %d: this family's experts are chosen by sigmoid scores, weighted at their input, with squared relu", i,
+                     l.experts, tgx::ROUTER_MAX_E, l.top, tgx::ROUTER_MAX_TOP, l.ff);
+    if (l.weights_of) {
+      const int j = weights_layer(layers, d.layers, i);
+      if (j < 0 || j == i) return set_err(nullptr, TGX_ERR_INVALID, "layer %d: uses the weights of layer %d, which leads to no layer with weights of its own", i, l.weights_of - 1);
+      const tgx_layer_desc& o = layers[j];
+      if (o.mixer != l.mixer || o.heads != l.heads || o.kv_heads != l.kv_heads || o.dim != l.dim || o.vdim != l.vdim || o.conv_taps != l.conv_taps || o.mlp != l.mlp || o.ff != l.ff || o.experts != l.experts ||
+          o.top != l.top || o.shared_ff != l.shared_ff || o.rot_dims != l.rot_dims || o.rot_base != l.rot_base || o.scale != l.scale || o.diff != l.diff)
+        return set_err(nullptr, TGX_ERR_INVALID, "layer %d: differs from layer %d, whose weights it uses", i, j);
+    }
+  }
+  return TGX_OK;
+}
+
+// what a hyper-connected design derives from its tensors, then every layer's cache or state
+int finalize_hyper(tgx_ctx* c) {
+  StackModel* sm = c->stack;
+  const tgx_stack_desc& d = sm->d;
+  const size_t W = (size_t)d.width, B = (size_t)d.max_seqs, es = c->esz;
+  int rc;
+  for (auto& w : sm->L) {
+    if (w.w_src >= 0) continue;
+    tgx_layer_desc& l = w.d;
+    if (l.mixer == TGX_MIXER_ATTENTION) {
+      double dot[2] = {0, 0};
+      for (int k = 0; k < 2; k++)
+        for (int i = 0; i < l.dim; i++) dot[k] += (double)w.lam_host[2 * (size_t)k][(size_t)i] * (double)w.lam_host[2 * (size_t)k + 1][(size_t)i];
+      w.lambda = (float)(exp(dot[0]) - exp(dot[1]) + (double)l.diff);
+    } else if (l.mixer == TGX_MIXER_CHANNEL_DELTA) {
+      const ChannelDeltaCols k(l);
+      ebyte* all = nullptr;
+      if ((rc = dev_alloc(c, &all, (size_t)k.n * W * es))) return rc;
+      HIP_OK(c, hipMemset(all, 0, (size_t)k.n * W * es));
+      struct Part { ebyte** src; int row0, rows; };
+      for (const Part& p : {Part{&w.w_in, 0, k.C}, Part{&w.w_w1, k.a1, l.decay_rank}, Part{&w.w_g1, k.g1, l.gate_rank}, Part{&w.w_b, k.b, l.heads}}) {
+        HIP_OK(c, hipMemcpy(all + (size_t)p.row0 * W * es, *p.src, (size_t)p.rows * W * es, hipMemcpyDeviceToDevice));
+        HIP_OK(c, hipDeviceSynchronize());
+        (void)hipFree(*p.src);
+        *p.src = nullptr;
+      }
+      w.w_in = all;
+      sm->max_in = std::max(sm->max_in, pad4(k.n));
+    }
+  }
+  for (auto& w : sm->L) {
+    if (w.w_src >= 0) {      // the lender's weights and what was derived from them; caches and states are allocated below
+      const int src = w.w_src;
+      w = sm->L[(size_t)src];
+      w.w_src = src;
+    }
+  }
+  for (auto& w : sm->L) {
+    const tgx_layer_desc& l = w.d;
+    if (l.mixer == TGX_MIXER_ATTENTION) {
+      const size_t rows = (size_t)sm->n_pages * sm->page, ke = rows * (size_t)l.maps * l.kv_heads * l.dim * es, ve = rows * (size_t)l.kv_heads * l.vdim * es;
+      if ((rc = dev_alloc(c, &w.pool, ke)) || (rc = dev_alloc(c, &w.poolV, ve))) return rc;
+      HIP_OK(c, hipMemset(w.pool, 0, ke));
+      HIP_OK(c, hipMemset(w.poolV, 0, ve));
+      if (gqa_mfma_shapes_ok(c->dt, l.dim, l.vdim, sm->page_shift, 4)) {      // (the projections' row stride is a multiple of four)
+        if ((rc = dev_alloc(c, &w.poolVT, ve))) return rc;
+        HIP_OK(c, hipMemset(w.poolVT, 0, ve));
+      }
+      continue;
+    }
+    const size_t se = B * (size_t)l.heads * l.dim * l.vdim;
+    if ((rc = dev_alloc(c, &w.mS, se))) return rc;
+    HIP_OK(c, hipMemset(w.mS, 0, se * 4));
+    if (l.mixer == TGX_MIXER_CHANNEL_DELTA && l.conv_taps > 1) {
+      const size_t ce = 2 * B * (size_t)(l.conv_taps - 1) * (size_t)ChannelDeltaCols(l).C;
+      if ((rc = dev_alloc(c, &w.conv_state, ce))) return rc;
+      HIP_OK(c, hipMemset(w.conv_state, 0, ce * 4));
+    }
+  }
+  return TGX_OK;
+}
+
 int run_layers(tgx_ctx* c, const MetaPtrs& mp, int T, int S, int max_keys, int max_count) {
+  if (c->stack->hyper) return run_layers_hyper(c, mp, T, S, max_keys, max_count);
   if (c->stack->post) return run_layers_post(c, mp, T, S, max_keys, max_count);
   if (c->stack->affine) return run_layers_affine(c, mp, T, S, max_keys, max_count);
   if (c->stack->joint) return run_layers_joint(c, mp, T, S, max_keys, max_count);
@@ -1478,7 +1968,7 @@ void run_logits(tgx_ctx* c, const int* want_dev, int nw, float* C, const int* c_
   StackModel* sm = c->stack;
   const int W = sm->d.width, V = sm->d.vocab;
   if (sm->affine) hipLaunchKernelGGL(tgx::layer_norm_rows_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->final_norm, sm->final_norm + W, sm->xn, W, sm->d.norm_eps);
-  else if (sm->joint || sm->post) hipLaunchKernelGGL(tgx::offset_norm_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->final_norm, sm->joint ? 1.0f : 0.0f, sm->xn, W, sm->d.norm_eps);
+  else if (sm->joint || sm->post || sm->hyper) hipLaunchKernelGGL(tgx::offset_norm_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->final_norm, sm->joint || sm->hyper ? 1.0f : 0.0f, sm->xn, W, sm->d.norm_eps);
   else if (sm->sandwich) hipLaunchKernelGGL(tgx::scalar_norm_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->norm_g + 4 * (size_t)sm->d.layers, sm->xn, W, sm->d.norm_eps);
   else hipLaunchKernelGGL(tgx::final_norm_rows_kernel, dim3(nw), dim3(256), 0, c->stream, sm->x, want_dev, sm->final_norm, sm->xn, W, sm->d.norm_groups, sm->d.norm_eps);
   tgx::StackGemmArgs g{};
@@ -1837,19 +2327,20 @@ int stack_create(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int d
   if (!desc || !layers || !out_ctx) return set_err(nullptr, TGX_ERR_INVALID, "null argument");
   *out_ctx = nullptr;
   const tgx_stack_desc& d = *desc;
-  if (d.family != TGX_FAMILY_ZAKUSUN && d.family != TGX_FAMILY_MODEPEL && d.family != TGX_FAMILY_VITUDRA && d.family != TGX_FAMILY_ZALUVIK && d.family != TGX_FAMILY_NUSOVIK) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "family %d is not a layered model", d.family);
-  const bool sandwich = d.family == TGX_FAMILY_MODEPEL, joint = d.family == TGX_FAMILY_VITUDRA, affine = d.family == TGX_FAMILY_ZALUVIK, post = d.family == TGX_FAMILY_NUSOVIK;
-  const bool latent = !sandwich && !joint && !affine && !post;
+  if (d.family != TGX_FAMILY_ZAKUSUN && d.family != TGX_FAMILY_MODEPEL && d.family != TGX_FAMILY_VITUDRA && d.family != TGX_FAMILY_ZALUVIK && d.family != TGX_FAMILY_NUSOVIK && d.family != TGX_FAMILY_KERONEX) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "family %d is not a layered model", d.family);
+  const bool sandwich = d.family == TGX_FAMILY_MODEPEL, joint = d.family == TGX_FAMILY_VITUDRA, affine = d.family == TGX_FAMILY_ZALUVIK, post = d.family == TGX_FAMILY_NUSOVIK, hyper = d.family == TGX_FAMILY_KERONEX;
+  const bool latent = !sandwich && !joint && !affine && !post && !hyper;
   if (d.width <= 0 || d.layers <= 0 || d.vocab <= 0 || d.max_seqs <= 0 || d.max_ctx <= 0) return set_err(nullptr, TGX_ERR_INVALID, "non-positive model dimension");
   if (d.compute_dtype != TGX_BF16 && d.compute_dtype != TGX_F16 && d.compute_dtype != TGX_F32) return set_err(nullptr, TGX_ERR_INVALID, "unknown compute dtype %d", d.compute_dtype);
   if (affine) { const int rc = check_affine_desc(d, layers); if (rc) return rc; }
   if (post) { const int rc = check_post_desc(d, layers); if (rc) return rc; }
+  if (hyper) { const int rc = check_hyper_desc(d, layers); if (rc) return rc; }
   if (latent && (d.norm_groups < 1 || d.norm_groups > tgx::NORM_MAX_GROUPS || d.width % d.norm_groups)) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "norm groups %d: 1..%d, dividing the width", d.norm_groups, tgx::NORM_MAX_GROUPS);
   if (latent && (d.canon_taps < 1 || d.canon_taps > tgx::CONV_MAX_TAPS)) return set_err(nullptr, TGX_ERR_UNSUPPORTED, "convolution taps %d: 1..%d", d.canon_taps, tgx::CONV_MAX_TAPS);
   int page = d.page_tokens > 0 ? d.page_tokens : 64;
   if (page & (page - 1)) return set_err(nullptr, TGX_ERR_INVALID, "page_tokens %d is not a power of two", page);
   int first_mix = -1;
-  for (int i = 0; i < d.layers && !affine && !post; i++) {
+  for (int i = 0; i < d.layers && !affine && !post && !hyper; i++) {
     const tgx_layer_desc& l = layers[i];
     if (joint) {
       auto attention_ok = [&](const char*& why) {
@@ -1927,8 +2418,8 @@ int stack_create(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int d
   while ((1 << sm->page_shift) < page) sm->page_shift++;
   // what the shared sampler / token rings read from the flat description
   c->d.family = d.family; c->d.hidden = d.width; c->d.layers = d.layers; c->d.vocab = d.vocab; c->d.max_ctx = d.max_ctx; c->d.max_batch = d.max_seqs;
-  c->d.compute_dtype = d.compute_dtype; c->d.tied = sandwich || joint || post ? 0 : 1; c->d.norm_eps = d.norm_eps;      // (a layer-norm design multiplies by the embedding table)
-  sm->sandwich = sandwich; sm->joint = joint; sm->affine = affine; sm->post = post;
+  c->d.compute_dtype = d.compute_dtype; c->d.tied = sandwich || joint || post || hyper ? 0 : 1; c->d.norm_eps = d.norm_eps;      // (a layer-norm design multiplies by the embedding table)
+  sm->sandwich = sandwich; sm->joint = joint; sm->affine = affine; sm->post = post; sm->hyper = hyper;
   c->device = device_ordinal;
   c->dt = d.compute_dtype == TGX_BF16 ? tgx::DT_BF16 : (d.compute_dtype == TGX_F16 ? tgx::DT_F16 : tgx::DT_F32);
   c->esz = d.compute_dtype == TGX_F32 ? 4 : 2;
@@ -1947,6 +2438,7 @@ int stack_create(const tgx_stack_desc* desc, const tgx_layer_desc* layers, int d
   if (joint) return create_joint_layers(c, layers);
   if (affine) return create_affine_layers(c, layers);
   if (post) return create_post_layers(c, layers);
+  if (hyper) return create_hyper_layers(c, layers);
   for (int i = 0; i < d.layers; i++) {
     StackLayerW& w = sm->L[(size_t)i];
     w.d = layers[i];
@@ -1989,6 +2481,7 @@ int stack_upload(tgx_ctx* c, const char* name, const void* host, const int64_t* 
   if (sm->joint) return upload_joint(c, name, host, shape, nd, src_dtype);
   if (sm->affine) return upload_affine(c, name, host, shape, nd, src_dtype);
   if (sm->post) return upload_post(c, name, host, shape, nd, src_dtype);
+  if (sm->hyper) return upload_hyper(c, name, host, shape, nd, src_dtype);
   if (!strcmp(name, "embed")) { if (probe) return TGX_ERR_SHAPE; if (!is(d.vocab, W)) return bad_shape(); return done(upload_param_ext(c, c->embed, host, d.vocab * W, src_dtype)); }
   if (!strcmp(name, "final.norm")) { if (probe) return TGX_ERR_SHAPE; if (!is(W, -1)) return bad_shape(); return done(upload_f32(c, sm->final_norm, host, W, src_dtype)); }
   int li = -1;
@@ -2102,8 +2595,9 @@ int stack_finalize(tgx_ctx* c) {
       }
     }
   }
+  if (sm->hyper && (rc = finalize_hyper(c))) return rc;
   for (auto& w : sm->L) {
-    if (sm->affine) break;
+    if (sm->affine || sm->hyper) break;
     if (sm->post) {
       const tgx_layer_desc& l = w.d;
       const bool par = l.mixer == TGX_MIXER_PARALLEL;
@@ -2239,6 +2733,12 @@ void stack_destroy(tgx_ctx* c) {
   auto fr = [](void* p) { if (p) (void)hipFree(p); };
   for (auto& w : sm->L) {
     if (w.kv_src >= 0) w.pool = w.poolV = w.poolVT = nullptr;      // borrowed
+    if (w.w_src >= 0) {      // everything but the cache and the states is the lender's
+      StackLayerW own;
+      own.pool = w.pool; own.poolV = w.poolV; own.poolVT = w.poolVT; own.mS = w.mS; own.conv_state = w.conv_state;
+      w = own;
+    }
+    fr(w.hc); fr(w.decays); fr(w.w_b); fr(w.w_g1); fr(w.w_g2);
     fr(w.conv_b); fr(w.d_skip); fr(w.decay2); fr(w.q_norm); fr(w.k_norm); fr(w.dist);
     fr(w.w_o2); fr(w.w_w1); fr(w.w_w2); fr(w.mu); fr(w.w0); fr(w.ubonus); fr(w.conv_w); fr(w.a_log); fr(w.dt_bias); fr(w.shift);
     fr(w.norm1); fr(w.norm2); fr(w.canon1); fr(w.canon2); fr(w.dwa); fr(w.w_in); fr(w.w_ukT); fr(w.w_uv); fr(w.w_o); fr(w.lat_norm); fr(w.sink);
@@ -2248,6 +2748,7 @@ void stack_destroy(tgx_ctx* c) {
   for (auto& r : sm->rot) fr(r.cs);
   for (auto& r : sm->runs) { fr(r.pool); fr(r.poolV); fr(r.poolT); }
   for (auto& w : sm->L) { fr(w.ln); fr(w.talk); fr(w.pb); }
+  fr(sm->pair); fr(sm->last_tok);
   fr(sm->w_loop); fr(sm->xcat); fr(sm->qplanes);
   fr(sm->mixed); fr(sm->lora); fr(sm->rec_in);
   fr(sm->head); fr(sm->norm_g); fr(sm->a2); fr(sm->ytmp); fr(sm->ysh); fr(sm->sgw); fr(sm->vfirst); fr(sm->hs);
@@ -2409,9 +2910,9 @@ int stack_read_latent(tgx_ctx* c, int row, int layer, float* out) {
   if (row < 0 || row >= sm->d.max_seqs || layer < 0 || layer >= sm->d.layers || !out) return set_err(c, TGX_ERR_INVALID, "read_kv: row / layer out of range");
   HIP_OK(c, hipStreamSynchronize(c->stream));
   const StackLayerW& w = sm->L[(size_t)layer];
-  if ((sm->sandwich && w.d.mixer != TGX_MIXER_ATTENTION) || ((sm->joint || sm->post) && !w.pool)) return set_err(c, TGX_ERR_UNSUPPORTED, "read_kv: layer %d caches no rows (its state is recurrent)", layer);
+  if ((sm->sandwich && w.d.mixer != TGX_MIXER_ATTENTION) || ((sm->joint || sm->post || sm->hyper) && !w.pool)) return set_err(c, TGX_ERR_UNSUPPORTED, "read_kv: layer %d caches no rows (its state is recurrent)", layer);
   const ebyte* pool = w.pool;
-  size_t R = sm->sandwich || sm->joint || sm->post ? (size_t)w.d.kv_heads * w.d.dim : (size_t)w.d.kv_rank;      // an attention layer's cached keys, all key heads of a token in a row
+  size_t R = sm->sandwich || sm->joint || sm->post || sm->hyper ? (size_t)std::max(1, w.d.maps) * w.d.kv_heads * w.d.dim : (size_t)w.d.kv_rank;      // an attention layer's cached keys, all key heads of a token in a row
   if (sm->affine) {      // the cache of the layer's first run: an attention layer's keys, a latent layer's rows [latent | rotated key part]
     for (const StackRun& r : sm->runs) if (r.layer == layer) { pool = r.pool; break; }
     R = w.d.mixer == TGX_MIXER_ATTENTION ? (size_t)w.d.kv_heads * w.d.dim : (size_t)(w.d.kv_rank + w.d.rot_dim);
@@ -2431,7 +2932,7 @@ int64_t stack_bytes_per_token(const tgx_ctx* c, int64_t T) {
   const StackModel* sm = c->stack;
   const int64_t W = sm->d.width, es = (int64_t)c->esz;
   int64_t b = (int64_t)sm->d.vocab * W * es;
-  if (sm->sandwich || sm->joint || sm->post) b *= 2;      // embedding row aside, the head is a matrix of its own
+  if (sm->sandwich || sm->joint || sm->post || sm->hyper) b *= 2;      // embedding row aside, the head is a matrix of its own
   if (sm->affine) {      // per run of a layer: its matrices (the chosen experts only) and the rows of its cache inside the mask's span
     if (sm->w_loop) b += (int64_t)sm->d.loop_times * 2 * W * W * es;
     for (const StackRun& r : sm->runs) {
@@ -2447,6 +2948,14 @@ int64_t stack_bytes_per_token(const tgx_ctx* c, int64_t T) {
   for (const auto& w : sm->L) {
     const tgx_layer_desc& l = w.d;
     const int64_t H = l.heads, qd = H * l.dim, R = l.kv_rank, vd = H * l.vdim;
+    if (sm->hyper) {     // a layer's matrices (the chosen experts only; a borrowing layer streams the lender's again), its cached rows, or its state (read and written)
+      if (l.mixer == TGX_MIXER_ATTENTION) b += (((int64_t)l.maps * (H + l.kv_heads) * l.dim + (int64_t)l.kv_heads * l.vdim) * W + W * vd) * es + T * l.kv_heads * ((int64_t)l.maps * l.dim + l.vdim) * es;
+      else if (l.mixer == TGX_MIXER_RETENTION) b += (2 * qd + 3 * vd) * W * es + 2 * qd * l.vdim * 4;
+      else b += ((2 * (int64_t)l.kv_heads * l.dim + 2 * vd + H + l.decay_rank + l.gate_rank) * W + (int64_t)l.decay_rank * qd + (int64_t)l.gate_rank * vd) * es + 2 * qd * l.vdim * 4;
+      if (l.mlp == TGX_MLP_DENSE) b += 3 * (int64_t)l.ff * W * es;
+      if (l.mlp == TGX_MLP_MOE) b += (int64_t)l.experts * W * 4 + (int64_t)l.top * 2 * l.ff * W * es + (int64_t)2 * l.shared_ff * W * es;
+      continue;
+    }
     if (sm->post) {      // the convolution tails are small beside a state, which is read and written
       if (l.mixer == TGX_MIXER_MAMBA1) b += ((int64_t)l.inner * (3 * W + 2 * l.dt_rank + 2 * l.d_dim)) * es + 3 * (int64_t)l.inner * l.d_dim * 4;
       else {

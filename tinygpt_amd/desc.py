@@ -273,14 +273,16 @@ FAMILY_MODEPEL = 7
 FAMILY_VITUDRA = 8
 FAMILY_ZALUVIK = 9
 FAMILY_NUSOVIK = 10
+FAMILY_KERONEX = 11
 STACK_FAMILY = {"zakusun": FAMILY_ZAKUSUN, "modepel": FAMILY_MODEPEL, "vitudra": FAMILY_VITUDRA, "zaluvik": FAMILY_ZALUVIK,
-                "nusovik": FAMILY_NUSOVIK}
-MIXER_BY_NAME = {"latent_attention": 1, "attention": 2, "mlstm": 3, "wkv": 4, "parallel": 5, "mamba1": 6}
+                "nusovik": FAMILY_NUSOVIK, "keronex": FAMILY_KERONEX}
+MIXER_BY_NAME = {"latent_attention": 1, "attention": 2, "mlstm": 3, "wkv": 4, "parallel": 5, "mamba1": 6, "retention": 7, "channel_delta": 8}
 MLP_BY_NAME = {None: 0, "moe": 1, "dense": 2}
 MASK_BY_NAME = {None: 0, "window": 1, "chunk": 2}
 # which mixers a design is made of (config.json "architecture" -> layer "type")
 MIXERS_OF = {"zakusun": ("latent_attention",), "modepel": ("attention", "mlstm"), "vitudra": ("attention", "wkv", "parallel"),
-             "zaluvik": ("attention", "latent_attention"), "nusovik": ("mamba1", "parallel")}
+             "zaluvik": ("attention", "latent_attention"), "nusovik": ("mamba1", "parallel"),
+             "keronex": ("retention", "attention", "channel_delta")}
 
 
 class CLayerDesc(ctypes.Structure):
@@ -300,7 +302,9 @@ class CLayerDesc(ctypes.Structure):
                 ("rot_dim", ctypes.c_int32), ("ff_act", ctypes.c_int32), ("router_fn", ctypes.c_int32), ("group_score", ctypes.c_int32),
                 ("router_norm", ctypes.c_int32),
                 ("v_is_k", ctypes.c_int32), ("head_sink", ctypes.c_int32), ("bias_max", ctypes.c_int32), ("bias_buckets", ctypes.c_int32),
-                ("right_kind", ctypes.c_int32), ("part_norms", ctypes.c_int32), ("inner", ctypes.c_int32), ("dt_rank", ctypes.c_int32)]
+                ("right_kind", ctypes.c_int32), ("part_norms", ctypes.c_int32), ("inner", ctypes.c_int32), ("dt_rank", ctypes.c_int32),
+                ("maps", ctypes.c_int32), ("diff", ctypes.c_float), ("gate_rank", ctypes.c_int32), ("router_in", ctypes.c_int32), ("expert_act", ctypes.c_int32),
+                ("weights_of", ctypes.c_int32), ("n_decays", ctypes.c_int32), ("decays", ctypes.POINTER(ctypes.c_float))]
 
 
 class CStackDesc(ctypes.Structure):
@@ -309,7 +313,8 @@ class CStackDesc(ctypes.Structure):
                 ("compute_dtype", ctypes.c_int32), ("max_seqs", ctypes.c_int32), ("max_ctx", ctypes.c_int32),
                 ("budget_tokens", ctypes.c_int32), ("page_tokens", ctypes.c_int32), ("norm_groups", ctypes.c_int32),
                 ("norm_eps", ctypes.c_float), ("canon_taps", ctypes.c_int32), ("logit_scale", ctypes.c_float), ("residual_mult", ctypes.c_float),
-                ("embed_scale", ctypes.c_float), ("loop_start", ctypes.c_int32), ("loop_stop", ctypes.c_int32), ("loop_times", ctypes.c_int32)]
+                ("embed_scale", ctypes.c_float), ("loop_start", ctypes.c_int32), ("loop_stop", ctypes.c_int32), ("loop_times", ctypes.c_int32),
+                ("streams", ctypes.c_int32), ("bigram_buckets", ctypes.c_int32), ("bigram_before", ctypes.c_int64), ("bigram_cur", ctypes.c_int64)]
 
 
 @dataclass
@@ -379,6 +384,14 @@ class LayerDesc:
     part_norms: int = 1
     inner: int = 0
     dt_rank: int = 0
+    # the hyper-connected design (Keronex): two-map attention, retention, the delta rule with channel decays, experts behind their weights, shared weights
+    maps: int = 1                     # score maps per head over the same values
+    diff: float = 0.0
+    gate_rank: int = 0
+    router_in: bool = False           # a router weight multiplies its expert's input
+    expert_act: "str | None" = None   # None: the family's own; "relu2"
+    weights_of: "int | None" = None   # the layer whose tensors this one uses
+    decays: tuple = ()                # retention: one per head
 
     def to_c(self) -> CLayerDesc:
         return CLayerDesc(MIXER_BY_NAME[self.mixer], self.heads, self.dim, self.vdim, self.kv_rank, self.scale,
@@ -389,9 +402,12 @@ class LayerDesc:
                           int(self.rot_pairs), self.rot_factor, 0 if self.kv_from is None else self.kv_from + 1, self.decay_rank,
                           self.d_heads, self.d_kv_heads, self.d_dim, self.d_vdim, self.conv_taps, self.left_scale, self.right_scale,
                           2 if self.qk_norm == "weighted" else int(self.qk_norm), {None: 0, "sigmoid": 1}[self.score_fn], int(self.head_mix), {None: 0, "channel": 1, "head": 2}[self.gate_kind],
-                          self.rot_dim, {None: 0, "gelu": 1, "relu2": 2}[self.ff_act], {None: 0, "sigmoid": 1}[self.router_fn], {None: 0, "top2": 1}[self.group_score],
+                          self.rot_dim, {None: 0, "gelu": 1, "relu2": 2, "gelu_tanh_gated": 3}[self.ff_act], {None: 0, "sigmoid": 1}[self.router_fn], {None: 0, "top2": 1}[self.group_score],
                           int(self.router_norm), int(self.v_is_k), int(self.head_sink), self.bias_max, self.bias_buckets,
-                          {None: 0, "ssd": 1}[self.right_kind], self.part_norms, self.inner, self.dt_rank)
+                          {None: 0, "ssd": 1}[self.right_kind], self.part_norms, self.inner, self.dt_rank,
+                          self.maps, self.diff, self.gate_rank, int(self.router_in), {None: 0, "relu2": 1}[self.expert_act],
+                          0 if self.weights_of is None else self.weights_of + 1, len(self.decays),
+                          (ctypes.c_float * len(self.decays))(*self.decays) if self.decays else None)
 
 
 @dataclass
@@ -415,6 +431,10 @@ class StackDesc:
     loop_start: int = 0          # Zaluvik: layers loop_start .. loop_stop - 1 run loop_times times with the same weights, a cache per pass
     loop_stop: int = 0
     loop_times: int = 1
+    streams: int = 0             # Keronex: residual streams with learned mixes (0: the plain residual)
+    bigram_buckets: int = 0      # Keronex: rows of the pair table without the first token's; row = (before * bigram_before + token * bigram_cur) mod bigram_buckets
+    bigram_before: int = 0
+    bigram_cur: int = 0
     name: str = ""
 
     # the fields the flat description shares (bench / reporting code reads them)
@@ -428,7 +448,8 @@ class StackDesc:
         arr = (CLayerDesc * len(self.layers))(*[l.to_c() for l in self.layers])
         sd = CStackDesc(STACK_FAMILY[self.family], self.width, len(self.layers), self.vocab, DTYPE_BY_NAME[self.compute_dtype], self.max_seqs,
                         self.max_ctx, self.budget_tokens, self.page_tokens, self.norm_groups, self.norm_eps, self.canon_taps,
-                        self.logit_scale, self.residual_mult, self.embed_scale, self.loop_start, self.loop_stop, self.loop_times)
+                        self.logit_scale, self.residual_mult, self.embed_scale, self.loop_start, self.loop_stop, self.loop_times,
+                        self.streams, self.bigram_buckets, self.bigram_before, self.bigram_cur)
         return sd, arr
 
     @property
@@ -455,6 +476,8 @@ class StackDesc:
             return _zaluvik_shapes(self, out)
         if self.family == "nusovik":
             return _nusovik_shapes(self, out)
+        if self.family == "keronex":
+            return _keronex_shapes(self, out)
         for i, l in enumerate(self.layers):
             p = f"l{i}."
             out[p + "norm1"] = (W,)
@@ -598,6 +621,76 @@ def _nusovik_shapes(self: StackDesc, out: dict) -> dict:
     return out
 
 
+def _keronex_shapes(self: StackDesc, out: dict) -> dict:
+    """checkpoint names and shapes of a Keronex model, in file order (a layer that uses another's weights has none)"""
+    W, n = self.width, self.streams
+    if self.bigram_buckets:
+        out["bigram"] = (self.bigram_buckets + 1, W)
+    for i, l in enumerate(self.layers):
+        if l.weights_of is not None:
+            continue
+        p, q, H, D, E = f"l{i}.", f"l{i}.mix.", l.heads, l.dim, l.vdim
+        out[p + "norm1"] = (W,)
+        if l.mlp:
+            out[p + "norm2"] = (W,)
+        if l.mixer == "retention":
+            out[q + "q"] = (H * D, W); out[q + "k"] = (H * D, W); out[q + "v"] = (H * E, W); out[q + "g"] = (H * E, W)
+        elif l.mixer == "attention":
+            out[q + "q"] = (l.maps * H * D, W); out[q + "k"] = (l.maps * l.kv_heads * D, W); out[q + "v"] = (l.kv_heads * E, W)
+            for s in ("lq1", "lk1", "lq2", "lk2"):
+                out[q + s] = (D,)
+        else:
+            for s, c in (("q", l.kv_heads * D), ("k", l.kv_heads * D), ("v", H * E)):
+                out[q + s] = (c, W); out[q + s + ".conv"] = (c, l.conv_taps)
+            out[q + "b"] = (H, W); out[q + "A_log"] = (H,); out[q + "norm"] = (E,)
+            out[q + "a1"] = (l.decay_rank, W); out[q + "a2"] = (H * D, l.decay_rank); out[q + "dt_bias"] = (H * D,)
+            out[q + "g1"] = (l.gate_rank, W); out[q + "g2"] = (H * E, l.gate_rank)
+        out[q + "o"] = (W, H * E)
+        if l.mlp == "dense":
+            out[p + "mlp.gate"] = (l.ff, W); out[p + "mlp.up"] = (l.ff, W); out[p + "mlp.down"] = (W, l.ff)
+        elif l.mlp == "moe":
+            for e in range(l.experts):
+                out[p + f"mlp.e{e}.up"] = (l.ff, W); out[p + f"mlp.e{e}.down"] = (W, l.ff)
+            out[p + "mlp.router"] = (l.experts, W)
+            if l.shared_ff:
+                out[p + "mlp.shared.up"] = (l.shared_ff, W); out[p + "mlp.shared.down"] = (W, l.shared_ff)
+        if n:
+            for s in ("hc1", "hc2") if l.mlp else ("hc1",):
+                out[p + s + ".in"] = (n,); out[p + s + ".out"] = (n,); out[p + s + ".mix"] = (n, n)
+    out["final.norm"] = (W,)
+    out["head"] = (self.vocab, W)
+    return out
+
+
+def _keronex_layer(i: int, l: dict, rank_a: int = 0, rank_g: int = 0) -> LayerDesc:
+    """one entry of a Keronex config's "layers": {"type": "retention" | "attention" | "channel_delta", "mixer": {...}, "mlp": null | {"kind": "dense" | "moe", ...},
+    "weights_of": layer}.  Attention has two maps per head; the inner sizes of a channel_delta layer's low-rank products are its tensors'."""
+    m, f = l["mixer"], l.get("mlp")
+    ld = LayerDesc(mixer=l["type"], heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])))
+    ld.kv_heads = int(m.get("kv_heads", ld.heads))
+    ld.weights_of = int(l["weights_of"]) if l.get("weights_of") is not None else None
+    if l["type"] == "channel_delta":
+        ld.conv_taps = int(m.get("conv", 1)); ld.decay_rank = int(rank_a); ld.gate_rank = int(rank_g)
+    else:
+        rot = m.get("rot") or {}
+        ld.rot_dims = int(rot.get("dims", 0)); ld.rot_base = float(rot.get("base", 10000.0))
+        if l["type"] == "retention":
+            ld.decays = tuple(float(d) for d in m["decay"])
+        else:
+            ld.maps = 2; ld.diff = float(m["diff"]); ld.scale = float(m["scale"])
+    if f is None:
+        return ld
+    if f.get("kind") == "dense":
+        ld.mlp = "dense"; ld.ff = int(f["ff"]); ld.ff_act = "gelu_tanh_gated"
+    elif f.get("kind") == "moe":
+        ld.mlp = "moe"; ld.experts = int(f["router"]["experts"]); ld.top = int(f["router"]["top"]); ld.ff = int(f["expert"]["ff"])
+        ld.shared_ff = int(f["shared"]["ff"]) if f.get("shared") else 0
+        ld.router_fn = "sigmoid"; ld.router_in = True; ld.expert_act = "relu2"
+    else:
+        raise ValueError(f"layer {i}: feed-forward kind {f.get('kind')!r} is not implemented")
+    return ld
+
+
 def _nusovik_layer(i: int, l: dict, buckets: int = 0) -> LayerDesc:
     """one entry of a Nusovik config's "layers": {"type": "mamba1" | "parallel", "mixer": {...}, "mlp": null | {"kind": "dense", "ff"}}.
     A parallel mixer is {"left": chunked attention whose values are its keys, with a bucketed distance bias, sinks and a gate per head, "right": a scalar-decay
@@ -718,8 +811,8 @@ def _modepel_layer(i: int, l: dict) -> LayerDesc:
 
 
 def stack_desc_from_config(cfg: dict, compute_dtype: str = "bf16", max_seqs: int = 4, max_ctx: int = 4096, budget_tokens: int = 0, tensor_shapes=None) -> StackDesc:
-    """config.json of a layered model ("architecture": "Zakusun" | "Modepel" | "Vitudra" | "Zaluvik" | "Nusovik") -> StackDesc.  Every size and constant comes from the file;
-    tensor_shapes (checkpoint name -> shape, optional) gives the sizes that only a tensor's shape tells (a wkv layer's decay rank, the rows of a distance table; left open without it:
+    """config.json of a layered model ("architecture": "Zakusun" | "Modepel" | "Vitudra" | "Zaluvik" | "Nusovik" | "Keronex") -> StackDesc.  Every size and constant comes from the file;
+    tensor_shapes (checkpoint name -> shape, optional) gives the sizes that only a tensor's shape tells (a wkv layer's decay rank, the rows of a distance table, the ranks of a channel_delta layer; left open without it:
     the device library then takes it from the tensor at upload)."""
     arch = str(cfg.get("architecture")).lower()
     if arch not in MIXERS_OF:
@@ -746,6 +839,14 @@ def stack_desc_from_config(cfg: dict, compute_dtype: str = "bf16", max_seqs: int
                          layers=[_nusovik_layer(i, l, (ts.get(f"l{i}.mix.left.rel") or (0,))[0]) for i, l in enumerate(cfg["layers"])], compute_dtype=compute_dtype,
                          max_seqs=max_seqs, max_ctx=max_ctx, budget_tokens=budget_tokens, norm_groups=1, norm_eps=float(cfg["norm"]["eps"]), canon_taps=1,
                          logit_scale=float(cfg.get("logit_scale", 1.0)), embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)), name="nusovik")
+    if arch == "keronex":
+        ts, em = tensor_shapes or {}, cfg.get("embedding") or {}
+        bg = em.get("bigram") or {}
+        rank = lambda i, n: (ts.get(f"l{i}.mix.{n}") or (0,))[0]
+        return StackDesc(family="keronex", width=int(cfg["width"]), vocab=int(cfg["vocab"]), layers=[_keronex_layer(i, l, rank(i, "a1"), rank(i, "g1")) for i, l in enumerate(cfg["layers"])],
+                         compute_dtype=compute_dtype, max_seqs=max_seqs, max_ctx=max_ctx, budget_tokens=budget_tokens, norm_groups=1, norm_eps=float(cfg["norm"]["eps"]),
+                         canon_taps=1, logit_scale=1.0, embed_scale=float(em.get("scale", 1.0)), streams=int(cfg.get("streams", 0)), bigram_buckets=int(bg.get("buckets", 0)),
+                         bigram_before=int(bg.get("mul_prev", 0)), bigram_cur=int(bg.get("mul_cur", 0)), name="keronex")
     if arch == "modepel":
         return StackDesc(family="modepel", width=int(cfg["width"]), vocab=int(cfg["vocab"]), layers=[_modepel_layer(i, l) for i, l in enumerate(cfg["layers"])],
                          compute_dtype=compute_dtype, max_seqs=max_seqs, max_ctx=max_ctx, budget_tokens=budget_tokens, norm_groups=1,

@@ -217,6 +217,48 @@ static bool load_nusovik_layer(const Json& L, size_t i, tgx_layer_desc& l, std::
   return true;
 }
 
+// one entry of a Keronex config's "layers": {"type": "retention" | "attention" | "channel_delta", "mixer": {...}, "mlp": null | {"kind": "dense" | "moe", ...}, "weights_of": layer}.
+// The inner sizes of a channel_delta layer's low-rank products are left open: the device library takes them from the tensors' shapes.
+static bool load_keronex_layer(const Json& L, size_t i, tgx_layer_desc& l, std::vector<float>& decays, std::string& err) {
+  auto dim = [](const Json& j, const char* key) -> int32_t { const int64_t v = j.get_int(key, -1); return (v < 0 || v > ((int64_t)1 << 30)) ? -1 : (int32_t)v; };
+  const Json* mx = L.get("mixer");
+  const Json* ff = L.get("mlp");
+  const std::string type = L.get_str("type", "");
+  auto bad = [&](const std::string& what) { err = "config.json: layer " + std::to_string(i) + ": " + what; return false; };
+  if (!mx || mx->kind != Json::Obj) return bad("no mixer");
+  l.heads = dim(*mx, "heads"); l.kv_heads = mx->has("kv_heads") ? dim(*mx, "kv_heads") : l.heads; l.dim = dim(*mx, "dim"); l.vdim = mx->has("vdim") ? dim(*mx, "vdim") : l.dim;
+  l.maps = 1; l.scale = 1.f; l.rot_base = 10000.f;
+  const Json* of = L.get("weights_of");
+  if (of && of->kind != Json::Null) { const int32_t j = dim(L, "weights_of"); if (j < 0) return bad("weights_of"); l.weights_of = j + 1; }
+  const Json* rot = mx->get("rot");
+  if (type != "channel_delta" && rot && rot->kind == Json::Obj) { l.rot_dims = dim(*rot, "dims"); l.rot_base = rot->get_float("base", 10000.f); }
+  if (type == "retention") {
+    l.mixer = TGX_MIXER_RETENTION;
+    const Json* d = mx->get("decay");
+    if (!d || d->kind != Json::Arr) return bad("retention without decays");
+    for (const Json& v : d->arr) { if (v.kind != Json::Num) return bad("decay"); decays.push_back((float)v.num); }
+    l.n_decays = (int32_t)decays.size(); l.decays = decays.data();
+  } else if (type == "attention") {
+    l.mixer = TGX_MIXER_ATTENTION;
+    l.maps = 2; l.diff = mx->get_float("diff", 0.f); l.scale = mx->get_float("scale", 1.f);
+  } else if (type == "channel_delta") {
+    l.mixer = TGX_MIXER_CHANNEL_DELTA;
+    l.conv_taps = mx->has("conv") ? dim(*mx, "conv") : 1;
+  } else return bad("mixer '" + type + "' is not implemented");
+  if (!ff || ff->kind != Json::Obj) return true;
+  const std::string kind = ff->get_str("kind", "");
+  if (kind == "dense") { l.mlp = TGX_MLP_DENSE; l.ff = dim(*ff, "ff"); l.ff_act = 3; return true; }
+  const Json* ex = ff->get("expert");
+  const Json* ro = ff->get("router");
+  if (kind != "moe" || !ro || ro->kind != Json::Obj || !ex || ex->kind != Json::Obj) return bad("feed-forward kind '" + kind + "' is not implemented");
+  l.mlp = TGX_MLP_MOE;
+  l.experts = dim(*ro, "experts"); l.top = dim(*ro, "top"); l.ff = dim(*ex, "ff"); l.router_scale = 1.f; l.groups = 1; l.groups_keep = 1;
+  l.router_fn = 1; l.router_in = 1; l.expert_act = 1;
+  const Json* sh = ff->get("shared");
+  l.shared_ff = sh && sh->kind == Json::Obj ? dim(*sh, "ff") : 0;
+  return true;
+}
+
 // config.json of a layered model: {"architecture": "Zakusun", "width", "vocab", "logit_scale", "norm": {"eps", "groups"}, "canon": {"taps"},
 // "layers": [{"type": mixer, "mixer": {heads, dim, vdim, kv_rank, scale}, "mlp": null | {"kind": "moe", "expert": {ff, limit}, "router": {experts, top}}}]}
 // or {"architecture": "Modepel", "width", "vocab", "norm": {"eps"}, "layers": [...]} with the layer entries of load_modepel_layer
@@ -225,19 +267,26 @@ static bool load_nusovik_layer(const Json& L, size_t i, tgx_layer_desc& l, std::
 // with the layer entries of load_zaluvik_layer (logits against the embedding table)
 // or {"architecture": "Nusovik", "width", "vocab", "logit_scale", "embedding": {"scale"}, "norm": {"eps"}, "layers": [...]} with the layer entries of
 // load_nusovik_layer
+// or {"architecture": "Keronex", "width", "vocab", "streams", "embedding": {"scale", "bigram": {"buckets", "mul_prev", "mul_cur"}}, "norm": {"eps"}, "layers": [...]} with the
+// layer entries of load_keronex_layer
 static bool load_stack_config(const Json& doc, const std::string& path, int compute_dtype, int max_batch, int max_ctx, int budget_tokens, ModelConfig& out, std::string& err) {
   const std::string arch = doc.get_str("architecture", "");
-  const bool vitudra = arch == "Vitudra", zaluvik = arch == "Zaluvik", nusovik = arch == "Nusovik", modepel = arch == "Modepel" || vitudra || zaluvik || nusovik;      // (all four: a config header without norm groups and taps)
+  const bool vitudra = arch == "Vitudra", zaluvik = arch == "Zaluvik", nusovik = arch == "Nusovik", keronex = arch == "Keronex", modepel = arch == "Modepel" || vitudra || zaluvik || nusovik || keronex;      // (all five: a config header without norm groups and taps)
   if (arch != "Zakusun" && !modepel) { err = "Unsupported architecture: " + arch; return false; }
   auto dim = [](const Json& j, const char* key) -> int32_t { const int64_t v = j.get_int(key, -1); return (v < 0 || v > ((int64_t)1 << 30)) ? -1 : (int32_t)v; };
   out.layered = true;
-  out.model_type = nusovik ? "nusovik" : zaluvik ? "zaluvik" : vitudra ? "vitudra" : modepel ? "modepel" : "zakusun";
+  out.model_type = keronex ? "keronex" : nusovik ? "nusovik" : zaluvik ? "zaluvik" : vitudra ? "vitudra" : modepel ? "modepel" : "zakusun";
   tgx_stack_desc& s = out.stack;
-  s.family = nusovik ? TGX_FAMILY_NUSOVIK : zaluvik ? TGX_FAMILY_ZALUVIK : vitudra ? TGX_FAMILY_VITUDRA : modepel ? TGX_FAMILY_MODEPEL : TGX_FAMILY_ZAKUSUN;
+  s.family = keronex ? TGX_FAMILY_KERONEX : nusovik ? TGX_FAMILY_NUSOVIK : zaluvik ? TGX_FAMILY_ZALUVIK : vitudra ? TGX_FAMILY_VITUDRA : modepel ? TGX_FAMILY_MODEPEL : TGX_FAMILY_ZAKUSUN;
   s.residual_mult = doc.get_float("residual_mult", 1.f);
   s.embed_scale = 1.f; s.loop_times = 1;
   const Json* em = doc.get("embedding");
-  if ((zaluvik || nusovik) && em && em->kind == Json::Obj) s.embed_scale = em->get_float("scale", 1.f);
+  if ((zaluvik || nusovik || keronex) && em && em->kind == Json::Obj) s.embed_scale = em->get_float("scale", 1.f);
+  if (keronex) {
+    s.streams = doc.has("streams") ? dim(doc, "streams") : 0;
+    const Json* bg = em && em->kind == Json::Obj ? em->get("bigram") : nullptr;
+    if (bg && bg->kind == Json::Obj) { s.bigram_buckets = dim(*bg, "buckets"); s.bigram_before = bg->get_int("mul_prev", 0); s.bigram_cur = bg->get_int("mul_cur", 0); }
+  }
   if (zaluvik) {
     const Json* lp = doc.get("loop");
     if (lp && lp->kind == Json::Obj) { s.loop_start = dim(*lp, "start"); s.loop_stop = dim(*lp, "stop"); s.loop_times = dim(*lp, "times"); }
@@ -255,11 +304,12 @@ static bool load_stack_config(const Json& doc, const std::string& path, int comp
     err = "config.json: norm / canon / layers are missing in " + path; return false;
   }
   s.norm_groups = modepel ? 1 : dim(*norm, "groups"); s.norm_eps = norm->get_float("eps", 1e-6f); s.canon_taps = modepel ? 1 : dim(*canon, "taps");
+  out.decays.resize(layers->arr.size());      // (sized once: the layers point into it)
   for (size_t i = 0; i < layers->arr.size(); i++) {
     const Json& L = layers->arr[i];
     tgx_layer_desc l{};
     if (modepel) {
-      if (!(nusovik ? load_nusovik_layer(L, i, l, err) : zaluvik ? load_zaluvik_layer(L, i, l, err) : vitudra ? load_vitudra_layer(L, i, l, err) : load_modepel_layer(L, i, l, err))) return false;
+      if (!(keronex ? load_keronex_layer(L, i, l, out.decays[i], err) : nusovik ? load_nusovik_layer(L, i, l, err) : zaluvik ? load_zaluvik_layer(L, i, l, err) : vitudra ? load_vitudra_layer(L, i, l, err) : load_modepel_layer(L, i, l, err))) return false;
       out.layers.push_back(l);
       continue;
     }

@@ -27,6 +27,7 @@ struct ModelConfig {
   bool layered = false;
   tgx_stack_desc stack{};
   std::vector<tgx_layer_desc> layers;
+  std::vector<std::vector<float>> decays;      // per layer: what tgx_layer_desc::decays points to
   std::string model_type;
   std::string torch_dtype;
   int64_t bos_token_id = -1, eos_token_id = -1;
