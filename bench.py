@@ -84,7 +84,7 @@ def parse():
     ap.add_argument("--layered", default=None, metavar="SIZE[,SIZE]", help="instead of the headline: prefill and decode throughput of the layered (Zakusun) design at "
                     "layer sizes of real models (1b, 0.5b; random weights), beside a Llama-family model of the same width, depth and active parameters")
     ap.add_argument("--only", default="", help="with --layered: measure these models only (names before the size, with commas; for profiling one of them)")
-    ap.add_argument("--design", default="zakusun", choices=["zakusun", "modepel", "vitudra", "zaluvik", "nusovik"], help="with --layered: which layered design is measured beside its closest relatives and the Llama-family model")
+    ap.add_argument("--design", default="zakusun", choices=["zakusun", "modepel", "vitudra", "zaluvik", "nusovik", "keronex"], help="with --layered: which layered design is measured beside its closest relatives and the Llama-family model")
     ap.add_argument("--cpu-seconds", type=float, default=15.0, help="target CPU time of the cpu_baseline sample")
     return ap.parse_args()
 
@@ -400,6 +400,30 @@ def nusovik_desc(key, z, L, V, dtype, B, ctx):
                      name=f"nusovik-{key}", layers=layers)
 
 
+def keronex_desc(key, z, L, V, dtype, B, ctx):
+    """Keronex at the size of `z`: four residual streams; channel-decay delta rule, retention (values twice as wide as keys) and two-map attention in turn, the last
+    retention layer on an earlier one's weights; a gated feed-forward in the first layer, sigmoid-routed experts with a shared expert in the others"""
+    from tinygpt_amd.desc import LayerDesc, StackDesc
+    W = z["width"]
+    layers = []
+    for i in range(L):
+        if i % 3 == 0:
+            l = LayerDesc(mixer="channel_delta", heads=W // 128, kv_heads=max(1, W // 256), dim=128, vdim=128, conv_taps=4, decay_rank=128, gate_rank=128)
+        elif i % 3 == 1:
+            H = W // 256
+            l = LayerDesc(mixer="retention", heads=H, kv_heads=H, dim=128, vdim=256, rot_dims=128, rot_base=10000.0, decays=tuple(1.0 - 2.0 ** (-5 - h % 8) for h in range(H)))
+        else:
+            l = LayerDesc(mixer="attention", heads=W // 128, kv_heads=max(1, W // 512), dim=64, vdim=128, maps=2, diff=0.4, scale=64 ** -0.5, rot_dims=64, rot_base=500000.0)
+        if i == 0:
+            l.mlp, l.ff, l.ff_act = "dense", z["top"] * z["ff"], "gelu_tanh_gated"
+        else:
+            l.mlp, l.experts, l.top, l.ff, l.shared_ff, l.router_fn, l.router_in, l.expert_act = "moe", z["experts"], z["top"], z["ff"], z["ff"], "sigmoid", True, "relu2"
+        layers.append(l)
+    layers[7].weights_of = 1
+    return StackDesc(family="keronex", width=W, vocab=V, compute_dtype=dtype, max_seqs=B, max_ctx=ctx, budget_tokens=B * (ctx + 64), norm_eps=1e-5, embed_scale=2.0, streams=4,
+                     bigram_buckets=4093, bigram_before=31, bigram_cur=7, name=f"keronex-{key}", layers=layers)
+
+
 def layered_compare(args):
     from tinygpt_amd.desc import LayerDesc, ModelDesc, StackDesc
     from tinygpt_amd.ffi import GREEDY, Model
@@ -448,7 +472,9 @@ def layered_compare(args):
         todo = {"zakusun": [(sd, True)], "modepel": [(modepel_desc(key, z, L, V, args.dtype, B, ctx), True), (sd, True)],
                 "vitudra": [(vitudra_desc(key, z, L, V, args.dtype, B, ctx), True), (modepel_desc(key, z, L, V, args.dtype, B, ctx), True)],
                 "zaluvik": [(zaluvik_desc(key, z, L, V, args.dtype, B, ctx), True), (modepel_desc(key, z, L, V, args.dtype, B, ctx), True), (sd, True)],
-                "nusovik": [(nusovik_desc(key, z, L, V, args.dtype, B, ctx), True), (vitudra_desc(key, z, L, V, args.dtype, B, ctx), True)]}[args.design] + [(ld, False)]
+                "nusovik": [(nusovik_desc(key, z, L, V, args.dtype, B, ctx), True), (vitudra_desc(key, z, L, V, args.dtype, B, ctx), True)],
+                "keronex": [(keronex_desc(key, z, L, V, args.dtype, B, ctx), True), (vitudra_desc(key, z, L, V, args.dtype, B, ctx), True),
+                            (modepel_desc(key, z, L, V, args.dtype, B, ctx), True), (nusovik_desc(key, z, L, V, args.dtype, B, ctx), True)]}[args.design] + [(ld, False)]
         if args.only:
             todo = [t for t in todo if t[0].name.split("-")[0] in args.only.split(",")]
         for desc, layered in todo:
