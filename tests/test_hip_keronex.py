@@ -174,6 +174,8 @@ MECH = {
     "experts_without_a_shared_one": [cd(moe(6, 2, 9, 0))],
     "experts_wide_shared": [cd(moe(6, 3, 9, 50))],
     "experts_more_than_a_wave": [ret(moe(90, 5, 6, 7))],
+    "experts_shared_of_the_same_size": [attn(moe(6, 2, 16, 16))],
+    "experts_shared_of_the_same_odd_size": [attn(moe(6, 2, 11, 11))],
     "shared_weights_next_to_each_other": [ret(moe()), dict(ret(moe()), weights_of=0)],
     "shared_weights_of_attention": [attn(dense()), cd(), dict(attn(dense()), weights_of=0)],
     "shared_weights_of_channel_delta": [cd(), attn(), dict(cd(), weights_of=0)],
@@ -407,6 +409,19 @@ def test_a_router_weight_stands_in_front_of_the_square():
     finally:
         ko.experts_ff = front
     assert np.abs(out - want).max() / np.abs(want).max() > 1e-2
+
+
+@pytest.mark.parametrize("dtype", ["fp32", "bf16"])
+@pytest.mark.parametrize("n", [2, 21, 31, 32, 33, 42, 43, 70])
+def test_a_shared_expert_of_the_routed_size(n, dtype):
+    """steps of few pairs take the shared expert as one more choice, longer ones compute it by itself: portions on both sides of the border (128 pairs)"""
+    cfg = config([ret(moe(5, 3, 16, 16)), cd(moe(9, 2, 24, 24))])
+    toks = tokens(cfg, n + 4, seed=n)
+    w = ko.random_tensors(cfg, 13)
+    want = clear(cfg, w, [toks], 13)[0]
+    eng, _ = engine(cfg, dtype, 13, w)
+    check_rows(np.concatenate([eng.step([("r", toks[:n], list(range(n)))])] + [eng.step([("r", [t], [0])]) for t in toks[n:]]), want, dtype, "", cfg)
+    eng.close()
 
 
 # ---- batches, slots, pages ----------------------------------------------------------------------------------------------------------------

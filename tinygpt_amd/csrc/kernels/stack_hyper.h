@@ -4,12 +4,14 @@
 //   pair_embed_kernel       embedding row * scale + the row of the pair (token before, token), into every stream; the first sublayer's normed input; the slot's last token
 //   hyper_seam_kernel       the seam between two sublayers: the streams take the sublayer's output and each other's shares, the next sublayer's normed input leaves
 //   map_difference_kernel   o_1 - lambda o_2 of a head's two maps, RMS norm over the head, constant factor
+//   map_difference_merge_kernel   the same on the records of an attention whose keys were divided between workgroups
 #pragma once
 #include "stack_seq.h"
 
 namespace tgx {
 
 constexpr int HYPER_MAX_STREAMS = 16;
+constexpr int PAIR_REG = 16;      // channels a thread of the embedding kernel keeps
 constexpr int HYPER_REG = 4;      // vectors of four channels a thread keeps between the passes: widths up to 4096
 
 // u_t = sum_s w_in[s] x_s, out_t = u_t / sqrt(mean(u_t^2) + eps) * (1 + w_norm)
@@ -39,19 +41,25 @@ __global__ __launch_bounds__(256) void pair_embed_kernel(StepMeta m, PairEmbedAr
     pr = reinterpret_cast<const elem_t<DT>*>(a.pair) + (size_t)b * a.W;
     if (i == m.tok_cnt[t] - 1 && threadIdx.x == 0) a.last[(size_t)(par ^ 1) * a.slots + row] = id;
   }
-  float* x = a.xs + (size_t)t * a.n * a.W;
-  float sum = 0.f, ss = 0.f;
+  float* __restrict__ x = a.xs + (size_t)t * a.n * a.W;
+  float* __restrict__ out = a.in.out + (size_t)t * a.W;
+  float sum = 0.f, ss = 0.f, v[PAIR_REG];
   for (int s = 0; s < a.n; s++) sum += a.in.w_in[s];
-  for (int c = threadIdx.x; c < a.W; c += 256) {
-    float v = elem_to_f32<DT>(er[c]) * a.scale;
-    if (pr) v += elem_to_f32<DT>(pr[c]);
-    for (int s = 0; s < a.n; s++) x[(size_t)s * a.W + c] = v;
-    const float u = sum * v;
-    ss = fmaf(u, u, ss);
-  }
+  auto value = [&](int c) -> float { return fmaf(elem_to_f32<DT>(er[c]), a.scale, pr ? elem_to_f32<DT>(pr[c]) : 0.f); };
+#pragma unroll
+  for (int k = 0; k < PAIR_REG; k++) { const int c = threadIdx.x + 256 * k; v[k] = c < a.W ? value(c) : 0.f; }
+#pragma unroll
+  for (int k = 0; k < PAIR_REG; k++) ss = fmaf(sum * v[k], sum * v[k], ss);
+  for (int c = threadIdx.x + 256 * PAIR_REG; c < a.W; c += 256) { const float u = sum * value(c); ss = fmaf(u, u, ss); }      // (channels beyond the registers are read again below)
   ss = block_sum_256(ss, s4);
   const float r = sum / sqrtf(ss / (float)a.W + a.in.eps);
-  for (int c = threadIdx.x; c < a.W; c += 256) a.in.out[(size_t)t * a.W + c] = x[c] * r * (1.0f + a.in.w_norm[c]);
+  auto store = [&](int c, float val) {
+    for (int s = 0; s < a.n; s++) x[(size_t)s * a.W + c] = val;
+    out[c] = val * r * (1.0f + a.in.w_norm[c]);
+  };
+#pragma unroll
+  for (int k = 0; k < PAIR_REG; k++) { const int c = threadIdx.x + 256 * k; if (c < a.W) store(c, v[k]); }
+  for (int c = threadIdx.x + 256 * PAIR_REG; c < a.W; c += 256) store(c, value(c));
 }
 
 // ---- the seam.  y_t = the sublayer's output: one row, or the sum of the token's `top` expert rows, plus the shared expert's row.  All streams at once from the old
@@ -173,6 +181,35 @@ __global__ __launch_bounds__(256) void map_difference_kernel(MapDifferenceArgs a
   const float f = a.scale / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
 #pragma unroll
   for (int k = 0; k < GQA_MAX_RPL; k++) { const int c = lane + 64 * k; if (c < a.vdim) a.out[(size_t)p * a.vdim + c] = d[k] * f; }
+}
+
+// ---- the same behind a divided attention: the split records (m, l, acc[vdim]) of both maps of one (token, head) are merged in split order first
+struct MapDifferenceMergeArgs { const float* part; int nsplit; float* out; int heads, vdim; float lambda, eps, scale; };      // part [T][heads][2][nsplit][vdim + 2]
+__global__ __launch_bounds__(256) void map_difference_merge_kernel(MapDifferenceMergeArgs a) {
+  __shared__ float s_f[2][64], s_inv[2], s4[4];
+  const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+  const size_t rs = (size_t)(a.vdim + 2);
+  const float* rec = a.part + ((size_t)t * a.heads + h) * 2 * a.nsplit * rs;
+  if (wv < 2) {      // a wave per map, a lane per record
+    const float* r = rec + (size_t)wv * a.nsplit * rs;
+    const float ms = lane < a.nsplit ? r[(size_t)lane * rs] : -INFINITY;
+    const float M = group_max<64>(ms), f = ms == -INFINITY ? 0.f : expf(ms - M);
+    const float L = group_sum<64>(lane < a.nsplit ? r[(size_t)lane * rs + 1] * f : 0.f);
+    s_f[wv][lane] = f;
+    if (lane == 0) s_inv[wv] = L > 0.f ? 1.0f / L : 0.f;
+  }
+  __syncthreads();
+  const int c = threadIdx.x;      // vdim <= 256
+  float d = 0.f;
+  if (c < a.vdim) {
+    float o[2] = {0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+      for (int s = 0; s < a.nsplit; s++) o[i] = fmaf(rec[((size_t)i * a.nsplit + s) * rs + 2 + c], s_f[i][s], o[i]);
+    d = fmaf(-a.lambda, o[1] * s_inv[1], o[0] * s_inv[0]);
+  }
+  const float f = a.scale / sqrtf(block_sum_256(d * d, s4) / (float)a.vdim + a.eps);
+  if (c < a.vdim) a.out[((size_t)t * a.heads + h) * a.vdim + c] = d * f;
 }
 
 }  // namespace tgx

@@ -515,10 +515,11 @@ struct RouterGroupArgs {
   int E, top, groups, keep;
   float scale;
   int sigmoid_scores, group_top2, normalise;
+  int shared;                // 1: every token has one more choice behind its top: expert E with weight 1 (a shared expert that rides among the routed ones)
 };
 __global__ __launch_bounds__(64) void router_group_kernel(RouterGroupArgs a) {
   __shared__ float s_s[ROUTER_MAX_E], s_c[ROUTER_MAX_E], s_g[ROUTER_MAX_E];
-  const int t = blockIdx.x, lane = threadIdx.x;
+  const int t = blockIdx.x, lane = threadIdx.x, stride = a.top + a.shared;
   const float* z = a.z + (size_t)t * a.ldz;
   if (a.sigmoid_scores) {
     for (int e = lane; e < a.E; e += 64) { s_s[e] = 1.0f / (1.0f + expf(-z[e])); s_c[e] = a.corr ? s_s[e] + a.corr[e] : s_s[e]; }
@@ -564,15 +565,16 @@ __global__ __launch_bounds__(64) void router_group_kernel(RouterGroupArgs a) {
     if (bi < a.E && (bi & 63) == lane) s_c[bi] = -INFINITY;
     if (lane == 0) {
       const int pick = bi < a.E ? bi : 0;
-      a.sel[(size_t)t * a.top + k] = pick;
-      a.selw[(size_t)t * a.top + k] = bi < a.E ? s_s[pick] * a.scale : 0.f;
+      a.sel[(size_t)t * stride + k] = pick;
+      a.selw[(size_t)t * stride + k] = bi < a.E ? s_s[pick] * a.scale : 0.f;
     }
   }
+  if (a.shared && lane == 0) { a.sel[(size_t)t * stride + a.top] = a.E; a.selw[(size_t)t * stride + a.top] = 1.f; }
   if (a.normalise && lane == 0) {      // in choice order
     float sum = 0.f;
-    for (int k = 0; k < a.top; k++) sum += a.selw[(size_t)t * a.top + k];
+    for (int k = 0; k < a.top; k++) sum += a.selw[(size_t)t * stride + k];
     const float inv = a.scale / (sum + 1e-20f * a.scale);
-    for (int k = 0; k < a.top; k++) a.selw[(size_t)t * a.top + k] *= inv;
+    for (int k = 0; k < a.top; k++) a.selw[(size_t)t * stride + k] *= inv;
   }
   if (a.sgw && lane == 0) a.sgw[t] = 1.0f / (1.0f + expf(-z[a.E]));
 }

@@ -70,6 +70,7 @@ struct StackLayerW {
   int w_src = -1;               // the layer whose weights this one uses: every pointer but the caches and states is borrowed
   float *hc = nullptr, *decays = nullptr;
   ebyte *w_b = nullptr, *w_g1 = nullptr, *w_g2 = nullptr;
+  bool shared_slot = false;     // the shared expert's matrices are the last of w_up / w_down (it has the routed ones' size)
   float lambda = 0.f;
   std::vector<std::vector<float>> lam_host;
 };

@@ -196,7 +196,7 @@ int ensure_ws(tgx_ctx* c, int T) {
       (rc = dev_alloc(c, &sm->proj, n * (size_t)sm->max_in)) || (rc = dev_alloc(c, &sm->ql, n * (size_t)sm->max_hr)) || (rc = dev_alloc(c, &sm->lat, n * (size_t)sm->max_hr)) ||
       (rc = dev_alloc(c, &sm->o, n * (size_t)sm->max_hv)) || (rc = dev_alloc(c, &sm->xn, n * W)) || (rc = dev_alloc(c, &sm->lg, n * (size_t)sm->d.vocab))) return rc;
   if (sm->max_top > 0) {
-    const size_t np = n * (size_t)sm->max_top;
+    const size_t np = std::max<size_t>(n * (size_t)sm->max_top, sm->hyper ? GROUPED_FEW_PAIRS : 0);      // (a shared expert that rides among the choices: at most that many pairs)
     if ((rc = dev_alloc(c, &sm->zr, n * (size_t)(sm->max_E + 1))) || (rc = dev_alloc(c, &sm->selw, np)) || (rc = dev_alloc(c, &sm->sel, np)) || (rc = dev_alloc(c, &sm->perm, np)) || (rc = dev_alloc(c, &sm->ptok, np)) ||
         (rc = dev_alloc(c, &sm->yh, np * (size_t)sm->max_ff + n * (size_t)sm->max_sff)) || (rc = dev_alloc(c, &sm->yd, np * W)) ||
         (rc = dev_alloc(c, &sm->tile_e, std::max<size_t>(np / 64, GROUPED_FEW_PAIRS / GROUPED_FEW_ROWS) + (size_t)sm->max_E + 1)) ||
@@ -364,10 +364,26 @@ struct GqaSpec {
   const float* sinks; const float* dist; int dist_len;         // per-head sinks, distance table
   int gate_per_head;
   float out_scale = 1.0f;
-  int maps = 1;                                                // score maps over the same values (heads and kv_heads count every map)
+  int maps = 1;                                                // score maps over the same values (heads and kv_heads count every map); with two, `out` takes the maps'
+  float lambda = 0.f, diff_eps = 0.f, diff_scale = 0.f;        // normed difference (map_difference_kernel) and map_out their own outputs on the way there
+  float* map_out = nullptr;
 };
-int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, int S, int max_keys, int max_count) {
+int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp_, int T, int S, int max_keys, int max_count) {
   StackModel* sm = c->stack;
+  GqaSpec sp = sp_;
+  if (sp.maps == 2) { sp.out = sp_.map_out; sp.ldo = (long long)sp.heads * sp.vdim; }
+  auto merge = [&](const tgx::GqaAttnArgs& mg) {      // the records of a divided attention
+    if (sp.maps != 2) { hipLaunchKernelGGL(tgx::gqa_attn_merge_kernel, dim3(T, sp.heads), dim3(256), 0, c->stream, mg); return; }
+    tgx::MapDifferenceMergeArgs da{};
+    da.part = mg.part; da.nsplit = mg.nsplit; da.out = sp_.out; da.heads = sp.heads / 2; da.vdim = sp.vdim; da.lambda = sp.lambda; da.eps = sp.diff_eps; da.scale = sp.diff_scale;
+    hipLaunchKernelGGL(tgx::map_difference_merge_kernel, dim3(T, da.heads), dim3(256), 0, c->stream, da);
+  };
+  auto finish = [&]() {                               // undivided: the maps' outputs stand in full
+    if (sp.maps != 2) return;
+    tgx::MapDifferenceArgs da{};
+    da.maps = sp.out; da.out = sp_.out; da.pairs = T * (sp.heads / 2); da.vdim = sp.vdim; da.lambda = sp.lambda; da.eps = sp.diff_eps; da.scale = sp.diff_scale;
+    hipLaunchKernelGGL(tgx::map_difference_kernel, dim3((da.pairs + 3) / 4), dim3(256), 0, c->stream, da);
+  };
   const int H = sp.heads, G = sp.kv_heads;
   tgx::GqaAppendArgs ap{};
   ap.proj = sp.proj; ap.ldp = sp.ldp; ap.heads = H; ap.kv_heads = G; ap.maps = sp.maps; ap.dim = sp.dim; ap.vdim = sp.vdim; ap.rot_dims = sp.cs ? sp.rot_dims : 0; ap.rot_pairs = sp.rot_pairs;
@@ -405,9 +421,10 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
       tgx::GqaAttnArgs mg{};
       mg.part = sm->part; mg.nsplit = nsplit; mg.heads = H; mg.vdim = sp.vdim; mg.gate = sp.gate; mg.ldg = sp.ldg; mg.out = sp.out; mg.ldo = sp.ldo;
       mg.gate_per_head = sp.gate_per_head; mg.out_scale = sp.out_scale;
-      hipLaunchKernelGGL(tgx::gqa_attn_merge_kernel, dim3(T, H), dim3(256), 0, c->stream, mg);
+      merge(mg);
     } else {
       launch_gqa_mfma(c, m, ma, dim3(tiles, S * G), false);
+      finish();
     }
     return TGX_OK;
   }
@@ -428,9 +445,10 @@ int run_gqa_core(tgx_ctx* c, const tgx::StepMeta& m, const GqaSpec& sp, int T, i
     if (rc) return rc;
     aa.part = sm->part; aa.nsplit = nsplit;
     TGX_DT_SWITCH(c->dt, (launch_gqa_t<DT, true>(c, m, aa, dim3(T, H, nsplit))))
-    hipLaunchKernelGGL(tgx::gqa_attn_merge_kernel, dim3(T, H), dim3(256), 0, c->stream, aa);
+    merge(aa);
   } else {
     TGX_DT_SWITCH(c->dt, (launch_gqa_t<DT, false>(c, m, aa, dim3(T, H))))
+    finish();
   }
   return TGX_OK;
 }
@@ -1485,12 +1503,9 @@ int run_two_map_attention(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, in
   GqaSpec sp{};
   sp.proj = sm->proj; sp.ldp = ldp; sp.heads = H; sp.kv_heads = G; sp.maps = M; sp.dim = ld.dim; sp.vdim = ld.vdim; sp.rot_dims = ld.rot_dims;
   sp.cs = w.rot >= 0 ? sm->rot[(size_t)w.rot].cs : nullptr; sp.poolK = w.pool; sp.poolV = w.poolV; sp.poolVT = w.poolVT; sp.append = true; sp.scale = ld.scale;
-  sp.out = sm->hs; sp.ldo = (long long)H * ld.vdim;
+  sp.out = sm->o; sp.ldo = vd; sp.map_out = sm->hs; sp.lambda = w.lambda; sp.diff_eps = sm->d.norm_eps; sp.diff_scale = 1.0f - ld.diff;
   int rc = run_gqa_core(c, m, sp, T, S, max_keys, max_count);
   if (rc) return rc;
-  tgx::MapDifferenceArgs da{};
-  da.maps = sm->hs; da.out = sm->o; da.pairs = T * ld.heads; da.vdim = ld.vdim; da.lambda = w.lambda; da.eps = sm->d.norm_eps; da.scale = 1.0f - ld.diff;
-  hipLaunchKernelGGL(tgx::map_difference_kernel, dim3((da.pairs + 3) / 4), dim3(256), 0, c->stream, da);
   sublayer_out(c, sm->o, vd, w.w_o, T);
   return TGX_OK;
 }
@@ -1567,7 +1582,13 @@ void run_channel_delta(tgx_ctx* c, const tgx::StepMeta& m, StackLayerW& w, int T
   sublayer_out(c, sm->o, k.HE, w.w_o, T);
 }
 
-// the feed-forward into yd (one row per token, or `top` rows for experts) and ysh (the shared expert's row)
+// whether the shared expert's products ride among the routed ones': steps of few pairs, where a product is a stream of weights and every launch counts.  (In long portions
+// the shared expert's product takes the wide tiles by itself.)
+bool shared_rides(const tgx_ctx* c, const StackLayerW& w, int T) {
+  const int np = T * (w.d.top + 1);
+  return w.shared_slot && np <= GROUPED_FEW_PAIRS && grouped_tile_rows(c, np, c->stack->d.width, w.d.ff) == GROUPED_FEW_ROWS;
+}
+// the feed-forward into yd (one row per token, or a row per choice for experts) and ysh (the shared expert's row, unless it rides among the choices)
 void run_hyper_ff(tgx_ctx* c, StackLayerW& w, int T) {
   StackModel* sm = c->stack;
   const tgx_layer_desc& ld = w.d;
@@ -1579,11 +1600,11 @@ void run_hyper_ff(tgx_ctx* c, StackLayerW& w, int T) {
     sublayer_out(c, sm->yh, ld.ff, w.w_down, T);
     return;
   }
-  const int E = ld.experts, top = ld.top, np = T * top;
-  g.A = sm->a; g.lda = W; g.B = w.w_router; g.ldb = W; g.C = sm->zr; g.ldc = E; g.M = T; g.N = E; g.K = W; g.scale = 1.f;
+  const int ride = shared_rides(c, w, T) ? 1 : 0, E = ld.experts + ride, top = ld.top + ride, np = T * top;
+  g.A = sm->a; g.lda = W; g.B = w.w_router; g.ldb = W; g.C = sm->zr; g.ldc = ld.experts; g.M = T; g.N = ld.experts; g.K = W; g.scale = 1.f;
   launch_gemm(c, g, tgx::SG_STORE, 1, 0, 0, 64, tgx::DT_F32);
   tgx::RouterGroupArgs ra{};
-  ra.z = sm->zr; ra.ldz = E; ra.sel = sm->sel; ra.selw = sm->selw; ra.E = E; ra.top = top; ra.groups = 1; ra.keep = 1; ra.scale = 1.f; ra.sigmoid_scores = ld.router_fn == 1; ra.normalise = ld.router_norm;
+  ra.z = sm->zr; ra.ldz = ld.experts; ra.sel = sm->sel; ra.selw = sm->selw; ra.E = ld.experts; ra.top = ld.top; ra.shared = ride; ra.groups = 1; ra.keep = 1; ra.scale = 1.f; ra.sigmoid_scores = ld.router_fn == 1; ra.normalise = ld.router_norm;
   hipLaunchKernelGGL(tgx::router_group_kernel, dim3(T), dim3(64), 0, c->stream, ra);
   tgx::MoePlanArgs pa{};
   pa.sel = sm->sel; pa.n_pairs = np; pa.E = E; pa.top = top; pa.tile_m = grouped_tile_rows(c, np, W, ld.ff); pa.E_tiles = E;
@@ -1598,7 +1619,7 @@ void run_hyper_ff(tgx_ctx* c, StackLayerW& w, int T) {
   g.A = sm->yh; g.lda = ld.ff; g.B = w.w_down; g.ldb = ld.ff; g.b_zstride = (long long)W * ld.ff; g.C = sm->yd; g.ldc = W; g.c_rows = sm->perm; g.scale = 1.f;
   g.z_off = sm->moe_off; g.tile_z = sm->tile_e; g.tile_m0 = sm->tile_m0; g.n_tiles = sm->n_tiles; g.M = np; g.N = W; g.K = ld.ff;
   launch_gemm(c, g, tgx::SG_STORE, 1, np, E, pa.tile_m);
-  if (ld.shared_ff > 0) {
+  if (ld.shared_ff > 0 && !ride) {
     float* hsh = sm->yh + (((size_t)np * ld.ff + 3) & ~(size_t)3);
     g = tgx::StackGemmArgs{};
     g.A = sm->a; g.lda = W; g.B = w.ws_up; g.ldb = W; g.C = hsh; g.ldc = ld.shared_ff; g.M = T; g.N = ld.shared_ff; g.K = W; g.scale = 1.f; g.act = tgx::SG_ACT_RELU2;
@@ -1646,7 +1667,8 @@ int run_layers_hyper(tgx_ctx* c, const MetaPtrs& mp, int T, int S, int max_keys,
     hyper_seam(c, w, 0, ff ? hyper_in(sm, w, 1) : next_in, ff ? w.norm2 : next_norm, T, 1, false);
     if (!ff) continue;
     run_hyper_ff(c, w, T);
-    hyper_seam(c, w, 1, next_in, next_norm, T, ld.mlp == TGX_MLP_MOE ? ld.top : 1, ld.mlp == TGX_MLP_MOE && ld.shared_ff > 0);
+    const bool experts = ld.mlp == TGX_MLP_MOE, ride = experts && shared_rides(c, w, T);
+    hyper_seam(c, w, 1, next_in, next_norm, T, experts ? ld.top + ride : 1, experts && ld.shared_ff > 0 && !ride);
   }
   return TGX_OK;
 }
@@ -1732,15 +1754,18 @@ int create_hyper_layers(tgx_ctx* c, const tgx_layer_desc* layers) {
       continue;
     }
     const size_t E = (size_t)l.experts, F = (size_t)l.ff, SF = (size_t)l.shared_ff;
-    if ((rc = dev_alloc(c, &w.w_router, E * W)) || (rc = dev_alloc(c, &w.w_up, E * F * W * es)) || (rc = dev_alloc(c, &w.w_down, E * W * F * es))) return rc;
+    w.shared_slot = SF == F;      // a shared expert of the routed ones' size stands behind them as one more
+    const size_t Es = E + (w.shared_slot ? 1 : 0);
+    if ((rc = dev_alloc(c, &w.w_router, E * W)) || (rc = dev_alloc(c, &w.w_up, Es * F * W * es)) || (rc = dev_alloc(c, &w.w_down, Es * W * F * es))) return rc;
     need(p, {"mlp.router"});
     for (int e = 0; e < l.experts; e++)
       for (const char* s : {".up", ".down"}) sm->missing.insert(p + "mlp.e" + std::to_string(e) + s);
     if (SF > 0) {
-      if ((rc = dev_alloc(c, &w.ws_up, SF * W * es)) || (rc = dev_alloc(c, &w.ws_down, W * SF * es))) return rc;
+      if (w.shared_slot) { w.ws_up = w.w_up + E * F * W * es; w.ws_down = w.w_down + E * W * F * es; }
+      else if ((rc = dev_alloc(c, &w.ws_up, SF * W * es)) || (rc = dev_alloc(c, &w.ws_down, W * SF * es))) return rc;
       need(p, {"mlp.shared.up", "mlp.shared.down"});
     }
-    sm->max_top = std::max(sm->max_top, l.top); sm->max_ff = std::max(sm->max_ff, l.ff); sm->max_E = std::max(sm->max_E, l.experts); sm->max_sff = std::max(sm->max_sff, l.shared_ff);
+    sm->max_top = std::max(sm->max_top, l.top); sm->max_ff = std::max(sm->max_ff, l.ff); sm->max_E = std::max(sm->max_E, (int)Es); sm->max_sff = std::max(sm->max_sff, l.shared_ff);
   }
   sm->max_sff += sm->max_sff > 0 ? 4 : 0;      // (the shared expert's rows start at a multiple of four)
   return TGX_OK;
@@ -2738,6 +2763,7 @@ void stack_destroy(tgx_ctx* c) {
       own.pool = w.pool; own.poolV = w.poolV; own.poolVT = w.poolVT; own.mS = w.mS; own.conv_state = w.conv_state;
       w = own;
     }
+    if (w.shared_slot) w.ws_up = w.ws_down = nullptr;      // (inside w_up / w_down)
     fr(w.hc); fr(w.decays); fr(w.w_b); fr(w.w_g1); fr(w.w_g2);
     fr(w.conv_b); fr(w.d_skip); fr(w.decay2); fr(w.q_norm); fr(w.k_norm); fr(w.dist);
     fr(w.w_o2); fr(w.w_w1); fr(w.w_w2); fr(w.mu); fr(w.w0); fr(w.ubonus); fr(w.conv_w); fr(w.a_log); fr(w.dt_bias); fr(w.shift);
